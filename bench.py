@@ -377,8 +377,24 @@ def kegorax_config(width, layers, vocab=32000):
     return cfg
 
 
+def girolorn_config(width, layers, vocab=32000):
+    """A Girolorn model of real layer sizes: soft-capped attention whose values are its keys (heads of 128, four query
+    heads a key/value head, the whole head rotated with YaRN for four times 4,096 positions, a learned sink a head), every
+    layer with 16 experts of width / 2 (2 a token) and a gated shared expert of the model's width; the last third of the
+    layers runs with the tensors of the first."""
+    again = layers // 3
+    H = width // 128
+    layer = {"type": "attention",
+             "mixer": {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+                       "rot": {"base": 1e6, "dims": 128, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}},
+             "mlp": {"kind": "moe", "expert": {"ff": width // 2, "limit": 7.0}, "router": {"experts": 16, "top": 2},
+                     "shared": {"ff": width, "limit": 7.0}}}
+    return {"architecture": "Girolorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_softcap": 20.0,
+            "layers": [dict(layer) for _ in range(layers - again)] + [dict(layer, weights_of=i) for i in range(again)]}
+
+
 DESIGNS = {"suripel": ("Suripel", suripel_config), "sugosun": ("Sugosun", sugosun_config), "dinasun": ("Dinasun", dinasun_config),
-           "kegorax": ("Kegorax", kegorax_config)}
+           "kegorax": ("Kegorax", kegorax_config), "girolorn": ("Girolorn", girolorn_config)}
 
 
 def llama_like(width, layers, vocab=32000):
@@ -481,7 +497,7 @@ def main():
                     help="also write the command and the JSON line into FILE (markdown)")
     ap.add_argument("--mixed", type=int, default=0, metavar="N",
                     help="also run N requests with prompts of 128..2048 tokens and 128 decoded tokens each through the scheduler")
-    ap.add_argument("--design", default="", choices=["", "suripel", "sugosun", "dinasun", "kegorax"],
+    ap.add_argument("--design", default="", choices=["", "suripel", "sugosun", "dinasun", "kegorax", "girolorn"],
                     help="instead of the serving benchmark: this design at real layer sizes beside the Llama decoder of equal size")
     ap.add_argument("--design-sizes", default="2048,4096", metavar="LIST", help="widths of the --design models")
     ap.add_argument("--design-layers", type=int, default=12, help="layers of the --design models")

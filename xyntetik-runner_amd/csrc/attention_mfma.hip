@@ -66,6 +66,7 @@ struct AttnArgs {
     int window;             // > 0: a row at position p reads the keys from p - window + 1 on
     int chunk;              // > 0: it reads from p - p mod chunk on (its own chunk of positions, counted from 0)
     const float* slopes;    // [H], or null: slopes[h] * (i - j) is taken off the score of query i and key j
+    float cap;              // > 0: a scaled score s counts as cap * tanh(s / cap) (no slopes then)
     const float* sinks;     // [H], or null: the softmax's denominator also holds exp(sinks[h]), an entry without key or value;
                             // it is added where a row's result is finished: by the item that writes the output, or by the merge
 };
@@ -74,6 +75,20 @@ struct AttnArgs {
 __device__ inline float with_sink(const float* sinks, int h, float m, float l) {
     return sinks ? l + __builtin_amdgcn_exp2f(sinks[h] * 1.44269504f - m) : l;
 }
+
+// What the kernels do to a score beside scaling it, each a kernel of its own: nothing, a bias that grows with the
+// distance, a soft cap.
+constexpr int MODE_PLAIN = 0, MODE_SLOPES = 1, MODE_CAP = 2;
+
+// The soft cap in units of log2: C tanh(y) = C - 2 C / (1 + 2^(k s)) for a raw product s, with k = 2 scale log2(e) / cap
+// and C = cap log2(e).  (Large |s|: 2^(k s) is 0 or infinite, and the quotient 2 C or 0.)
+struct SoftCap {
+    float k, C;
+    __device__ inline SoftCap(float scale, float cap) : k(cap > 0.f ? 2.0f * 1.44269504088896340736f * scale / cap : 0.f), C(cap * 1.44269504088896340736f) {}
+    __device__ __forceinline__ float less(float s, float off) const {           // capped score minus off
+        return fmaf(-2.0f * C, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s * k)), C - off);
+    }
+};
 
 __device__ inline uint4 ldg16(const bf16_t* p) { return *reinterpret_cast<const uint4*>(p); }
 __device__ inline bf16x8 as_bf16x8(uint4 v) {
@@ -121,10 +136,10 @@ __device__ inline float max_across_halves(float x) {
 // bias over the tile's keys in units of the scale, (slope_h / scale) * (key - pos), so that the product's sum
 // times the scale is the biased score and the softmax below needs to know nothing of it.  (Far keys make the
 // sum large and coarse, and have no weight; the row's own key, at distance 0, is always among the visible.)
-template <bool SLOPES>
+template <int MODE>
 __device__ __forceinline__ f32x16 score_start(float sb, int kt, int lg, int pos) {
     f32x16 z;
-    if constexpr (SLOPES) {
+    if constexpr (MODE == MODE_SLOPES) {
         const float tb = sb * (float)(kt + 8 * lg - pos);
 #pragma unroll
         for (int e = 0; e < 16; ++e) z[e] = fmaf(sb, (float)(16 * (e >> 3) + (e & 7)), tb);
@@ -289,6 +304,7 @@ struct CtaWave {
     uint32_t vbase[2];          // and of its V^T fragments of channels 0-31, keys 0-15 and 16-31
     bf16x8 qf[KD];
     float c2;
+    SoftCap cap = SoftCap(0.f, 0.f);
     float sb;                   // the row's head's slope over the scale (0 without slopes)
     int pos, lo, lg;
     bool row_ok;
@@ -307,8 +323,8 @@ struct CtaWave {
 // The softmax of a whole tile cut into 18 pieces (the maximum over the lane's scores; the exchange, the
 // reference and the factor; the 16 weights) and dealt to the NS product slots of a step by their cost
 // in cycles of the vector unit (an exponential is a quarter-rate instruction).
-template <int NS> struct CtaPlan {
-    static constexpr int WA = 32, WB = 44, WP = 26, TOTAL = WA + WB + 16 * WP;
+template <int NS, int MODE> struct CtaPlan {
+    static constexpr int WA = 32, WB = MODE == MODE_CAP ? 84 : 44, WP = MODE == MODE_CAP ? 66 : 26, TOTAL = WA + WB + 16 * WP;
     static constexpr int slot_of(int piece) {
         const int before = piece == 0 ? 0 : piece == 1 ? WA : WA + WB + (piece - 2) * WP;
         return before * NS / TOTAL;
@@ -342,11 +358,11 @@ struct CtaFrags {
     }
 };
 
-template <int STAGE, bool SLOPES>
+template <int STAGE, int MODE>
 __device__ __forceinline__ void cta_step_whole(const CtaWave& w, int v, f32x16& s_new, const f32x16& s_cur,
                                                uint4 (&pf_new)[2], const uint4 (&pf_old)[2], f32x16 (&o)[DB], float& m, float& l) {
     constexpr int NS = KD + 2 * DB, AHEAD = 3 < NS ? 3 : NS;
-    const f32x16 start = score_start<SLOPES>(w.sb, w.kbeg + v * 32, w.lg, w.pos);
+    const f32x16 start = score_start<MODE>(w.sb, w.kbeg + v * 32, w.lg, w.pos);
     const CtaFrags f(w, v, std::integral_constant<int, STAGE>{});
     const f32x16& s = s_cur;
     uint4 fr[NS];
@@ -365,7 +381,7 @@ __device__ __forceinline__ void cta_step_whole(const CtaWave& w, int v, f32x16& 
         }
         static_for<0, 18>([&](auto pc) {
             constexpr int piece = decltype(pc)::value;
-            if constexpr (CtaPlan<NS>::slot_of(piece) == k) {
+            if constexpr (CtaPlan<NS, MODE>::slot_of(piece) == k) {
                 if constexpr (piece == 0) {
                     mt = fmaxf(s[0], s[15]);        // the compiler's own instruction reads s first
                     mt = max3(mt, s[1], s[2]);
@@ -373,7 +389,8 @@ __device__ __forceinline__ void cta_step_whole(const CtaWave& w, int v, f32x16& 
                     for (int e = 3; e < 15; e += 2) mt = max3(mt, s[e], s[e + 1]);
                 } else if constexpr (piece == 1) {
                     mt = max_across_halves(mt);
-                    mn = mt * w.c2 > m + MAX_SLACK ? mt * w.c2 : m;
+                    const float mc = MODE == MODE_CAP ? w.cap.less(mt, 0.f) : mt * w.c2;        // (the cap keeps the order)
+                    mn = mc > m + MAX_SLACK ? mc : m;
                     corr = __builtin_amdgcn_exp2f(m - mn);
                     asm volatile("" : "+v"(corr));
                 } else {
@@ -381,7 +398,7 @@ __device__ __forceinline__ void cta_step_whole(const CtaWave& w, int v, f32x16& 
                     // put off all the weights, which nothing in this step reads, to behind the step's
                     // last branch, and the vector unit's work would again follow the matrix unit's)
                     constexpr int e = piece - 2;
-                    const float x = __builtin_amdgcn_exp2f(fmaf(s[e], w.c2, -mn));
+                    const float x = __builtin_amdgcn_exp2f(MODE == MODE_CAP ? w.cap.less(s[e], mn) : fmaf(s[e], w.c2, -mn));
                     rs += x;
                     asm volatile("" : "+v"(rs));
                     if constexpr (e % 2 == 1) {
@@ -405,7 +422,7 @@ __device__ __forceinline__ void cta_step_whole(const CtaWave& w, int v, f32x16& 
     }
 }
 
-template <int STAGE, bool SLOPES>
+template <int STAGE, int MODE>
 __device__ __forceinline__ void cta_step_edge(const CtaWave& w, int v, f32x16& s_new, const f32x16& s_cur,
                                               uint4 (&pf_new)[2], const uint4 (&pf_old)[2], f32x16 (&o)[DB], float& m, float& l) {
     constexpr int NS = KD + 2 * DB;
@@ -414,7 +431,7 @@ __device__ __forceinline__ void cta_step_edge(const CtaWave& w, int v, f32x16& s
     if (w.sees(v)) {
         uint4 kf[KD];
         static_for<0, KD>([&](auto kc) { kf[decltype(kc)::value] = f.template get<decltype(kc)::value>(); });
-        s_new = score_start<SLOPES>(w.sb, w.kbeg + v * 32, w.lg, w.pos);
+        s_new = score_start<MODE>(w.sb, w.kbeg + v * 32, w.lg, w.pos);
 #pragma unroll
         for (int kd = 0; kd < KD; ++kd) s_new = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16x8(kf[kd]), w.qf[kd], s_new, 0, 0, 0);
     }
@@ -446,7 +463,11 @@ __device__ __forceinline__ void cta_step_edge(const CtaWave& w, int v, f32x16& s
     }
     __builtin_amdgcn_sched_barrier(0);
     if (w.sees(v - 1)) {
-        const f32x16& s = s_cur;
+        f32x16 s = s_cur;
+        if constexpr (MODE == MODE_CAP) {
+#pragma unroll
+            for (int e = 0; e < 16; ++e) s[e] = w.cap.less(s[e], 0.f);
+        }
         const int kt = w.kbeg + (v - 1) * 32;
         const bool row_ok = w.row_ok;
         const int pos = w.pos, lo = w.lo, pos_min = w.pos_min, lo_max = w.lo_max;
@@ -460,7 +481,7 @@ __device__ __forceinline__ void cta_step_edge(const CtaWave& w, int v, f32x16& s
 }
 
 // The kernel.  A place of the ring holds K of tile v beside V^T of tile v-2, which is what step v reads.
-template <bool SLOPES>
+template <int MODE>
 __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
     using SH = CtaShape;
     constexpr int SET_THREADS = SH::SET_THREADS, LOADS = SH::LOADS, STAGE = SH::STAGE, SETS = SH::SETS;
@@ -500,7 +521,7 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
         w.pos = start + tok;
         w.lo = a.chunk > 0 ? w.pos - w.pos % a.chunk : (a.window > 0 && w.pos - a.window + 1 > 0) ? w.pos - a.window + 1 : 0;
         w.lg = lg;
-        w.sb = SLOPES ? a.slopes[kvh * G + hg] / a.scale : 0.f;
+        w.sb = MODE == MODE_SLOPES ? a.slopes[kvh * G + hg] / a.scale : 0.f;
         const bf16_t* qp = a.q + ((size_t)(row_ok ? it[5] + tok : it[5]) * a.H + kvh * G + hg) * HD + lg * 8;
 #pragma unroll
         for (int kd = 0; kd < KD; ++kd) w.qf[kd] = as_bf16x8(keep_if(row_ok, ldg16(qp + kd * 16)));
@@ -638,7 +659,8 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
         w.pos_min = __builtin_amdgcn_readfirstlane(pos_min); w.lo_max = __builtin_amdgcn_readfirstlane(lo_max);
         w.pos_max = __builtin_amdgcn_readfirstlane(pos_max); w.lo_min = __builtin_amdgcn_readfirstlane(lo_min);
     }
-    w.c2 = a.scale * 1.44269504088896340736f;
+    w.c2 = MODE == MODE_CAP ? 1.0f : a.scale * 1.44269504088896340736f;       // (capped scores are in units of log2 already)
+    w.cap = SoftCap(a.scale, a.cap);
     w.kbeg = kbeg; w.kend = kend; w.nt = nt; w.seq_len = seq_len;
 
     // Step v of a wave touches place v of the ring only, so the places are filled and waited for two
@@ -676,18 +698,18 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
     int v = 0;
     for (; v < v1; v += 2) {
         STEPS_SYNC(v)
-        cta_step_edge<STAGE, SLOPES>(w, v, s_even, s_odd, pf_odd, pf_even, o, m, l);
-        cta_step_edge<STAGE, SLOPES>(w, v + 1, s_odd, s_even, pf_even, pf_odd, o, m, l);
+        cta_step_edge<STAGE, MODE>(w, v, s_even, s_odd, pf_odd, pf_even, o, m, l);
+        cta_step_edge<STAGE, MODE>(w, v + 1, s_odd, s_even, pf_even, pf_odd, o, m, l);
     }
     for (; v < v2; v += 2) {
         STEPS_SYNC(v)
-        cta_step_whole<STAGE, SLOPES>(w, v, s_even, s_odd, pf_odd, pf_even, o, m, l);
-        cta_step_whole<STAGE, SLOPES>(w, v + 1, s_odd, s_even, pf_even, pf_odd, o, m, l);
+        cta_step_whole<STAGE, MODE>(w, v, s_even, s_odd, pf_odd, pf_even, o, m, l);
+        cta_step_whole<STAGE, MODE>(w, v + 1, s_odd, s_even, pf_even, pf_odd, o, m, l);
     }
     for (; v < n_steps; v += 2) {
         STEPS_SYNC(v)
-        cta_step_edge<STAGE, SLOPES>(w, v, s_even, s_odd, pf_odd, pf_even, o, m, l);
-        cta_step_edge<STAGE, SLOPES>(w, v + 1, s_odd, s_even, pf_even, pf_odd, o, m, l);
+        cta_step_edge<STAGE, MODE>(w, v, s_even, s_odd, pf_odd, pf_even, o, m, l);
+        cta_step_edge<STAGE, MODE>(w, v + 1, s_odd, s_even, pf_even, pf_odd, o, m, l);
     }
 #undef STEPS_SYNC
 #undef STEPS_ISSUE
@@ -770,7 +792,7 @@ constexpr int STREAM_LDS_BYTES = STREAM_RING_BYTES > STREAM_MERGE_BYTES ? STREAM
 static_assert(W_LOADS * (STREAM_STAGES - 1) < 64, "too many copies in flight for the counter");
 static_assert(STREAM_LDS_BYTES <= 160 * 1024, "the rings do not fit into LDS");
 
-template <bool SLOPES>
+template <int MODE>
 __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
     extern __shared__ uint4 lds[];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -795,7 +817,7 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
     const int t = q0 + tok, h = kvh * G + hg;
     const int pos = start + tok;
     const int lo = a.chunk > 0 ? pos - pos % a.chunk : (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
-    const float sb = SLOPES ? a.slopes[h] / a.scale : 0.f;
+    const float sb = MODE == MODE_SLOPES ? a.slopes[h] / a.scale : 0.f;
 
     bf16x8 qf[KD];
     {
@@ -890,7 +912,8 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
 #pragma unroll
         for (int e = 0; e < 16; ++e) o[d][e] = 0.f;
     float m = -INFINITY, l = 0.f;      // m in units of log2
-    const float c2 = a.scale * 1.44269504088896340736f;
+    const float c2 = MODE == MODE_CAP ? 1.0f : a.scale * 1.44269504088896340736f;
+    const SoftCap cap(a.scale, a.cap);
     int pos_min = row_ok ? pos : 0x7fffffff, lo_max = row_ok ? lo : 0;
 #pragma unroll
     for (int o_ = 32; o_ > 0; o_ >>= 1) {
@@ -930,10 +953,14 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
                 }
             }
         }
-        f32x16 s = score_start<SLOPES>(sb, kt, lg, pos);
+        f32x16 s = score_start<MODE>(sb, kt, lg, pos);
 #pragma unroll
         for (int kd = 0; kd < KD; ++kd)
             s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16x8(kf[kd]), qf[kd], s, 0, 0, 0);
+        if constexpr (MODE == MODE_CAP) {
+#pragma unroll
+            for (int e = 0; e < 16; ++e) s[e] = cap.less(s[e], 0.f);
+        }
         float p[16];
         float corr;
         ATTN_SOFTMAX_STEP(kt, kend)
@@ -1072,6 +1099,40 @@ __global__ __launch_bounds__(256) void k_attn_merge(MergeArgs a) {
     }
 }
 
+static int allow_lds(const void* kernel, int bytes, bool& done) {
+    if (done) return XR_OK;
+    hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
+    if (e != hipSuccess) (void)hipGetLastError();     // or the next launch's check would report this refusal
+    XR_REQUIRE(e == hipSuccess, "attention: %d bytes of LDS refused: %s", bytes, hipGetErrorString(e));
+    done = true;
+    return XR_OK;
+}
+
+template <int MODE>
+static int launch_mode(const AttnArgs& a, const int* jobs, int n_jobs, const int* cu_q, hipStream_t stream) {
+    static bool cta_ready = false, stream_ready = false;
+    if (a.n_cta_items > 0) {
+        const int rc = allow_lds((const void*)k_attn_cta<MODE>, CtaShape::LDS_BYTES, cta_ready);
+        if (rc != XR_OK) return rc;
+        k_attn_cta<MODE><<<dim3((unsigned)a.n_cta_items * (unsigned)a.Hk), CtaShape::THREADS, CtaShape::LDS_BYTES, stream>>>(a);
+        XR_CHECK_LAUNCH("attention_cta");
+    }
+    if (a.n_items > 0) {
+        const int rc = allow_lds((const void*)k_attn_stream<MODE>, STREAM_LDS_BYTES, stream_ready);
+        if (rc != XR_OK) return rc;
+        k_attn_stream<MODE><<<dim3((unsigned)a.n_items * (unsigned)a.Hk), 64 * STREAM_WAVES, STREAM_LDS_BYTES, stream>>>(a);
+        XR_CHECK_LAUNCH("attention_stream");
+    }
+    if (n_jobs > 0) {
+        MergeArgs mg;
+        mg.jobs = jobs; mg.cu_q = cu_q; mg.part_o = a.part_o; mg.part_ml = a.part_ml; mg.out = a.out;
+        mg.H = a.H; mg.Hk = a.Hk; mg.sinks = a.sinks;
+        k_attn_merge<<<dim3(n_jobs, a.Hk), 256, 0, stream>>>(mg);
+        XR_CHECK_LAUNCH("attention_merge");
+    }
+    return XR_OK;
+}
+
 extern "C" int xr_attn_head_dim() { return HD; }
 
 extern "C" int xr_attention_mfma(void* out, const void* q, const void* k_cache, const void* v_cache,
@@ -1079,7 +1140,7 @@ extern "C" int xr_attention_mfma(void* out, const void* q, const void* k_cache, 
                                  const int* cu_q,
                                  const int* starts, const int* block_table, int table_stride, float* part_o,
                                  float* part_ml, int H, int Hk, int D, int page_size, float scale, int window,
-                                 int chunk, const float* slopes, const float* sinks, hipStream_t stream) {
+                                 int chunk, const float* slopes, const float* sinks, float cap, hipStream_t stream) {
     XR_REQUIRE(D == HD, "attention: this library is compiled for head size %d, got %d", HD, D);
     XR_REQUIRE(H > 0 && Hk > 0 && H % Hk == 0, "attention: %d query heads are not a multiple of %d key/value heads", H, Hk);
     int shift = ilog2_exact(page_size);
@@ -1098,40 +1159,10 @@ extern "C" int xr_attention_mfma(void* out, const void* q, const void* k_cache, 
     a.page_shift = shift; a.page_mask = page_size - 1; a.page_size = page_size; a.scale = scale; a.window = window; a.chunk = chunk;
     a.slopes = slopes;
     a.sinks = sinks;        // (an item that writes the output adds it; rows of split work are finished by the merge, which adds it there)
+    a.cap = cap;
+    XR_REQUIRE(cap >= 0.f && (cap == 0.f || (scale > 0.f && !slopes)), "attention: a soft cap %g of the scores needs a positive scale and no slopes", (double)cap);
     XR_REQUIRE(!slopes || scale > 0.f, "attention: distance slopes need a positive scale, got %g", (double)scale);
-    if (n_cta_items > 0) {
-        constexpr int smem = CtaShape::LDS_BYTES;
-        static bool attr_set[2] = {false, false};
-        const void* kernel = slopes ? (const void*)k_attn_cta<true> : (const void*)k_attn_cta<false>;
-        if (!attr_set[slopes != nullptr]) {
-            hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
-            if (e != hipSuccess) (void)hipGetLastError();     // or the next launch's check would report this refusal
-            XR_REQUIRE(e == hipSuccess, "attention: %d bytes of LDS refused: %s", smem, hipGetErrorString(e));
-            attr_set[slopes != nullptr] = true;
-        }
-        if (slopes) k_attn_cta<true><<<dim3((unsigned)n_cta_items * (unsigned)Hk), CtaShape::THREADS, smem, stream>>>(a);
-        else k_attn_cta<false><<<dim3((unsigned)n_cta_items * (unsigned)Hk), CtaShape::THREADS, smem, stream>>>(a);
-        XR_CHECK_LAUNCH("attention_cta");
-    }
-    if (n_items > 0) {
-        static bool attr_set[2] = {false, false};
-        const void* kernel = slopes ? (const void*)k_attn_stream<true> : (const void*)k_attn_stream<false>;
-        if (!attr_set[slopes != nullptr]) {
-            hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, STREAM_LDS_BYTES);
-            if (e != hipSuccess) (void)hipGetLastError();
-            XR_REQUIRE(e == hipSuccess, "attention: %d bytes of LDS refused: %s", STREAM_LDS_BYTES, hipGetErrorString(e));
-            attr_set[slopes != nullptr] = true;
-        }
-        if (slopes) k_attn_stream<true><<<dim3((unsigned)n_items * (unsigned)Hk), 64 * STREAM_WAVES, STREAM_LDS_BYTES, stream>>>(a);
-        else k_attn_stream<false><<<dim3((unsigned)n_items * (unsigned)Hk), 64 * STREAM_WAVES, STREAM_LDS_BYTES, stream>>>(a);
-        XR_CHECK_LAUNCH("attention_stream");
-    }
-    if (n_jobs > 0) {
-        MergeArgs mg;
-        mg.jobs = jobs; mg.cu_q = cu_q; mg.part_o = part_o; mg.part_ml = part_ml; mg.out = (bf16_t*)out;
-        mg.H = H; mg.Hk = Hk; mg.sinks = sinks;
-        k_attn_merge<<<dim3(n_jobs, Hk), 256, 0, stream>>>(mg);
-        XR_CHECK_LAUNCH("attention_merge");
-    }
-    return XR_OK;
+    if (cap > 0.f) return launch_mode<MODE_CAP>(a, jobs, n_jobs, cu_q, stream);
+    if (slopes) return launch_mode<MODE_SLOPES>(a, jobs, n_jobs, cu_q, stream);
+    return launch_mode<MODE_PLAIN>(a, jobs, n_jobs, cu_q, stream);
 }

@@ -12,8 +12,9 @@
 // taken off every score: s_t = (q . K_t) * scale - slope_h * (p - t).
 // Other masks: `chunk` > 0: lo = p - p mod chunk (a position reads its own chunk of positions, counted from 0);
 // `keep` > 0: the keys [0, keep) are read as well wherever lo lies.  `sinks` (one number a query head): the
-// softmax's denominator also holds exp(sink_h), an entry that has no key and no value.  Values may have another
+// softmax's denominator also holds exp(sink_h) (of the sink as it is: no scale, no cap), an entry that has no key and no value.  Values may have another
 // size than keys (Dv; cache layout K [page][kv_head][slot][D], V [page][kv_head][Dv][slot]).
+// With `cap` > 0 a scaled score s counts as cap * tanh(s / cap), before a slope's bias.
 #include "common.h"
 
 #define AR_MAX_D 256
@@ -24,7 +25,7 @@ __global__ __launch_bounds__(64) void k_attention_ref(
     const int* __restrict__ positions, const int* __restrict__ req_of_token,
     const int* __restrict__ block_table, int table_stride, int H, int Hk, int D, int Dv, int page_shift,
     int page_mask, int page_size, float scale, int window, int chunk, int keep, const float* __restrict__ slopes,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, float cap) {
     __shared__ float qs[AR_MAX_D];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = positions[t];
@@ -54,7 +55,9 @@ __global__ __launch_bounds__(64) void k_attention_ref(
             const T* kr = kc + (((size_t)page * Hk + kvh) * page_size + off) * D;
             float dot = 0.f;
             for (int d = 0; d < D; ++d) dot = fmaf(qs[d], ld<T>(kr, d), dot);
-            s = dot * scale - slope * (float)(pos - key);
+            s = dot * scale;
+            if (cap > 0.f) s = cap * tanhf(s / cap);
+            s -= slope * (float)(pos - key);
         }
         const float mn = fmaxf(m, wave_max(s));
         const float p = valid ? expf(s - mn) : 0.f;
@@ -97,7 +100,8 @@ extern "C" int xr_attention_ref(void* out, const void* q, const void* k_cache, c
                                 const int* positions, const int* req_of_token, const int* block_table,
                                 int table_stride, int T, int H, int Hk, int D, int Dv, int page_size, float scale,
                                 int window, int chunk, int keep, int dtype, const float* slopes, const float* sinks,
-                                hipStream_t stream) {
+                                float cap, hipStream_t stream) {
+    XR_REQUIRE(cap >= 0.f, "attention: soft cap %g of the scores is negative", (double)cap);
     XR_REQUIRE(T >= 0 && H > 0 && Hk > 0 && D > 0, "attention: bad sizes T=%d H=%d Hk=%d D=%d", T, H, Hk, D);
     XR_REQUIRE(H % Hk == 0, "attention: %d query heads are not a multiple of %d key/value heads", H, Hk);
     XR_REQUIRE(D <= AR_MAX_D && Dv > 0 && Dv <= AR_MAX_D, "attention: head size %d or value size %d exceeds %d", D, Dv, AR_MAX_D);
@@ -110,11 +114,11 @@ extern "C" int xr_attention_ref(void* out, const void* q, const void* k_cache, c
     if (dtype == XR_F32)
         k_attention_ref<float><<<grid, 64, 0, stream>>>((float*)out, (const float*)q, (const float*)k_cache,
                                                         (const float*)v_cache, positions, req_of_token, block_table,
-                                                        table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks);
+                                                        table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks, cap);
     else if (dtype == XR_BF16)
         k_attention_ref<bf16_t><<<grid, 64, 0, stream>>>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k_cache,
                                                          (const bf16_t*)v_cache, positions, req_of_token, block_table,
-                                                         table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks);
+                                                         table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks, cap);
     else { xr_set_error("attention: bad dtype %d", dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("attention_ref");
     return XR_OK;

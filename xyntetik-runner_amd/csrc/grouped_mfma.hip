@@ -377,15 +377,17 @@ __global__ __launch_bounds__(1024) void k_moe_sort(const int* __restrict__ idx, 
     }
 }
 
-// y[t] (+)= sum_j wts[t][j] * yz[t * top + j], in the order of the choice
+// y[t] (+)= sum_j wts[t][j] * yz[t * top + j], in the order of the choice  (+ g_side[t] * y_side[t])
 __global__ void k_moe_combine(float* __restrict__ y, const float* __restrict__ yz, const float* __restrict__ wts, int E, int ld_y,
-                              int top, size_t n, int accumulate) {
+                              int top, size_t n, int accumulate, const float* __restrict__ y_side,
+                              const float* __restrict__ g_side) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
     const size_t t = i / E;
     const int c = (int)(i - t * E);
     float s = 0.f;
     for (int j = 0; j < top; ++j) s += wts[t * top + j] * yz[(t * top + j) * E + c];
+    if (y_side) s = fmaf(g_side[t], y_side[i], s);
     float* o = y + t * ld_y + c;
     *o = accumulate ? *o + s : s;
 }
@@ -393,12 +395,16 @@ __global__ void k_moe_combine(float* __restrict__ y, const float* __restrict__ y
 // The routed experts over many rows: sort, z = relu(up)^2 by expert, yz = down by expert, y = the weighted sum.
 // scratch: ints [A + 3 * (ceil(A / 16) + n) + 1]; z: bf16 [A, F]; yz: float [A, E].
 // Gated experts (`gu` given: float [A, 2F]; w_up [n, 2F, E], an expert's gate rows before its up rows): the first
-// product leaves both branches in 32 bits and the gate's own kernel makes z = silu(gate) * up of them.
+// product leaves both branches in 32 bits and the gate's own kernel makes z of them (`gate`: its code, `param` its number).
+// y_side / g_side: rows [T, E] that enter the sum with one weight a row, or null.
 extern "C" int xr_gate_mul(void* out, const void* gu, int T, int F, int ld_gu, int dtype, int out_dtype, int act, float param,
                            hipStream_t stream);
 extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch, const void* h, const void* w_up,
                                       const void* w_down, const int* idx, const float* wts, int T, int E, int F, int ld_h,
-                                      int ld_y, int n, int top, int accumulate, float* gu, hipStream_t stream) {
+                                      int ld_y, int n, int top, int accumulate, float* gu, int gate, float param, const float* y_side,
+                                      const float* g_side, hipStream_t stream) {
+    XR_REQUIRE(gate >= 0 && gate < XR_ACT_COUNT, "moe_experts_grouped: unknown gate %d", gate);
+    XR_REQUIRE(!y_side == !g_side, "moe_experts_grouped: rows beside the experts come with a weight a row");
     XR_REQUIRE(T >= 0 && E > 0 && F > 0 && ld_h >= E && ld_y >= E, "moe_experts_grouped: bad sizes T=%d E=%d F=%d", T, E, F);
     XR_REQUIRE(n >= 1 && n <= SORT_MAX_EXPERTS && top >= 1 && top <= n, "moe_experts_grouped: %d experts (at most %d), %d chosen", n,
                SORT_MAX_EXPERTS, top);
@@ -427,7 +433,7 @@ extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch
     g.N = Fu; g.K = E; g.out_bf16 = gu ? 0 : 1; g.act = gu ? GM_ACT_NONE : GM_ACT_RELU2; g.gather_div = top;
     launch_grouped(g, max_tiles, bm, stream);
     if (gu) {
-        const int rc = xr_gate_mul(z, gu, A, F, 2 * F, XR_F32, XR_BF16, XR_ACT_SILU, 0.f, stream);
+        const int rc = xr_gate_mul(z, gu, A, F, 2 * F, XR_F32, XR_BF16, gate, param, stream);
         if (rc != XR_OK) return rc;
     }
     // down: rows of z by choice, results by choice
@@ -435,7 +441,7 @@ extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch
     g.N = E; g.K = F; g.out_bf16 = 0; g.act = GM_ACT_NONE; g.gather_div = 1;
     launch_grouped(g, max_tiles, bm, stream);
     const size_t cnt = (size_t)T * E;
-    k_moe_combine<<<(unsigned)((cnt + 255) / 256), 256, 0, stream>>>(y, yz, wts, E, ld_y, top, cnt, accumulate);
+    k_moe_combine<<<(unsigned)((cnt + 255) / 256), 256, 0, stream>>>(y, yz, wts, E, ld_y, top, cnt, accumulate, y_side, g_side);
     XR_CHECK_LAUNCH("moe_experts_grouped");
     return XR_OK;
 }

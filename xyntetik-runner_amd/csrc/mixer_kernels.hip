@@ -10,6 +10,7 @@
 //                    the row with a weight of its own a side; and, if asked, the RMS norm of the updated row times
 //                    a weight (the norm that the next sublayer reads through) in the same pass.
 // k_add_rows:        x[t] += s y[t] + v, a vector added to every row (y absent: the vector alone).
+// k_softcap:         x <- cap tanh(x / cap) in place on 32-bit rows.
 // k_attn_extra_partial: for the matrix-core attention kernels, which take a window's (or a chunk's) keys: what else
 //                    enters the same softmax, as a partial result of its own that their merge adds: a sink (a score
 //                    without key or value, one a head) and the first `keep` keys of the request where the
@@ -151,7 +152,14 @@ struct ExtraArgs {
     int window, chunk, keep;
     const float* sinks;     // [H] or null
     const float* slopes;    // [H] or null
+    float cap;              // > 0: a scaled score s counts as cap * tanh(s / cap)
 };
+
+__device__ inline float extra_score(const ExtraArgs& a, float dot, float slope, int pos, int key) {
+    float s = dot * a.scale;
+    if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
+    return s - slope * (float)(pos - key);
+}
 
 __device__ inline int mask_lo(int pos, int window, int chunk) {
     if (chunk > 0) return pos - pos % chunk;
@@ -194,7 +202,7 @@ __global__ __launch_bounds__(256) void k_attn_extra_partial(float* __restrict__ 
         const T* kr = kc + (((size_t)page * a.Hk + kvh) * a.page_size + off) * a.D;
         float dot = 0.f;
         for (int d = lane; d < a.D; d += 64) dot = fmaf(qs[wave][d], ld<T>(kr, d), dot);
-        const float s = wave_sum(dot) * a.scale - slope * (float)(pos - j);
+        const float s = extra_score(a, wave_sum(dot), slope, pos, j);
         const float mn = fmaxf(m, s);
         const float p = expf(s - mn);
         const float corr = m == -INFINITY ? 0.f : expf(m - mn);
@@ -215,7 +223,7 @@ __global__ __launch_bounds__(256) void k_attn_extra_partial(float* __restrict__ 
             const T* kr = kc + (((size_t)bt[key >> a.page_shift] * a.Hk + kvh) * a.page_size + (key & a.page_mask)) * a.D;
             float dot = 0.f;
             for (int d = 0; d < a.D; ++d) dot = fmaf(qs[wave][d], ld<T>(kr, d), dot);
-            s = dot * a.scale - slope * (float)(pos - key);
+            s = extra_score(a, dot, slope, pos, key);
         }
         const float mn = fmaxf(m, wave_max(s));
         const float p = valid ? expf(s - mn) : 0.f;
@@ -252,7 +260,8 @@ __global__ __launch_bounds__(256) void k_attn_extra_partial(float* __restrict__ 
 extern "C" int xr_attn_extra_partial(float* part_o, float* part_ml, const void* q, const void* k_cache, const void* v_cache,
                                      const int* extras, int n_extras, const int* block_table, int table_stride, int H,
                                      int Hk, int D, int page_size, float scale, int window, int chunk, int keep,
-                                     const float* sinks, const float* slopes, int dtype, hipStream_t stream) {
+                                     const float* sinks, const float* slopes, float cap, int dtype, hipStream_t stream) {
+    XR_REQUIRE(cap >= 0.f, "attention extras: soft cap %g of the scores is negative", (double)cap);
     XR_REQUIRE(n_extras >= 0 && H > 0 && Hk > 0 && H % Hk == 0, "attention extras: %d query heads over %d key/value heads", H, Hk);
     XR_REQUIRE(D > 0 && D <= MK_MAX_D, "attention extras: head size %d (1 to %d)", D, MK_MAX_D);
     const int shift = ilog2_exact(page_size);
@@ -260,7 +269,7 @@ extern "C" int xr_attn_extra_partial(float* part_o, float* part_ml, const void* 
     XR_REQUIRE(window >= 0 && chunk >= 0 && keep >= 0, "attention extras: window %d, chunk %d, kept %d", window, chunk, keep);
     XR_REQUIRE(part_o && part_ml && q && extras && (keep == 0 || (k_cache && v_cache && block_table)), "attention extras: an operand is missing");
     if (n_extras == 0) return XR_OK;
-    ExtraArgs a{block_table, table_stride, H, Hk, D, shift, page_size - 1, page_size, scale, window, chunk, keep, sinks, slopes};
+    ExtraArgs a{block_table, table_stride, H, Hk, D, shift, page_size - 1, page_size, scale, window, chunk, keep, sinks, slopes, cap};
     dim3 grid((unsigned)n_extras * 8, Hk);
     if (dtype == XR_F32)
         k_attn_extra_partial<float><<<grid, 256, 0, stream>>>(part_o, part_ml, (const float*)q, (const float*)k_cache, (const float*)v_cache, extras, a);
@@ -268,5 +277,24 @@ extern "C" int xr_attn_extra_partial(float* part_o, float* part_ml, const void* 
         k_attn_extra_partial<bf16_t><<<grid, 256, 0, stream>>>(part_o, part_ml, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, extras, a);
     else { xr_set_error("attention extras: bad dtype %d", dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("attn_extra_partial");
+    return XR_OK;
+}
+
+// x <- cap * tanh(x / cap) in place on 32-bit rows
+__global__ void k_softcap(float* __restrict__ x, int W, int ld, size_t n, float cap, float inv) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n) return;
+    const size_t t = i / W;
+    float* p = x + t * ld + (i - t * W);
+    *p = cap * tanhf(*p * inv);
+}
+
+extern "C" int xr_softcap(float* x, int R, int W, int ld, float cap, hipStream_t stream) {
+    XR_REQUIRE(R >= 0 && W > 0 && ld >= W, "softcap: bad sizes R=%d W=%d ld=%d", R, W, ld);
+    XR_REQUIRE(cap > 0.f, "softcap: cap %g must be positive", (double)cap);
+    const size_t n = (size_t)R * W;
+    if (n == 0) return XR_OK;
+    k_softcap<<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(x, W, ld, n, cap, 1.0f / cap);
+    XR_CHECK_LAUNCH("softcap");
     return XR_OK;
 }

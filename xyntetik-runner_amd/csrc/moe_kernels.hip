@@ -6,12 +6,15 @@
 // sigmoid(logit), every expert for itself, instead of a softmax; the experts form `groups` equal groups of
 // neighbours, a group's score is the sum of its two largest score + correction, and only experts of the `keep`
 // groups that score highest can be chosen (ties: the lower group); the weights are the chosen scores times a
-// given number instead of their share of their sum.
+// given number instead of their share of their sum; or the choice is by logit + correction (the router's bias) and
+// the weights are the softmax of these over the chosen experts.  `side` given: column n of a token's logits is no
+// expert's, and its sigmoid goes to side[t].
 // k_moe_up / k_moe_down: the experts' two products token by token, a wave an output column, the
 // weights of the chosen experts streamed: what a few decoded tokens need.  Expert:
-// down(act(up h)), act = relu squared, or gated: down(silu(gate h) * (up h)) with the gate's rows before
-// the up rows in one matrix [2F, E].  The down product adds a token's experts up in the order
-// of its choice and writes (or adds to) 32-bit rows.
+// down(act(up h)), act = relu squared, or gated: down(value(gate h, up h)) with a gate of common.h (SiLU: silu(g) u)
+// and the gate's rows before the up rows in one matrix [2F, E].  The down product adds a token's experts up in the order
+// of its choice, then rows that come from elsewhere times the token's weight for them (a shared expert's), and writes
+// (or adds to) 32-bit rows.
 // k_moe_table_route: the choice without a router, a row of a table [vocab, top] by the token's id, every
 // chosen expert with the same weight.
 #include "common.h"
@@ -19,15 +22,60 @@
 #define MOE_MAX_EXPERTS 1024
 #define MOE_MAX_TOP 64      // lane j of the routing wave keeps the j-th choice
 
-__global__ __launch_bounds__(64) void k_moe_route(int* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ logits,
-                                                  const float* __restrict__ correction, int ld, int n, int top, int sigmoid,
+#define MOE_SCORES_SOFTMAX 0
+#define MOE_SCORES_SIGMOID 1
+#define MOE_SCORES_LOGITS 2
+
+__global__ __launch_bounds__(64) void k_moe_route(int* __restrict__ idx, float* __restrict__ wts, float* __restrict__ side,
+                                                  const float* __restrict__ logits,
+                                                  const float* __restrict__ correction, int ld, int n, int top, int scores,
                                                   int groups, int keep, float weight_scale) {
     __shared__ float z[MOE_MAX_EXPERTS];
     __shared__ float gsc[MOE_MAX_EXPERTS];          // a group's score; then 1 if its experts can be chosen, else 0
     const int t = blockIdx.x, lane = threadIdx.x;
+    if (side && lane == 0) side[t] = 1.0f / (1.0f + expf(-logits[(size_t)t * ld + n]));
+    if (scores == MOE_SCORES_LOGITS) {
+        // `top` passes of: the largest logit + bias not yet taken, the lower index on a tie (no number counts as the
+        // smallest, as below); then a softmax over the lanes that hold a choice
+        for (int e = lane; e < n; e += 64) {
+            const float c = logits[(size_t)t * ld + e] + correction[e];
+            z[e] = c == c ? c : -INFINITY;
+            gsc[e] = 0.f;           // 1: taken
+        }
+        __syncthreads();
+        int mine = 0;
+        float mine_z = -INFINITY;
+        for (int j = 0; j < top; ++j) {
+            float best = -INFINITY;
+            int at = n;
+            for (int e = lane; e < n; e += 64) {
+                if (gsc[e] != 0.f) continue;
+                if (at == n || z[e] > best) { best = z[e]; at = e; }
+            }
+#pragma unroll
+            for (int o = 32; o > 0; o >>= 1) {
+                const float ob = __shfl_xor(best, o, 64);
+                const int oa = __shfl_xor(at, o, 64);
+                if (oa < n && (at == n || ob > best || (ob == best && oa < at))) { best = ob; at = oa; }
+            }
+            at = at < n ? at : 0;
+            if (lane == j) { mine = at; mine_z = best; }
+            __syncthreads();
+            if (lane == 0) gsc[at] = 1.f;
+            __syncthreads();
+        }
+        const float m = wave_max(mine_z);
+        const float e = (lane < top && m > -INFINITY) ? expf(mine_z - m) : (lane < top ? 1.f : 0.f);
+        const float total = wave_sum(e);
+        if (lane < top) {
+            idx[(size_t)t * top + lane] = mine;
+            wts[(size_t)t * top + lane] = e / total;
+        }
+        return;
+    }
     for (int e = lane; e < n; e += 64) z[e] = logits[(size_t)t * ld + e];
     __syncthreads();
-    if (sigmoid) {
+    if (scores == MOE_SCORES_SIGMOID) {
         for (int e = lane; e < n; e += 64) z[e] = 1.0f / (1.0f + expf(-z[e]));      // the scores
     } else {
         float m = -INFINITY;
@@ -105,16 +153,18 @@ __global__ __launch_bounds__(64) void k_moe_route(int* __restrict__ idx, float* 
     }
 }
 
-extern "C" int xr_moe_route(int* idx, float* wts, const float* logits, const float* correction, int T, int ld, int n, int top,
-                            int sigmoid, int groups, int keep, float weight_scale, hipStream_t stream) {
-    XR_REQUIRE(T >= 0 && ld >= n, "moe_route: bad sizes T=%d ld=%d", T, ld);
+extern "C" int xr_moe_route(int* idx, float* wts, float* side, const float* logits, const float* correction, int T, int ld, int n,
+                            int top, int scores, int groups, int keep, float weight_scale, hipStream_t stream) {
+    XR_REQUIRE(T >= 0 && ld >= n + (side ? 1 : 0), "moe_route: bad sizes T=%d ld=%d", T, ld);
+    XR_REQUIRE(scores >= MOE_SCORES_SOFTMAX && scores <= MOE_SCORES_LOGITS, "moe_route: unknown scores %d", scores);
+    XR_REQUIRE(scores != MOE_SCORES_LOGITS || (groups == 1 && weight_scale == 0.f), "moe_route: a choice by the logits has no groups and no weight scale");
     XR_REQUIRE(n >= 1 && n <= MOE_MAX_EXPERTS && top >= 1 && top <= n && top <= MOE_MAX_TOP,
                "moe_route: %d experts (at most %d), %d chosen (at most %d)", n, MOE_MAX_EXPERTS, top, MOE_MAX_TOP);
     XR_REQUIRE(groups >= 1 && n % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (n / groups),
                "moe_route: %d experts in %d groups of which %d are kept cannot give %d choices", n, groups, keep, top);
     XR_REQUIRE(weight_scale >= 0.f, "moe_route: weight scale %g (0: the chosen scores' shares of their sum)", (double)weight_scale);
     if (T == 0) return XR_OK;
-    k_moe_route<<<T, 64, 0, stream>>>(idx, wts, logits, correction, ld, n, top, sigmoid, groups, keep, weight_scale);
+    k_moe_route<<<T, 64, 0, stream>>>(idx, wts, side, logits, correction, ld, n, top, scores, groups, keep, weight_scale);
     XR_CHECK_LAUNCH("moe_route");
     return XR_OK;
 }
@@ -173,14 +223,14 @@ template <> __device__ inline float wave_dot<bf16_t>(const bf16_t* __restrict__ 
     return wave_sum(acc);
 }
 
-// z[t * top + j][f] = relu(W_up[e][f] . h[t])^2 for e = idx[t][j]; `gated`: silu(W_up[e][f] . h[t]) * (W_up[e][F + f] . h[t]).
+// z[t * top + j][f] = relu(W_up[e][f] . h[t])^2 for e = idx[t][j]; `gated`: the gate's value of W_up[e][f] . h[t] and W_up[e][F + f] . h[t].
 // Grid (T * top, ceil(F / 4)); a wave a column.
 #define MOE_ACT_RELU2 0
-#define MOE_ACT_SWIGLU 1
+#define MOE_ACT_GATED 1
 template <typename TW>
 __global__ __launch_bounds__(256) void k_moe_up(TW* __restrict__ z, const TW* __restrict__ h, const TW* __restrict__ w_up,
                                                 const int* __restrict__ idx, int E, int F, int ld_h, int top, int n, int vec,
-                                                int gated) {
+                                                int gated, int gate, float param) {
     const int a = blockIdx.x, f = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (f >= F) return;
     const int t = a / top, e = min(max(idx[a], 0), n - 1);
@@ -189,7 +239,7 @@ __global__ __launch_bounds__(256) void k_moe_up(TW* __restrict__ z, const TW* __
     const float acc = wave_dot<TW>(w, row, E, lane, vec != 0);
     if (gated) {
         const float up = wave_dot<TW>(w + (size_t)F * E, row, E, lane, vec != 0);
-        if (lane == 0) st<TW>(z, (size_t)a * F + f, gate_value<false>(XR_ACT_SILU, 0.f, acc, up));
+        if (lane == 0) st<TW>(z, (size_t)a * F + f, gate_value<false>(gate, param, acc, up));
         return;
     }
     if (lane == 0) {
@@ -198,11 +248,12 @@ __global__ __launch_bounds__(256) void k_moe_up(TW* __restrict__ z, const TW* __
     }
 }
 
-// y[t][c] (+)= sum_j wts[t][j] * (W_down[e_j][c] . z[t * top + j]).  Grid (T, ceil(E / 4)); a wave a column.
+// y[t][c] (+)= sum_j wts[t][j] * (W_down[e_j][c] . z[t * top + j])  (+ g_side[t] * y_side[t][c]).  Grid (T, ceil(E / 4)); a wave a column.
 template <typename TW>
 __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const TW* __restrict__ z, const TW* __restrict__ w_down,
                                                   const int* __restrict__ idx, const float* __restrict__ wts, int E, int F,
-                                                  int ld_y, int top, int n, int accumulate, int vec) {
+                                                  int ld_y, int top, int n, int accumulate, int vec,
+                                                  const float* __restrict__ y_side, const float* __restrict__ g_side) {
     const int t = blockIdx.x, c = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (c >= E) return;
     float sum = 0.f;
@@ -213,6 +264,7 @@ __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const T
         sum += wts[(size_t)t * top + j] * wave_dot<TW>(w, zr, F, lane, vec != 0);
     }
     if (lane == 0) {
+        if (y_side) sum = fmaf(g_side[t], y_side[(size_t)t * E + c], sum);
         float* o = y + (size_t)t * ld_y + c;
         *o = accumulate ? *o + sum : sum;
     }
@@ -220,9 +272,12 @@ __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const T
 
 extern "C" int xr_moe_experts(float* y, void* z, const void* h, const void* w_up, const void* w_down, const int* idx,
                               const float* wts, int T, int E, int F, int ld_h, int ld_y, int n, int top, int accumulate,
-                              int dtype, int act, hipStream_t stream) {
-    XR_REQUIRE(act == MOE_ACT_RELU2 || act == MOE_ACT_SWIGLU, "moe_experts: activation %d (0 = relu squared, 1 = SiLU-gated)", act);
-    const int gated = act == MOE_ACT_SWIGLU;
+                              int dtype, int act, int gate, float param, const float* y_side, const float* g_side,
+                              hipStream_t stream) {
+    XR_REQUIRE(act == MOE_ACT_RELU2 || act == MOE_ACT_GATED, "moe_experts: activation %d (0 = relu squared, 1 = gated)", act);
+    XR_REQUIRE(gate >= 0 && gate < XR_ACT_COUNT, "moe_experts: unknown gate %d", gate);
+    XR_REQUIRE(!y_side == !g_side, "moe_experts: rows beside the experts come with a weight a row");
+    const int gated = act == MOE_ACT_GATED;
     XR_REQUIRE(T >= 0 && E > 0 && F > 0 && ld_h >= E && ld_y >= E, "moe_experts: bad sizes T=%d E=%d F=%d", T, E, F);
     XR_REQUIRE(n >= 1 && top >= 1 && top <= n && top <= MOE_MAX_TOP, "moe_experts: %d experts, %d chosen", n, top);
     XR_REQUIRE((long long)T * top <= 0x7fffffffLL, "moe_experts: too many rows");
@@ -232,11 +287,11 @@ extern "C" int xr_moe_experts(float* y, void* z, const void* h, const void* w_up
     const bool al = ((uintptr_t)h % 16) == 0 && ((uintptr_t)w_up % 16) == 0 && ((uintptr_t)w_down % 16) == 0 && ((uintptr_t)z % 16) == 0;
     const int vu = al && E % per16 == 0 && ld_h % per16 == 0, vd = al && F % per16 == 0;
     if (dtype == XR_F32) {
-        k_moe_up<float><<<gu, 256, 0, stream>>>((float*)z, (const float*)h, (const float*)w_up, idx, E, F, ld_h, top, n, vu, gated);
-        k_moe_down<float><<<gd, 256, 0, stream>>>(y, (const float*)z, (const float*)w_down, idx, wts, E, F, ld_y, top, n, accumulate, vd);
+        k_moe_up<float><<<gu, 256, 0, stream>>>((float*)z, (const float*)h, (const float*)w_up, idx, E, F, ld_h, top, n, vu, gated, gate, param);
+        k_moe_down<float><<<gd, 256, 0, stream>>>(y, (const float*)z, (const float*)w_down, idx, wts, E, F, ld_y, top, n, accumulate, vd, y_side, g_side);
     } else if (dtype == XR_BF16) {
-        k_moe_up<bf16_t><<<gu, 256, 0, stream>>>((bf16_t*)z, (const bf16_t*)h, (const bf16_t*)w_up, idx, E, F, ld_h, top, n, vu, gated);
-        k_moe_down<bf16_t><<<gd, 256, 0, stream>>>(y, (const bf16_t*)z, (const bf16_t*)w_down, idx, wts, E, F, ld_y, top, n, accumulate, vd);
+        k_moe_up<bf16_t><<<gu, 256, 0, stream>>>((bf16_t*)z, (const bf16_t*)h, (const bf16_t*)w_up, idx, E, F, ld_h, top, n, vu, gated, gate, param);
+        k_moe_down<bf16_t><<<gd, 256, 0, stream>>>(y, (const bf16_t*)z, (const bf16_t*)w_down, idx, wts, E, F, ld_y, top, n, accumulate, vd, y_side, g_side);
     } else { xr_set_error("moe_experts: bad dtype %d", dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("moe_experts");
     return XR_OK;

@@ -67,8 +67,9 @@ _PROTOS = {
     "xr_gemm_bf16": [_p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p, _sz, _p, _p, _p],
     "xr_pack_weight": [_p, _p, _i, _i, _p],
     "xr_rope_table": [_p, _p, _p, _i, _i, _f, _p],
-    "xr_attention_ref": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p, _p, _p],
-    "xr_attn_extra_partial": [_p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p, _p, _i, _p],
+    "xr_attention_ref": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p, _p, _f, _p],
+    "xr_attn_extra_partial": [_p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p, _p, _f, _i, _p],
+    "xr_softcap": [_p, _i, _i, _i, _f, _p],
     "xr_decay_prepare": [_p, _i, _i, _i, _i, _i, _f, _p, _p, _p],
     "xr_head_gate": [_p, _p, _i, _i, _i, _i, _i, _p],
     "xr_pair_combine": [_p, _p, _p, _p, _p, _f, _f, _f, _i, _i, _i, _i, _p, _p, _f, _i, _p],
@@ -90,10 +91,10 @@ _PROTOS = {
     "xr_streams_sum": [_p, _p, _i, _i, _i, _p],
     "xr_streams_step": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _f, _i, _p],
     "xr_latent_prepare": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p],
-    "xr_moe_route": [_p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _p],
-    "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p, _p],
+    "xr_moe_route": [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _p],
+    "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p, _i, _f, _p, _p, _p],
     "xr_heads_gemm_bf16": [_p, _p, _p, _i, _i, _i, _i, _i, C.c_longlong, _i, C.c_longlong, _i, _p],
-    "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p],
+    "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p],
     "xr_delta_prepare": [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _p],
     "xr_linear_recurrence": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p, _p, _i, _f, _f, _p],
     "xr_qkv_store": [_p, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p],
@@ -105,7 +106,10 @@ _PROTOS = {
 CONV_ACTIVATIONS = {None: 0, "none": 0, "silu": 1}      # XR_CONV_* of sequence_kernels.hip
 RECURRENCES = {"retention": 0, "delta": 1, "wkv": 2, "gla": 3, "delta_channel": 4}    # XR_REC_* of recurrent_kernels.hip
 ROW_ACTIVATIONS = {"silu": 1, "tanh": 2}                # what act_rows_ applies in place
-EXPERT_ACTIVATIONS = {"relu2": 0, "swiglu": 1}          # MOE_ACT_* of moe_kernels.hip
+ROUTE_SCORES = {"softmax": 0, "sigmoid": 1, "logits": 2}    # MOE_SCORES_* of moe_kernels.hip
+# what an expert applies between its products: (MOE_ACT_* of moe_kernels.hip, the gate's code)
+EXPERT_ACTIVATIONS = {"relu2": (0, 0), "swiglu": (1, GATE_ACTIVATIONS["silu"]),
+                      **{name: (1, GATE_ACTIVATIONS[name]) for name in ("clamped_swish", "gelu_tanh")}}
 
 
 def _ptr(t: Optional[torch.Tensor]) -> Optional[int]:
@@ -609,16 +613,17 @@ class Ops:
     def attention(self, q, k_cache, v_cache, ctx, group: int, H: int, Hk: int, D: int, page_size: int,
                   scale: float, window: Optional[int] = None, slopes: Optional[torch.Tensor] = None,
                   chunk: Optional[int] = None, keep_first: int = 0, sinks: Optional[torch.Tensor] = None,
-                  v_head_dim: Optional[int] = None) -> torch.Tensor:
+                  v_head_dim: Optional[int] = None, softcap: float = 0.0) -> torch.Tensor:
         """Causal attention of every token of the step over its request's cached keys and values.
         ``slopes`` (32-bit ``[H]``): ``slopes[h] * (i - j)`` is taken off the score of query i and key j.
         ``window``: a position reads the last ``window`` keys; ``chunk``: it reads the keys of its own chunk of
         ``chunk`` positions, counted from 0; ``keep_first``: the first so many keys are read whatever the window.
         ``sinks`` (32-bit ``[H]``): the softmax's denominator also holds ``exp(sinks[h])``, an entry without key
         or value.  ``v_head_dim``: the size of a value where it is not the keys' (``[T, H * v_head_dim]`` comes back).
+        ``softcap`` c > 0: a scaled score s counts as ``c tanh(s / c)`` (a slope's bias is taken off that; the sink is not capped).
 
         bfloat16 runs on the matrix cores (head sizes in steps of 16 up to 256, pages of at least
-        16 positions); float32, and what the MFMA kernel does not take, runs the 32-bit kernel.
+        16 positions, a cap or slopes); float32, and what the MFMA kernel does not take, runs the 32-bit kernel.
         """
         positions, req_of_token, block_table = ctx.positions, ctx.req_of_token, ctx.block_table(group)
         self._dev(q, k_cache, v_cache, positions, req_of_token, block_table)
@@ -637,7 +642,8 @@ class Ops:
                     raise KernelError(f"attention: the {name} must be float32 [{H}]")
         if chunk and window:
             raise KernelError("attention: a layer reads a window or its chunk, not both")
-        if (self.use_mfma and q.dtype == torch.bfloat16 and D == Dv and D % 16 == 0 and 16 <= D <= 256 and page_size >= 16):
+        if (self.use_mfma and q.dtype == torch.bfloat16 and D == Dv and D % 16 == 0 and 16 <= D <= 256 and page_size >= 16
+                and not (softcap and slopes is not None)):
             # The first keys that a window has passed enter the same softmax as a partial result of its own, which
             # the kernels' merge adds to the key ranges' (with the sink, if there is one); a sink alone is added by
             # the kernels themselves where they finish a row.
@@ -655,19 +661,27 @@ class Ops:
                     part_o.data_ptr(), part_ml.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                     plan.extras.data_ptr(), plan.n_extras, block_table.data_ptr(), block_table.stride(0), H, Hk, D, page_size,
                     float(scale), int(window or 0), int(chunk or 0), int(keep_first), _ptr(sinks), _ptr(slopes),
-                    dtype_code(q.dtype), _stream()))
+                    float(softcap), dtype_code(q.dtype), _stream()))
             lib.check(lib.xr_attention_mfma(
                 out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), plan.items.data_ptr(),
                 plan.n_items, plan.n_cta_items, _ptr(plan.jobs), plan.n_jobs, ctx.cu_q.data_ptr(),
                 ctx.starts_dev.data_ptr(), block_table.data_ptr(), block_table.stride(0), _ptr(part_o), _ptr(part_ml), H, Hk, D, page_size,
-                float(scale), int(window or 0), int(chunk or 0), _ptr(slopes), None if extra else _ptr(sinks), _stream()))
+                float(scale), int(window or 0), int(chunk or 0), _ptr(slopes), None if extra else _ptr(sinks),
+                float(softcap), _stream()))
             return out
         self.lib.check(self.lib.xr_attention_ref(
             out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), positions.data_ptr(),
             req_of_token.data_ptr(), block_table.data_ptr(), block_table.stride(0), T, H, Hk, D, Dv, page_size,
             float(scale), int(window or 0), int(chunk or 0), int(keep_first), dtype_code(q.dtype), _ptr(slopes),
-            _ptr(sinks), _stream()))
+            _ptr(sinks), float(softcap), _stream()))
         return out
+
+    def softcap_(self, x: torch.Tensor, cap: float) -> None:
+        """``x <- cap tanh(x / cap)`` in place on a 32-bit view ``[rows, width]`` with unit column stride."""
+        self._dev(x)
+        if x.dtype != torch.float32 or x.dim() != 2 or x.stride(1) != 1:
+            raise KernelError("softcap_: x must be a float32 view [rows, width] with unit column stride")
+        self.lib.check(self.lib.xr_softcap(x.data_ptr(), x.shape[0], x.shape[1], x.stride(0), float(cap), _stream()))
 
     def head_gate_(self, o: torch.Tensor, g: torch.Tensor, H: int, Dv: int) -> None:
         """``o[t, h, :] *= sigmoid(g[t, h])`` in place: ``o [T, H * Dv]`` contiguous, ``g`` a 32-bit view ``[T, H]``."""
@@ -741,7 +755,7 @@ class Ops:
             unit = f"attn_d{D}"
             path = _build.find_built(unit) or _build.build_unit(unit)
             lib = _Lib(path, {"xr_attention_mfma": [_p, _p, _p, _p, _p, _i, _i, _p, _i, _p, _p, _p, _i, _p, _p,
-                                                    _i, _i, _i, _i, _f, _i, _i, _p, _p, _p]})
+                                                    _i, _i, _i, _i, _f, _i, _i, _p, _p, _f, _p]})
             self._attn_libs[D] = lib
         return lib
 
@@ -1103,32 +1117,39 @@ class Ops:
         """``(experts [T, top] int32, weights [T, top] float32)``: 32-bit logits ``h @ router [n, E]^T`` (a matrix
         product with 32-bit accumulation and a 32-bit result; ``router`` in ``h``'s dtype, a matrix or a
         ``PackedWeight``), a softmax over all experts, the ``top`` largest of score + ``correction`` (the lower
-        index on a tie), weights = the chosen scores over their sum + 1e-20."""
+        index on a tie), weights = the chosen scores over their sum + 1e-20.  Options as in ``route_logits``."""
         logits = self.linear(h, router, out_dtype=torch.float32)
         return self.route_logits(logits, correction, top, **how)
 
     def route_logits(self, logits: torch.Tensor, correction: torch.Tensor, top: int, scores: str = "softmax",
-                     groups: int = 1, keep_groups: int = 1, weight_scale: Optional[float] = None):
+                     groups: int = 1, keep_groups: int = 1, weight_scale: Optional[float] = None, side_gate: bool = False):
         """``moe_route`` from the 32-bit logits ``[T, n]``.  ``scores`` "sigmoid": every expert's score is the sigmoid
         of its logit.  ``groups`` > 1: the experts form that many equal groups of neighbours, a group scores the
         sum of its two largest score + correction, and only the ``keep_groups`` best groups' experts can be chosen.
-        ``weight_scale``: the weights are the chosen scores times it instead of their shares of their sum."""
-        if scores not in ("softmax", "sigmoid"):
-            raise KernelError(f"route_logits: scores {scores!r} (softmax or sigmoid)")
+        ``weight_scale``: the weights are the chosen scores times it instead of their shares of their sum.  ``scores``
+        "logits": the choice is by logit + ``correction`` (the router's bias), the weights are the softmax of these over
+        the chosen experts.  ``side_gate``: the logits have one column more, ``[T, n + 1]``, which is no expert's; its
+        sigmoid comes back as a third result ``[T]``."""
+        if scores not in ROUTE_SCORES:
+            raise KernelError(f"route_logits: scores {scores!r} ({', '.join(ROUTE_SCORES)})")
+        if scores == "logits" and (groups != 1 or weight_scale is not None):
+            raise KernelError("route_logits: a choice by the logits has no groups and no weight scale")
         if weight_scale is not None and not weight_scale > 0:
             raise KernelError(f"route_logits: weight scale {weight_scale} must be positive")
         self._dev(logits, correction)
         if logits.dtype != torch.float32 or logits.dim() != 2 or logits.stride(1) != 1:
             raise KernelError("route_logits: logits must be float32 [rows, experts] with unit column stride")
         T, n = logits.shape
+        n -= 1 if side_gate else 0
         if correction.dtype != torch.float32 or correction.numel() != n:
             raise KernelError(f"route_logits: the correction must be float32 [{n}]")
         idx = torch.empty((T, top), dtype=torch.int32, device=logits.device)
         wts = torch.empty((T, top), dtype=torch.float32, device=logits.device)
-        self.lib.check(self.lib.xr_moe_route(idx.data_ptr(), wts.data_ptr(), logits.data_ptr(), correction.data_ptr(), T,
-                                             logits.stride(0), n, int(top), 1 if scores == "sigmoid" else 0, int(groups),
+        side = torch.empty((T,), dtype=torch.float32, device=logits.device) if side_gate else None
+        self.lib.check(self.lib.xr_moe_route(idx.data_ptr(), wts.data_ptr(), _ptr(side), logits.data_ptr(), correction.data_ptr(), T,
+                                             logits.stride(0), n, int(top), ROUTE_SCORES[scores], int(groups),
                                              int(keep_groups), float(weight_scale or 0.0), _stream()))
-        return idx, wts
+        return (idx, wts, side) if side_gate else (idx, wts)
 
     def table_route(self, table: torch.Tensor, ids: torch.Tensor, n_experts: int):
         """``(experts [T, top] int32, weights [T, top] float32)`` without a router: row ``ids[t]`` of ``table
@@ -1147,11 +1168,13 @@ class Ops:
     GROUPED_EXPERTS_FROM = 32       # choices (rows x top) from which the experts' rows are sorted and run on the matrix cores
 
     def moe_experts(self, h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor,
-                    out: Optional[torch.Tensor] = None, accumulate: bool = False, activation: str = "relu2") -> torch.Tensor:
+                    out: Optional[torch.Tensor] = None, accumulate: bool = False, activation: str = "relu2", param: float = 0.0,
+                    beside=None) -> torch.Tensor:
         """``out[t] (+)= sum_j wts[t, j] * w_down[e] @ relu(w_up[e] @ h[t])^2`` with ``e = idx[t, j]``, as 32-bit
         rows; ``w_up [n, F, E]`` and ``w_down [n, E, F]`` in ``h``'s dtype.  ``activation`` "swiglu": gated experts,
         ``w_down[e] @ (silu(g) * u)`` with ``[g; u] = w_up[e] @ h[t]`` for ``w_up [n, 2F, E]`` (an expert's gate rows
-        before its up rows).  A few choices stream the chosen
+        before its up rows); "clamped_swish" and "gelu_tanh" likewise with that gate (its number ``param``).  ``beside`` =
+        (32-bit rows ``[T, E]``, one weight a row ``[T]``): these rows enter the sum too.  A few choices stream the chosen
         experts' weights, a wave an output column; from ``GROUPED_EXPERTS_FROM`` choices on (bfloat16, widths
         that are multiples of 8) the rows are sorted by expert on the device, both products run on the matrix
         cores and a last kernel adds a token's experts up in the order of its choice."""
@@ -1159,7 +1182,14 @@ class Ops:
         T, E = h.shape
         if activation not in EXPERT_ACTIVATIONS:
             raise KernelError(f"moe_experts: activation {activation!r} (known: {sorted(EXPERT_ACTIVATIONS)})")
-        gated = activation == "swiglu"
+        form, gate = EXPERT_ACTIVATIONS[activation]
+        gated = form == 1
+        y_beside, g_beside = beside if beside is not None else (None, None)
+        if beside is not None:
+            self._dev(y_beside, g_beside)
+            if (y_beside.dtype != torch.float32 or tuple(y_beside.shape) != tuple(h.shape) or not y_beside.is_contiguous()
+                    or g_beside.dtype != torch.float32 or g_beside.numel() != h.shape[0] or not g_beside.is_contiguous()):
+                raise KernelError(f"moe_experts: the rows beside must be contiguous float32 {tuple(h.shape)} with a float32 weight a row")
         n, Fu, _ = w_up.shape
         F = Fu // 2 if gated else Fu
         top = idx.shape[1]
@@ -1186,12 +1216,13 @@ class Ops:
             self.lib.check(self.lib.xr_moe_experts_grouped(out.data_ptr(), z.data_ptr(), yz.data_ptr(), scratch.data_ptr(),
                                                            h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(), idx.data_ptr(),
                                                            wts.data_ptr(), T, E, F, h.stride(0), out.stride(0), n, top,
-                                                           1 if accumulate else 0, _ptr(gu), _stream()))
+                                                           1 if accumulate else 0, _ptr(gu), gate, float(param), _ptr(y_beside),
+                                                           _ptr(g_beside), _stream()))
             return out
         self.lib.check(self.lib.xr_moe_experts(out.data_ptr(), z.data_ptr(), h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(),
                                                idx.data_ptr(), wts.data_ptr(), T, E, F, h.stride(0), out.stride(0), n, top,
-                                               1 if accumulate else 0, dtype_code(h.dtype), EXPERT_ACTIVATIONS[activation],
-                                               _stream()))
+                                               1 if accumulate else 0, dtype_code(h.dtype), form, gate, float(param),
+                                               _ptr(y_beside), _ptr(g_beside), _stream()))
         return out
 
     def delta_prepare_(self, q, k, b, a, a_log, dt_bias, G: int, H: int, D: int, q_scale: float, unit_eps: float) -> None:
@@ -1358,7 +1389,7 @@ class Ops:
                 out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), plan.items.data_ptr(),
                 plan.n_items, plan.n_cta_items, _ptr(plan.jobs), plan.n_jobs, ctx.cu_q.data_ptr(),
                 ctx.starts_dev.data_ptr(), table.data_ptr(), table.stride(0), _ptr(part_o), _ptr(part_ml), H, Hk, D, page_size,
-                float(scale), int(size), 0, None, None, _stream()))
+                float(scale), int(size), 0, None, None, 0.0, _stream()))
             return out
         self.lib.check(self.lib.xr_attention_pooled(
             out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), _ptr(pk) if P else None,

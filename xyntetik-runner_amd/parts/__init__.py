@@ -5,13 +5,13 @@ from .base import (Part, Norm, PositionEncoding, QKTransform, Mixer, FeedForward
 from . import norm, rotary, embedding, head, mlp, attention, block, filters, pooled_attention, recurrent, latent_attention    # noqa: F401  (registers the built-in parts)
 from . import qk_norm, injection, parallel    # noqa: F401
 from .norm import RMSNorm, LayerNorm, DynamicTanh
-from .qk_norm import HeadRMSNorm
+from .qk_norm import HeadRMSNorm, RowRMSNorm
 from .injection import ConcatProjection, StepAddition
 from .parallel import ParallelMixers
 from .filters import CausalConv
 from .pooled_attention import PooledWindowAttention
 from .recurrent import Retention, GatedDelta, TimeMixWKV, GatedLinearAttention
-from .rotary import Rotary, NoPosition, rotary_inv_freq
+from .rotary import Rotary, NoPosition, rotary_inv_freq, yarn_mscale
 from .embedding import TokenEmbedding, PairHashEmbedding
 from .head import LinearHead
 from .mlp import GatedMLP, DenseMLP, RoutedExperts
@@ -28,5 +28,5 @@ __all__ = [
     "Retention", "GatedDelta", "DenseMLP", "FilteredPreNormBlock", "register_connection", "Connection", "PairHashEmbedding",
     "RoutedExperts", "LatentAttention", "StreamsPreNormBlock", "StreamConnection", "DynamicTanh", "HeadRMSNorm",
     "ConcatProjection", "TimeMixWKV", "SandwichBlock", "register_injection", "Injection", "StepAddition", "ParallelMixers",
-    "GatedLinearAttention",
+    "GatedLinearAttention", "RowRMSNorm", "yarn_mscale",
 ]

@@ -22,7 +22,7 @@ run in); ``keep_first``: with a window, the first so many keys stay readable, at
 ``sink``: the softmax's denominator holds one entry more, without key or value: "learned" (a score a head, the
 tensor ``sink_name``, unscaled) or "zero" (the score 0: one is added to the denominator); ``gate_name``: a
 projection ``[H, E]`` of the mixer's input whose sigmoid multiplies every head's output before the output
-projection.
+projection; ``softcap`` c > 0: every scaled score s becomes ``c tanh(s / c)`` (before a slope's bias and not the sink).
 """
 from __future__ import annotations
 
@@ -45,7 +45,8 @@ class PagedAttention(Mixer):
                  q_name: str = "q_proj", k_name: str = "k_proj", v_name: str = "v_proj",
                  o_name: str = "o_proj", values: str = "projection", slopes=None, weight_suffix: str = ".weight",
                  bias_suffix: str = ".bias", v_head_dim: Optional[int] = None, chunk: Optional[int] = None,
-                 keep_first: int = 0, sink: Optional[str] = None, sink_name: str = "sink", gate_name: Optional[str] = None):
+                 keep_first: int = 0, sink: Optional[str] = None, sink_name: str = "sink", gate_name: Optional[str] = None,
+                 softcap: float = 0.0):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are not a multiple of {num_kv_heads} key/value heads")
         if window is not None and window < 1:
@@ -70,6 +71,9 @@ class PagedAttention(Mixer):
             raise ValueError(f"attention value size {v_head_dim} is outside what the attention kernels take (1 to {MAX_HEAD_DIM})")
         if self.v_head_dim != int(head_dim) and values == "keys":
             raise ValueError("attention: values that are the keys have the keys' size")
+        if float(softcap) < 0.0:
+            raise ValueError(f"attention: soft cap {softcap} of the scores is negative (0: none)")
+        self.softcap = float(softcap)
         self.sinks = self.w_gate = None
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.head_dim)
         self.bias = bool(bias)
@@ -235,7 +239,7 @@ class PagedAttention(Mixer):
                               rot.mscale if rot else 1.0, cache.page_size, paired=self.paired)
         o = ops.attention(q, cache.k, cache.v, ctx, cache.group, H, Hk, D, cache.page_size, self.scale,
                           self.window, slopes=self.slopes, chunk=self.chunk, keep_first=self.keep_first, sinks=self.sinks,
-                          v_head_dim=Dv)
+                          v_head_dim=Dv, softcap=self.softcap)
         if gate is not None:
             ops.head_gate_(o, gate, H, Dv)
         return o

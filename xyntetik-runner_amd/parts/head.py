@@ -1,5 +1,6 @@
 """The output head: ``logits = W h`` in 32-bit, with ``W`` its own tensor or the
-embedding table when the model ties them (src/model.c:2353-2366, :6481).
+embedding table when the model ties them (src/model.c:2353-2366, :6481).  ``softcap`` c > 0:
+the logits leave as ``c tanh(logits / c)``.
 """
 from __future__ import annotations
 
@@ -11,9 +12,12 @@ from .base import Part, ParamSpec, register_head
 
 
 class LinearHead(Part):
-    def __init__(self, vocab_size: int, hidden_size: int, tied: bool = False, weight_name: str = "weight"):
+    def __init__(self, vocab_size: int, hidden_size: int, tied: bool = False, weight_name: str = "weight",
+                 softcap: float = 0.0):
         self.vocab_size, self.hidden_size, self.tied = int(vocab_size), int(hidden_size), bool(tied)
-        self.weight_name = weight_name
+        if float(softcap) < 0.0:
+            raise ValueError(f"output head: soft cap {softcap} is negative (0: none)")
+        self.weight_name, self.softcap = weight_name, float(softcap)
         self.weight = None
 
     def param_specs(self) -> Dict[str, ParamSpec]:
@@ -35,7 +39,10 @@ class LinearHead(Part):
             tied_to.share_table(self.weight)
 
     def forward(self, ctx, h):
-        return self.rt.ops.linear(h, self.weight, out_dtype=torch.float32)
+        logits = self.rt.ops.linear(h, self.weight, out_dtype=torch.float32)
+        if self.softcap > 0.0:
+            self.rt.ops.softcap_(logits, self.softcap)
+        return logits
 
 
 register_head("linear", LinearHead)

@@ -17,7 +17,11 @@ added to the sum (``shared_size``: its inner width; a gated feed-forward with th
 the sigmoid of each expert's logit instead of a softmax over all (``scores="sigmoid"``); a choice limited to the best
 groups (``groups`` equal groups of neighbouring experts, a group's score the sum of its two largest score +
 correction, ``keep_groups`` groups whose experts can be chosen; the others count as minus infinity); weights that are
-the chosen scores times a number (``weight_scale``) instead of their shares of their sum.
+the chosen scores times a number (``weight_scale``) instead of their shares of their sum; a choice by the logits
+themselves, the correction being the router's bias (``scores="logits"``: the weights are the softmax over the chosen
+logits, bias included); experts and a shared expert gated by any gate of ``GATE_ACTIVATIONS`` with a number of its own
+(``activation``, ``activation_param``; ``shared_activation``, ``shared_param``); a number a token on the shared expert,
+``sigmoid(w . h)`` (``shared_gate_name``: the ``[1, E]`` tensor ``w``).
 
 Dense feed-forward: ``down(act(up(h)))`` with an activation over the whole row.  "polynorm":
 ``a N(z) + b N(z^2) + c N(z^3) + e`` with four learned numbers, powers element by element and
@@ -25,7 +29,7 @@ Dense feed-forward: ``down(act(up(h)))`` with an activation over the whole row. 
 """
 from __future__ import annotations
 
-from typing import Dict
+from typing import Dict, Optional
 
 import torch
 
@@ -137,7 +141,7 @@ class RoutedExperts(FeedForward):
     ``table [vocab, top]`` (integers); with a shared expert ``shared.gate``, ``shared.up``, ``shared.down``.
     Nothing here reads the choice on the host: the kernels find a token's
     experts on the device, so decode steps are recorded like any other."""
-    ACTIVATIONS = ("relu2", "swiglu")
+    ACTIVATIONS = ("relu2", "swiglu", "clamped_swish", "gelu_tanh")      # all but the first are gates
     ROUTINGS = ("router", "table")
     MAX_EXPERTS, MAX_TOP = 1024, 64     # MOE_MAX_EXPERTS, MOE_MAX_TOP of csrc/moe_kernels.hip
 
@@ -145,7 +149,9 @@ class RoutedExperts(FeedForward):
                  router_name: str = "router", correction_name: str = "correction", expert_prefix: str = "e",
                  up_name: str = "up", down_name: str = "down", gate_name: str = "gate", routing: str = "router",
                  vocab_size: int = 0, table_name: str = "table", shared_size: int = 0, shared_prefix: str = "shared.",
-                 scores: str = "softmax", groups: int = 1, keep_groups: int = 1, weight_scale=None):
+                 scores: str = "softmax", groups: int = 1, keep_groups: int = 1, weight_scale=None,
+                 activation_param: float = 0.0, shared_activation: str = "silu", shared_param: float = 0.0,
+                 shared_gate_name: Optional[str] = None):
         if activation not in self.ACTIVATIONS:
             raise ValueError(f"routed experts: activation {activation!r} is not built (known: {list(self.ACTIVATIONS)})")
         if routing not in self.ROUTINGS:
@@ -154,9 +160,13 @@ class RoutedExperts(FeedForward):
             raise ValueError("routed experts: a table of experts by token id needs the vocabulary's size")
         self.activation, self.routing, self.vocab_size = activation, routing, int(vocab_size)
         self.gate_name, self.table_name = gate_name, table_name
-        self.shared = (GatedMLP(hidden_size, int(shared_size), activation="silu", gate_name=shared_prefix + "gate",
+        self.activation_param = float(activation_param)
+        self.shared = (GatedMLP(hidden_size, int(shared_size), activation=shared_activation, activation_param=shared_param, gate_name=shared_prefix + "gate",
                                 up_name=shared_prefix + "up", down_name=shared_prefix + "down", weight_suffix="")
                        if int(shared_size) > 0 else None)
+        self.shared_gate_name = shared_gate_name
+        if shared_gate_name is not None and (self.shared is None or routing != "router"):
+            raise ValueError("routed experts: a gate on the shared expert needs one, and a router whose product makes its logit")
         if not (1 <= int(top) <= int(num_experts)):
             raise ValueError(f"routed experts: {top} of {num_experts} experts a token")
         if int(num_experts) > self.MAX_EXPERTS or int(top) > self.MAX_TOP:       # refused when the model is built, not at its first step
@@ -165,8 +175,10 @@ class RoutedExperts(FeedForward):
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.num_experts, self.top = int(num_experts), int(top)
         groups, keep_groups = int(groups), int(keep_groups)
-        if scores not in ("softmax", "sigmoid"):
-            raise ValueError(f"routed experts: scores {scores!r} (softmax or sigmoid)")
+        if scores not in ("softmax", "sigmoid", "logits"):
+            raise ValueError(f"routed experts: scores {scores!r} (softmax, sigmoid or logits)")
+        if scores == "logits" and (groups != 1 or weight_scale is not None):
+            raise ValueError("routed experts: a choice by the logits has no groups, and its weights are the softmax over the chosen")
         if (groups < 1 or self.num_experts % groups or not (1 <= keep_groups <= groups)
                 or self.top > keep_groups * (self.num_experts // groups)):
             raise ValueError(f"routed experts: {num_experts} experts in {groups} groups of which {keep_groups} are kept "
@@ -176,6 +188,10 @@ class RoutedExperts(FeedForward):
         self.how = dict(scores=scores, groups=groups, keep_groups=keep_groups,
                         weight_scale=float(weight_scale) if weight_scale is not None else None)
         self.names = (router_name, correction_name, expert_prefix, up_name, down_name)
+
+    @property
+    def gated(self) -> bool:
+        return self.activation != "relu2"
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         E, F = self.hidden_size, self.intermediate_size
@@ -187,12 +203,14 @@ class RoutedExperts(FeedForward):
             specs = {r: ParamSpec((self.num_experts, E), init="normal:0.5"),
                      c: ParamSpec((self.num_experts,), role="vector", init="normal:0.1")}
         for e in range(self.num_experts):
-            if self.activation == "swiglu":
+            if self.gated:
                 specs[f"{p}{e}.{self.gate_name}"] = ParamSpec((F, E))
             specs[f"{p}{e}.{u}"] = ParamSpec((F, E))
             specs[f"{p}{e}.{d}"] = ParamSpec((E, F))
         if self.shared is not None:
             specs.update(self.shared.param_specs())
+        if self.shared_gate_name is not None:
+            specs[self.shared_gate_name] = ParamSpec((1, E), init="normal:0.1")
         return specs
 
     def bind(self, tensors, rt) -> None:
@@ -201,9 +219,13 @@ class RoutedExperts(FeedForward):
         if self.routing == "table":
             self.table = tensors[self.table_name].to(torch.int32).contiguous()
         else:
-            self.router = rt.ops.pack_weight(tensors[r])        # in the rows' dtype: the logits are a 32-bit product of the two
+            # in the rows' dtype: the logits are a 32-bit product of the two; a gate on the shared expert is one more row of it
+            rows = tensors[r]
+            if self.shared_gate_name is not None:
+                rows = torch.cat([rows, tensors[self.shared_gate_name]], dim=0)
+            self.router = rt.ops.pack_weight(rows.contiguous())
             self.correction = tensors[c].float().contiguous()
-        if self.activation == "swiglu":     # an expert's gate rows before its up rows: one matrix [2F, E] an expert
+        if self.gated:      # an expert's gate rows before its up rows: one matrix [2F, E] an expert
             self.w_up = torch.stack([torch.cat([tensors[f"{p}{e}.{self.gate_name}"], tensors[f"{p}{e}.{u}"]], dim=0)
                                      for e in range(self.num_experts)]).contiguous()
         else:
@@ -214,12 +236,17 @@ class RoutedExperts(FeedForward):
 
     def _run(self, ctx, h, out=None, accumulate=False):
         ops = self.rt.ops
+        beside = None
         if self.routing == "table":
             idx, wts = ops.table_route(self.table, ctx.token_ids, self.num_experts)
-        else:
+        elif self.shared_gate_name is None:
             idx, wts = ops.moe_route(h, self.router, self.correction, self.top, **self.how)
-        out = ops.moe_experts(h, self.w_up, self.w_down, idx, wts, out=out, accumulate=accumulate, activation=self.activation)
-        if self.shared is not None:
+        else:       # the shared expert's rows enter the sum of the chosen ones with the token's gate
+            idx, wts, gate = ops.moe_route(h, self.router, self.correction, self.top, side_gate=True, **self.how)
+            beside = (self.shared.forward_f32(ctx, h), gate)
+        out = ops.moe_experts(h, self.w_up, self.w_down, idx, wts, out=out, accumulate=accumulate, activation=self.activation,
+                              param=self.activation_param, beside=beside)
+        if self.shared is not None and beside is None:
             self.shared.forward_add(ctx, h, out)
         return out
 

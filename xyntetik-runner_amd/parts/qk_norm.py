@@ -5,6 +5,9 @@ the root) and multiplied by a weight over the head's channels that all heads sha
 queries, one for the keys; the plain weight, not one plus it).  With ``temp_every`` the queries of the
 token at position p are also multiplied by ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)``, which
 sharpens the attention of tokens far into a sequence.
+
+``RowRMSNorm``: the queries of all heads together are divided by their one root mean square and multiplied by
+a weight over the whole projection, and so are the keys.
 """
 from __future__ import annotations
 
@@ -40,4 +43,32 @@ class HeadRMSNorm(QKTransform):
                                   self.temp_coef, self.temp_every)
 
 
+class RowRMSNorm(QKTransform):
+    def __init__(self, q_size: int, k_size: int, eps: float, q_name: str = "q_norm", k_name: str = "k_norm"):
+        self.q_size, self.k_size, self.eps = int(q_size), int(k_size), float(eps)
+        self.q_name, self.k_name = q_name, k_name
+        self.w_q = self.w_k = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        return {self.q_name: ParamSpec((self.q_size,), role="vector", init="ones_jitter"),
+                self.k_name: ParamSpec((self.k_size,), role="vector", init="ones_jitter")}
+
+    def bind(self, tensors, rt) -> None:
+        self.rt = rt
+        self.w_q = tensors[self.q_name].float().contiguous()
+        self.w_k = tensors[self.k_name].float().contiguous()
+
+    def row_norm(self):
+        """(query weight, key weight, eps) for the kernel that also rotates and caches the row (``Ops.row_norm_rope_write``)."""
+        return self.w_q, self.w_k, self.eps
+
+    def apply(self, ctx, q, k) -> None:
+        # a row is one head of its whole width
+        ops = self.rt.ops
+        ops.head_rmsnorm_(q.flatten(1).unsqueeze(1), None, self.w_q, None, self.eps)
+        if k is not None:
+            ops.head_rmsnorm_(k.flatten(1).unsqueeze(1), None, self.w_k, None, self.eps)
+
+
 register_qk_transform("head_rmsnorm", HeadRMSNorm)
+register_qk_transform("row_rmsnorm", RowRMSNorm)

@@ -11,7 +11,14 @@ The reference then divides by per-dimension factors that the model file brings f
     otherwise, with s = (orig / wavelen - low) / (high - low):
                                          (1 - s) * inv_freq / factor + s * inv_freq
 
-"linear" divides every frequency by ``factor`` (src/model.c:317-321).
+"linear" divides every frequency by ``factor`` (src/model.c:317-321).  "yarn" mixes the two by how often a pair
+turns within ``orig`` positions: with ``pair(t) = rotary_dim ln(orig / (2 pi t)) / (2 ln theta)``, the (real) number of
+the pair that turns t times, ``lo = max(floor(pair(beta_fast)), 0)``, ``hi = min(ceil(pair(beta_slow)), rotary_dim - 1)``
+and ``r_j = clamp((j - lo) / max(hi - lo, 0.001), 0, 1)``:
+
+    inv_freq_j = r_j inv_freq_j / factor + (1 - r_j) inv_freq_j
+
+``yarn_mscale(factor)`` is the factor on cosines and sines that goes with it.
 The rotation itself (pairing, angle = position * inv_freq in 32-bit) is applied by
 the kernel that writes keys to the cache (src/model.c:3514-3532).
 """
@@ -23,6 +30,8 @@ from typing import Any, Mapping, Optional
 import torch
 
 from .base import PositionEncoding, RotaryParams, register_position
+
+YARN_MIN_RAMP = 0.001       # the ramp between turned and slowed pairs is at least this long
 
 
 def rotary_inv_freq(rotary_dim: int, theta: float, scaling: Optional[Mapping[str, Any]] = None) -> torch.Tensor:
@@ -49,7 +58,22 @@ def rotary_inv_freq(rotary_dim: int, theta: float, scaling: Optional[Mapping[str
         out = torch.where(wavelen > orig / low, inv / factor, inv)
         between = (wavelen <= orig / low) & (wavelen >= orig / high)
         return torch.where(between, mid, out)
+    if kind == "yarn":
+        orig = float(scaling["original_max_position_embeddings"])
+
+        def pair(turns: float) -> float:
+            return rotary_dim * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(theta))
+
+        lo = max(math.floor(pair(float(scaling.get("beta_fast", 32.0)))), 0)
+        hi = min(math.ceil(pair(float(scaling.get("beta_slow", 1.0)))), rotary_dim - 1)
+        slowed = ((j - lo) / max(hi - lo, YARN_MIN_RAMP)).clamp(0.0, 1.0)
+        return slowed * inv / factor + (1.0 - slowed) * inv
     raise ValueError(f"rope scaling {kind!r} is not supported")
+
+
+def yarn_mscale(factor: float) -> float:
+    """What YaRN multiplies cosines and sines by: ``0.1 ln(factor) + 1``."""
+    return 0.1 * math.log(factor) + 1.0
 
 
 class Rotary(PositionEncoding):
