@@ -434,6 +434,175 @@ extern "C" int xr_rope_kv_write(const float* q_in, const float* k_in, const floa
     return XR_OK;
 }
 
+// ---------------------------------------------------------------- norm over all heads + rotary + cache write
+// The same for queries and keys that are normed over all their heads at once first (RMS, eps inside the root, a
+// weight a channel of the whole projection): a workgroup takes a token, sums the squares of its queries and of its
+// keys, and rotates what it scales.  Values come from rows of their own, which may be the keys' before norm and
+// rotation; they are stored as above.  NW waves: 4 where there are tokens enough to fill the chip, 16 for the few of a
+// decode step.  VEC: neighbouring pairs, head size, rotated part, widths and strides multiples of 4, bases on 16 bytes:
+// a lane takes 4 channels (two pairs) of a head.
+struct RowNormArgs {
+    RopeArgs r;
+    const float* wq;        // [H * D]
+    const float* wk;        // [Hk * D]
+    float eps;
+};
+
+template <typename T> __device__ inline void put4(T* p, float a, float b, float c, float d);
+template <> __device__ inline void put4<float>(float* p, float a, float b, float c, float d) {
+    *reinterpret_cast<float4*>(p) = make_float4(a, b, c, d);
+}
+template <> __device__ inline void put4<bf16_t>(bf16_t* p, float a, float b, float c, float d) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(c, d));
+}
+
+template <typename T, int NW, bool VEC>
+__global__ __launch_bounds__(64 * NW) void k_row_norm_rope_write(RowNormArgs n) {
+    constexpr int NT = 64 * NW;
+    __shared__ float cs[2][128];
+    __shared__ float part[2][NW];
+    const RopeArgs& a = n.r;
+    const int t = blockIdx.x, tid = threadIdx.x;
+    const int D = a.D, half = a.rot >> 1, Q = a.H * D, K = a.Hk * D;
+    const float* qr = a.q_in + (size_t)t * a.in_stride;
+    const float* kr = a.Hk ? a.k_in + (size_t)t * a.in_stride : qr;
+    const int pos = a.positions[t];
+    float sq = 0.f, sk = 0.f;
+    if (VEC) {
+        for (int i = tid * 4; i < Q; i += NT * 4) {
+            const float4 x = *reinterpret_cast<const float4*>(qr + i);
+            sq += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+        }
+        for (int i = tid * 4; i < K; i += NT * 4) {
+            const float4 x = *reinterpret_cast<const float4*>(kr + i);
+            sk += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+        }
+    } else {
+        for (int i = tid; i < Q; i += NT) sq = fmaf(qr[i], qr[i], sq);
+        for (int i = tid; i < K; i += NT) sk = fmaf(kr[i], kr[i], sk);
+    }
+    for (int j = tid; j < half; j += NT) {
+        const float ang = (float)pos * a.inv_freq[j];
+        cs[0][j] = cosf(ang) * a.mscale;
+        cs[1][j] = sinf(ang) * a.mscale;
+    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((tid & 63) == 0) { part[0][tid >> 6] = sq; part[1][tid >> 6] = sk; }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) { sq += part[0][w]; sk += part[1][w]; }
+    const float rq = 1.0f / sqrtf(sq / (float)Q + n.eps);
+    const float rk = K ? 1.0f / sqrtf(sk / (float)K + n.eps) : 0.f;
+    PageRef pr{0, 0};
+    int req = 0;
+    if (K) {
+        req = a.req_of_token[t];
+        pr = page_of(a.block_table, a.table_stride, req, pos, a.page_shift, a.page_mask);
+    }
+    T* qo = (T*)a.q_out + (size_t)t * Q;
+    // channel d of key head g of this token: kpage + g * (page_size * D) + d
+    T* kpage = (T*)a.k_cache + ((size_t)pr.page * a.Hk * a.page_size + pr.off) * D;
+    const int total = Q + K;
+    if (VEC) {
+        for (int i4 = tid * 4; i4 < total; i4 += NT * 4) {
+            const bool is_q = i4 < Q;
+            const int i = is_q ? i4 : i4 - Q;
+            const int head = i / D, d = i - head * D;
+            float4 x = *reinterpret_cast<const float4*>((is_q ? qr : kr) + i);
+            const float4 w = *reinterpret_cast<const float4*>((is_q ? n.wq : n.wk) + i);
+            const float f = is_q ? rq : rk;
+            x.x *= f * w.x; x.y *= f * w.y; x.z *= f * w.z; x.w *= f * w.w;
+            if (d < a.rot) {
+                const int j = d >> 1;
+                const float c0 = cs[0][j], s0 = cs[1][j], c1 = cs[0][j + 1], s1 = cs[1][j + 1];
+                x = make_float4(x.x * c0 - x.y * s0, x.x * s0 + x.y * c0, x.z * c1 - x.w * s1, x.z * s1 + x.w * c1);
+            }
+            put4<T>(is_q ? qo + i : kpage + (size_t)head * a.page_size * D + d, x.x, x.y, x.z, x.w);
+        }
+    } else {
+        for (int ii = tid; ii < total; ii += NT) {
+            const bool is_q = ii < Q;
+            const int i = is_q ? ii : ii - Q;
+            const int head = i / D, d = i - head * D;
+            const float* src = is_q ? qr : kr;
+            const float* w = is_q ? n.wq : n.wk;
+            const float f = is_q ? rq : rk;
+            float y = src[i] * f * w[i];
+            if (d < a.rot) {
+                const int j = a.interleaved ? d >> 1 : (d < half ? d : d - half);
+                const bool first = a.interleaved ? (d & 1) == 0 : d < half;
+                const int o = i + (first ? 1 : -1) * (a.interleaved ? 1 : half);     // the pair's other channel
+                const float z = src[o] * f * w[o];
+                y = first ? y * cs[0][j] - z * cs[1][j] : z * cs[1][j] + y * cs[0][j];
+            }
+            st<T>(is_q ? qo : kpage + (size_t)head * a.page_size * D, is_q ? i : d, y);
+        }
+    }
+    if (!K) return;
+    // values: see k_rope_kv_write
+    const float* vr = a.v_in + (size_t)t * a.in_stride;
+    T* vpage = (T*)a.v_cache + (size_t)pr.page * K * a.page_size + pr.off;
+    const int lead = t - (pos & 7);
+    const bool whole = a.page_size >= 8 && lead >= 0 && lead + 7 < a.T && a.req_of_token[lead] == req &&
+                       a.req_of_token[lead + 7] == req && a.positions[lead] == pos - (pos & 7);
+    if (!whole) {
+        for (int i = tid; i < K; i += NT) st<T>(vpage, (size_t)i * a.page_size, vr[i]);
+    } else if ((pos & 7) == 0) {
+        for (int i = tid; i < K; i += NT) {
+            float v[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] = vr[(size_t)j * a.in_stride + i];
+            store8<T>(vpage + (size_t)i * a.page_size, v);
+        }
+    }
+}
+
+extern "C" int xr_row_norm_rope_write(const float* q_in, const float* k_in, const float* v_in, int in_stride, const float* wq,
+                                      const float* wk, float eps, void* q_out, void* k_cache, void* v_cache,
+                                      const int* positions, const int* req_of_token, const int* block_table,
+                                      int table_stride, const float* inv_freq, int T, int H, int Hk, int D, int rot,
+                                      int interleaved, float mscale, int page_size, int dtype, hipStream_t stream) {
+    XR_REQUIRE(T >= 0 && H > 0 && Hk >= 0 && D > 0, "row_norm_rope_write: bad sizes T=%d H=%d Hk=%d D=%d", T, H, Hk, D);
+    XR_REQUIRE(rot >= 0 && rot <= D && (rot % 2) == 0 && rot <= 256, "row_norm_rope_write: rotary width %d must be even, at most head_dim %d and 256", rot, D);
+    XR_REQUIRE(rot == 0 || inv_freq, "row_norm_rope_write: rotary width %d without a frequency table", rot);
+    XR_REQUIRE(eps >= 0.f, "row_norm_rope_write: eps %g is negative", (double)eps);
+    const int shift = ilog2_exact(page_size);
+    XR_REQUIRE(Hk == 0 || shift >= 0, "row_norm_rope_write: page size %d is not a power of two", page_size);
+    XR_REQUIRE(Hk == 0 || (k_in && v_in && wk && k_cache && v_cache && block_table && req_of_token),
+               "row_norm_rope_write: keys and values to cache but a null operand");
+    XR_REQUIRE(q_in && q_out && wq && positions, "row_norm_rope_write: an operand is missing");
+    XR_REQUIRE(dtype == XR_F32 || dtype == XR_BF16, "row_norm_rope_write: bad dtype %d", dtype);
+    if (T == 0) return XR_OK;
+    RowNormArgs n;
+    RopeArgs& a = n.r;
+    a.q_in = q_in; a.k_in = k_in; a.v_in = v_in; a.in_stride = in_stride;
+    a.q_out = q_out; a.k_cache = k_cache; a.v_cache = v_cache;
+    a.positions = positions; a.req_of_token = req_of_token;
+    a.block_table = block_table; a.table_stride = table_stride; a.inv_freq = inv_freq;
+    a.T = T; a.H = H; a.Hk = Hk; a.D = D; a.rot = rot; a.interleaved = interleaved; a.mscale = mscale;
+    a.page_shift = shift < 0 ? 0 : shift; a.page_mask = page_size - 1; a.page_size = page_size;
+    a.heads_per_block = 0; a.paired = 0;
+    n.wq = wq; n.wk = wk; n.eps = eps;
+    auto on16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };
+    const bool vec = (interleaved || rot == 0) && D % 4 == 0 && rot % 4 == 0 && in_stride % 4 == 0 && on16(q_in) && on16(k_in) &&
+                     on16(wq) && on16(wk) && on16(q_out) && on16(k_cache);
+    const bool few = T <= 128 && (H + Hk) * D >= 1024;
+#define RNW(TT)                                                                                    \
+    do {                                                                                            \
+        if (vec && few) k_row_norm_rope_write<TT, 16, true><<<T, 1024, 0, stream>>>(n);             \
+        else if (vec) k_row_norm_rope_write<TT, 4, true><<<T, 256, 0, stream>>>(n);                 \
+        else if (few) k_row_norm_rope_write<TT, 16, false><<<T, 1024, 0, stream>>>(n);              \
+        else k_row_norm_rope_write<TT, 4, false><<<T, 256, 0, stream>>>(n);                         \
+    } while (0)
+    if (dtype == XR_F32) RNW(float);
+    else RNW(bf16_t);
+#undef RNW
+    XR_CHECK_LAUNCH("row_norm_rope_write");
+    return XR_OK;
+}
+
 // ---------------------------------------------------------------- gate
 // h = act(g) * u; act = SiLU: g / (1 + exp(-g)) (src/model.c:4451-4452,
 // src/kernels.cu:2868-2874).  gu row = [gate(F) | up(F)].

@@ -76,6 +76,7 @@ struct GemmArgs {
     float* partial;    // [splits][M][rows of w]
     int raw;           // 1: raw sums go to `partial` also when K is whole (an epilogue of k_gemm_finish is wanted)
     int norm_whole;    // 1: k_gemm_finish_norm writes the whole norm of the updated rows to xg
+    int norm_centred;  // 1: that norm is a layer norm (the rows' mean taken off first), else an RMS norm
     int col0, col1;    // the tile kernel computes output columns col0 .. col1-1 (col0 a multiple of the tile's width)
     int vec_out;       // 1: the tile kernel may write 4 columns a lane (widths and row strides are multiples of 4, bases 16-byte aligned)
     // RMSNorm folded into the skinny kernel (all null or zero: off).
@@ -120,6 +121,7 @@ struct XrGemmNorm {
     void* xg;
     float* ss_out;
     int ss_out_rows;   // in: partial rows that ss_out has room for; out: partial rows written
+    int centred;       // the norm after the product is a layer norm (more than 16 rows, finished by k_gemm_finish_norm)
 };
 
 __device__ inline uint4 ldg16(const bf16_t* p) { return *reinterpret_cast<const uint4*>(p); }
@@ -946,12 +948,12 @@ __global__ __launch_bounds__(256) void k_gemm_finish(GemmArgs g) {
 }
 
 // The same for a product that adds into the 32-bit residual stream and is followed by an
-// RMSNorm: a workgroup takes a whole row, so it can also sum the squares of the updated row
+// RMSNorm or a layer norm: a workgroup takes a whole row, so it can also sum the squares of the updated row
 // (threads, then waves, in a fixed order) and write the normed row, times the norm's weight,
 // to xg.  N is a multiple of 4.
 __global__ __launch_bounds__(1024) void k_gemm_finish_norm(GemmArgs g) {
     __shared__ float wave_sq[16];
-    __shared__ float rstd_s;
+    __shared__ float rstd_s, mean_s;
     const int m = blockIdx.x, tid = threadIdx.x;
     const size_t step = (size_t)g.M * g.N;
     float* xrow = (float*)g.out + (size_t)m * g.ldo;
@@ -971,12 +973,32 @@ __global__ __launch_bounds__(1024) void k_gemm_finish_norm(GemmArgs g) {
         float4 x = *reinterpret_cast<const float4*>(xrow + n);
         x.x += v.x; x.y += v.y; x.z += v.z; x.w += v.w;
         *reinterpret_cast<float4*>(xrow + n) = x;
-        sq += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+        sq += g.norm_centred ? x.x + x.y + x.z + x.w : x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
     }
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) sq += __shfl_xor(sq, o);
     if ((tid & 63) == 0) wave_sq[tid >> 6] = sq;
     __syncthreads();
+    float mean = 0.f;
+    if (g.norm_centred) {               // that was the row's sum: the squares of what lies beside the mean follow
+        if (tid == 0) {
+            float t = 0.f;
+            for (int w = 0; w < 16; ++w) t += wave_sq[w];
+            mean_s = t * g.ss_inv_width;
+        }
+        __syncthreads();
+        mean = mean_s;
+        sq = 0.f;
+        for (int n = tid * 4; n < g.N; n += 1024 * 4) {
+            const float4 x = *reinterpret_cast<const float4*>(xrow + n);     // what this thread wrote above
+            const float a = x.x - mean, b = x.y - mean, c = x.z - mean, d = x.w - mean;
+            sq += a * a + b * b + c * c + d * d;
+        }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) sq += __shfl_xor(sq, o);
+        if ((tid & 63) == 0) wave_sq[tid >> 6] = sq;
+        __syncthreads();
+    }
     if (tid == 0) {
         float t = 0.f;
         for (int w = 0; w < 16; ++w) t += wave_sq[w];
@@ -991,8 +1013,8 @@ __global__ __launch_bounds__(1024) void k_gemm_finish_norm(GemmArgs g) {
         for (int i = 0; i < 4; ++i)
             w[i] = g.norm_w_bf16 ? bf16_to_f32(((const bf16_t*)g.norm_w)[n + i]) : ((const float*)g.norm_w)[n + i];
         uint2 o;
-        o.x = pack_bf16x2(x.x * rstd * w[0], x.y * rstd * w[1]);
-        o.y = pack_bf16x2(x.z * rstd * w[2], x.w * rstd * w[3]);
+        o.x = pack_bf16x2((x.x - mean) * rstd * w[0], (x.y - mean) * rstd * w[1]);
+        o.y = pack_bf16x2((x.z - mean) * rstd * w[2], (x.w - mean) * rstd * w[3]);
         *reinterpret_cast<uint2*>(g.xg + (size_t)m * g.N + n) = o;
     }
 }
@@ -1390,7 +1412,7 @@ extern "C" int xr_gemm_bf16(void* out, const void* a, const void* w, const float
     g.a = (const bf16_t*)a; g.w = (const bf16_t*)w; g.w_packed = w_packed ? 1 : 0; g.bias = bias; g.out = out;
     g.M = M; g.N = N; g.K = K; g.lda = lda; g.ldo = ldo; g.out_bf16 = out_dtype == XR_BF16; g.epi = epi; g.act = act; g.act_param = act_param;
     g.m_fast = 0; g.splits = 1; g.k_per_split = 0; g.partial = workspace; g.col0 = 0; g.col1 = N;
-    g.raw = 0; g.norm_whole = 0; g.vec_out = 0;
+    g.raw = 0; g.norm_whole = 0; g.norm_centred = 0; g.vec_out = 0;
     bool want_whole_norm = false;      // a norm after a product of more than 16 rows is asked for and possible
     g.ss_in = nullptr; g.n_ss = 0; g.ss_inv_width = 0.f; g.ss_eps = 0.f;
     g.norm_w = nullptr; g.norm_w_bf16 = 0; g.xg = nullptr; g.ss_out = nullptr;
@@ -1405,6 +1427,8 @@ extern "C" int xr_gemm_bf16(void* out, const void* a, const void* w, const float
             XR_REQUIRE(epi == EPI_ACCUM && norm->norm_w, "gemm: the norm after a product needs the accumulating epilogue and a weight");
             XR_REQUIRE(M > 16 || (norm->ss_out && norm->ss_out_rows >= (N + 15) / 16),
                        "gemm: room for %d partial sums of squares, %d needed", norm->ss_out ? norm->ss_out_rows : 0, (N + 15) / 16);
+            XR_REQUIRE(!norm->centred || M > 16, "gemm: a layer norm after a product of %d rows: from 17 rows on", M);
+            g.norm_centred = norm->centred ? 1 : 0;
             g.norm_w = norm->norm_w; g.norm_w_bf16 = norm->norm_w_bf16; g.xg = (bf16_t*)norm->xg; g.ss_out = norm->ss_out;
             if (M > 16) {
                 // The kernel that adds up the K ranges of a split product takes whole rows and writes the

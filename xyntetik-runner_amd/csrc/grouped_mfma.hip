@@ -13,7 +13,9 @@
 // operand, rows as the B operand: a lane then holds 4 consecutive output columns of one row) and
 // reads its fragments straight from memory, 16 bytes a lane; the four waves of a workgroup take
 // four neighbouring groups of weight rows and share the rows' fragments through the caches.
-// Epilogue: nothing, or relu squared.
+// Epilogue: nothing, relu squared, or (GATED) a gate of common.h: the weight matrix then has F gate rows before F up
+// rows, the rows a wave takes are half gate rows and half the up rows of the same outputs, so that a lane holds both
+// branches of an output, and the output has F columns.
 #include "common.h"
 
 typedef __bf16 gm_bf16x8 __attribute__((ext_vector_type(8)));
@@ -21,13 +23,16 @@ typedef float gm_f32x4 __attribute__((ext_vector_type(4)));
 
 #define GM_ACT_NONE 0
 #define GM_ACT_RELU2 1
+#define GM_ACT_GATED 2
 
 struct GroupedArgs {
     const bf16_t* a;
     const bf16_t* w;
     void* out;
     long long a_group_stride, w_group_stride, o_group_stride;
-    int lda, ldo, N, K, out_bf16, act;
+    int lda, ldo, N, K, out_bf16, act;      // N: output columns (GATED: half the weight's rows)
+    int gate;               // with GM_ACT_GATED: the gate's code and its number
+    float gate_param;
     // experts: tiles from the sort; heads: tile_group null, tiles_per_group tiles of every group
     const int* perm;
     const int* tile_group;
@@ -45,8 +50,9 @@ __device__ inline gm_bf16x8 gm_frag(const bf16_t* p, bool ok) {
     return c.b;
 }
 
-template <int MT, int RT>
+template <int MT, int RT, bool GATED>
 __global__ __launch_bounds__(256) void k_grouped_gemm(GroupedArgs g) {
+    constexpr int RO = GATED ? RT / 2 : RT;     // groups of 16 output columns a wave
     const int tile = blockIdx.x;
     int group, row0, rows;
     if (g.tile_group) {
@@ -61,7 +67,7 @@ __global__ __launch_bounds__(256) void k_grouped_gemm(GroupedArgs g) {
     }
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int l16 = lane & 15, lq = lane >> 4;
-    const int n0 = (blockIdx.y * 4 + wave) * (16 * RT);
+    const int n0 = (blockIdx.y * 4 + wave) * (16 * RO);
     if (n0 >= g.N) return;
 
     const bf16_t* ap[MT];
@@ -86,9 +92,9 @@ __global__ __launch_bounds__(256) void k_grouped_gemm(GroupedArgs g) {
     bool w_ok[RT];
 #pragma unroll
     for (int r = 0; r < RT; ++r) {
-        const int n = n0 + r * 16 + l16;
+        const int n = n0 + (r % RO) * 16 + l16;
         w_ok[r] = n < g.N;
-        wp[r] = g.w + (long long)group * g.w_group_stride + (long long)(w_ok[r] ? n : 0) * g.K;
+        wp[r] = g.w + (long long)group * g.w_group_stride + (long long)((w_ok[r] ? n : 0) + (r >= RO ? g.N : 0)) * g.K;
     }
     gm_f32x4 acc[RT][MT];
 #pragma unroll
@@ -121,13 +127,14 @@ __global__ __launch_bounds__(256) void k_grouped_gemm(GroupedArgs g) {
     for (int i = 0; i < MT; ++i) {
         if (!a_ok[i]) continue;
 #pragma unroll
-        for (int r = 0; r < RT; ++r) {
+        for (int r = 0; r < RO; ++r) {
             const int n = n0 + r * 16 + lq * 4;
             float v[4];
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 v[e] = acc[r][i][e];
-                if (g.act == GM_ACT_RELU2) { v[e] = fmaxf(v[e], 0.f); v[e] *= v[e]; }
+                if (GATED) v[e] = gate_value<true>(g.gate, g.gate_param, v[e], acc[RT - RO + r][i][e]);
+                else if (g.act == GM_ACT_RELU2) { v[e] = fmaxf(v[e], 0.f); v[e] *= v[e]; }
             }
             if (vec_out && n + 3 < g.N) {       // the lane's 4 columns in one store
                 if (g.out_bf16) {
@@ -158,8 +165,9 @@ __global__ __launch_bounds__(256) void k_grouped_gemm(GroupedArgs g) {
 #define GL_BM 128
 #define GL_KS 64
 #define GL_LD 72
-template <int RT>        // groups of 16 weight rows a wave: 4 (128 weight rows a workgroup) or 8 (256)
+template <int RT, bool GATED>        // groups of 16 weight rows a wave: 4 (128 weight rows a workgroup) or 8 (256)
 __global__ __launch_bounds__(256) void k_grouped_gemm_lds(GroupedArgs g) {
+    constexpr int RO = GATED ? RT / 2 : RT;       // groups of 16 output columns a wave
     constexpr int GL_BN = 32 * RT, WP = RT;       // weight rows a workgroup; 16-byte pieces of them a thread copies a slice
     __shared__ __attribute__((aligned(16))) bf16_t As[GL_BM * GL_LD];
     __shared__ __attribute__((aligned(16))) bf16_t Ws[GL_BN * GL_LD];
@@ -178,7 +186,7 @@ __global__ __launch_bounds__(256) void k_grouped_gemm_lds(GroupedArgs g) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int l16 = lane & 15, lq = lane >> 4;
     const int wm = wave & 1, wn = wave >> 1;
-    const int nb = blockIdx.y * GL_BN;
+    const int nb = blockIdx.y * (32 * RO);
 
     // what this thread copies of a slice: 4 pieces of 16 bytes of the rows and 4 of the weights;
     // piece j is row (tid / 8) + 32 j, columns (tid % 8) * 8 .. + 8 of the slice
@@ -195,9 +203,12 @@ __global__ __launch_bounds__(256) void k_grouped_gemm_lds(GroupedArgs g) {
     }
 #pragma unroll
     for (int j = 0; j < WP; ++j) {
-        const int n = nb + crow + 32 * j;
+        // row wr of the staged weights belongs to the waves wn = wr / (16 RT); of a wave's rows the last 16 (RT - RO) are up rows
+        const int wr = crow + 32 * j, in_wave = wr % (16 * RT);
+        const bool up = GATED && in_wave >= 16 * RO;
+        const int n = nb + (wr / (16 * RT)) * (16 * RO) + in_wave - (up ? 16 * RO : 0);
         w_on[j] = n < g.N;
-        w_src[j] = g.w + (long long)group * g.w_group_stride + (long long)(w_on[j] ? n : 0) * g.K + ccol;
+        w_src[j] = g.w + (long long)group * g.w_group_stride + (long long)((w_on[j] ? n : 0) + (up ? g.N : 0)) * g.K + ccol;
     }
     gm_f32x4 acc[RT][4];
 #pragma unroll
@@ -250,7 +261,7 @@ __global__ __launch_bounds__(256) void k_grouped_gemm_lds(GroupedArgs g) {
                     acc[r][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[r], af[i], acc[r][i], 0, 0, 0);
         }
     }
-    // acc[r][i][e]: output column nb + wn * 16 RT + r * 16 + 4 * (lane / 16) + e of the tile's row wm * 64 + i * 16 + lane % 16
+    // acc[r][i][e]: output column nb + wn * 16 RO + r * 16 + 4 * (lane / 16) + e of the tile's row wm * 64 + i * 16 + lane % 16
     const bool vec_out = g.ldo % 4 == 0 && g.o_group_stride % 4 == 0 && ((uintptr_t)g.out % 16) == 0;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -259,13 +270,14 @@ __global__ __launch_bounds__(256) void k_grouped_gemm_lds(GroupedArgs g) {
         const int p = g.perm ? g.perm[row0 + r_in_tile] : row0 + r_in_tile;
         const long long orow = (long long)p * g.ldo + (long long)group * g.o_group_stride;
 #pragma unroll
-        for (int r = 0; r < RT; ++r) {
-            const int n = nb + wn * 16 * RT + r * 16 + lq * 4;
+        for (int r = 0; r < RO; ++r) {
+            const int n = nb + wn * 16 * RO + r * 16 + lq * 4;
             float v[4];
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 v[e] = acc[r][i][e];
-                if (g.act == GM_ACT_RELU2) { v[e] = fmaxf(v[e], 0.f); v[e] *= v[e]; }
+                if (GATED) v[e] = gate_value<true>(g.gate, g.gate_param, v[e], acc[RT - RO + r][i][e]);
+                else if (g.act == GM_ACT_RELU2) { v[e] = fmaxf(v[e], 0.f); v[e] *= v[e]; }
             }
             if (vec_out && n + 3 < g.N) {
                 if (g.out_bf16) {
@@ -294,29 +306,35 @@ static int g_grouped_variant = 0;       // measurements only: 0 = choose; 1 = na
 static int g_grouped_bm = 0;            // measurements only: rows of an experts' tile (0 = choose; 64 or 128)
 extern "C" void xr_grouped_set_variant(int v, int bm) { g_grouped_variant = v; g_grouped_bm = (bm == 64 || bm == 128) ? bm : 0; }
 
-static int launch_grouped(const GroupedArgs& g, int n_tiles_max, int rows_a_tile, hipStream_t stream) {
-    bool wide = g.N >= 128 && rows_a_tile >= 64 && (long long)n_tiles_max * ((g.N + 255) / 256) >= 256;    // enough such workgroups for the chip
+template <bool GATED>
+static void launch_grouped_as(const GroupedArgs& g, int n_tiles_max, int rows_a_tile, hipStream_t stream) {
+    const int NW = GATED ? 2 * g.N : g.N;       // weight rows
+    bool wide = NW >= 128 && rows_a_tile >= 64 && (long long)n_tiles_max * ((NW + 255) / 256) >= 256;    // enough such workgroups for the chip
     if (g_grouped_variant == 1) wide = false;
     if (g_grouped_variant == 2) wide = rows_a_tile >= 64;
-    if (rows_a_tile == 128 && g.N >= 128 && g_grouped_variant != 1 && g_grouped_variant != 2) {     // operands through LDS
+    if (rows_a_tile == 128 && NW >= 128 && g_grouped_variant != 1 && g_grouped_variant != 2) {     // operands through LDS
         // (256 weight rows a workgroup, 64 x 128 results a wave, was measured slower: sort, both products and
         // the sum took 176 us against 126 for 4,096 rows over 16 experts of 1,024 x 2,048; it stays for measurements)
         const bool big = g_grouped_variant == 4;
         const int bn = big ? 256 : 128;
-        const dim3 grid_lds(n_tiles_max, (g.N + bn - 1) / bn);
-        if (big) k_grouped_gemm_lds<8><<<grid_lds, 256, 0, stream>>>(g);
-        else k_grouped_gemm_lds<4><<<grid_lds, 256, 0, stream>>>(g);
-        return 0;
+        const dim3 grid_lds(n_tiles_max, (NW + bn - 1) / bn);
+        if (big) k_grouped_gemm_lds<8, GATED><<<grid_lds, 256, 0, stream>>>(g);
+        else k_grouped_gemm_lds<4, GATED><<<grid_lds, 256, 0, stream>>>(g);
+        return;
     }
     const int per_wg = wide ? 256 : 128;                    // 4 waves x 4 or 2 groups of 16 weight rows
-    const dim3 grid(n_tiles_max, (g.N + per_wg - 1) / per_wg);
-    if (rows_a_tile == 16) k_grouped_gemm<1, 2><<<grid, 256, 0, stream>>>(g);
-    else if (rows_a_tile == 32) k_grouped_gemm<2, 2><<<grid, 256, 0, stream>>>(g);
-    else if (rows_a_tile == 64 && !wide) k_grouped_gemm<4, 2><<<grid, 256, 0, stream>>>(g);
-    else if (rows_a_tile == 64) k_grouped_gemm<4, 4><<<grid, 256, 0, stream>>>(g);
-    else if (!wide) k_grouped_gemm<8, 2><<<grid, 256, 0, stream>>>(g);
-    else k_grouped_gemm<8, 4><<<grid, 256, 0, stream>>>(g);
-    return 0;
+    const dim3 grid(n_tiles_max, (NW + per_wg - 1) / per_wg);
+    if (rows_a_tile == 16) k_grouped_gemm<1, 2, GATED><<<grid, 256, 0, stream>>>(g);
+    else if (rows_a_tile == 32) k_grouped_gemm<2, 2, GATED><<<grid, 256, 0, stream>>>(g);
+    else if (rows_a_tile == 64 && !wide) k_grouped_gemm<4, 2, GATED><<<grid, 256, 0, stream>>>(g);
+    else if (rows_a_tile == 64) k_grouped_gemm<4, 4, GATED><<<grid, 256, 0, stream>>>(g);
+    else if (!wide) k_grouped_gemm<8, 2, GATED><<<grid, 256, 0, stream>>>(g);
+    else k_grouped_gemm<8, 4, GATED><<<grid, 256, 0, stream>>>(g);
+}
+
+static void launch_grouped(const GroupedArgs& g, int n_tiles_max, int rows_a_tile, hipStream_t stream) {
+    if (g.act == GM_ACT_GATED) launch_grouped_as<true>(g, n_tiles_max, rows_a_tile, stream);
+    else launch_grouped_as<false>(g, n_tiles_max, rows_a_tile, stream);
 }
 
 static bool grouped_operands_ok(const void* a, const void* w, int K, int lda, long long a_gs, long long w_gs) {
@@ -378,40 +396,135 @@ __global__ __launch_bounds__(1024) void k_moe_sort(const int* __restrict__ idx, 
 }
 
 // y[t] (+)= sum_j wts[t][j] * yz[t * top + j], in the order of the choice  (+ g_side[t] * y_side[t])
-__global__ void k_moe_combine(float* __restrict__ y, const float* __restrict__ yz, const float* __restrict__ wts, int E, int ld_y,
-                              int top, size_t n, int accumulate, const float* __restrict__ y_side,
-                              const float* __restrict__ g_side) {
+struct CombineArgs {
+    float* y;
+    const float* yz;
+    const float* wts;
+    int E, ld_y, top, accumulate;
+    const float* y_side;    // [T, E], or null
+    const float* g_side;    // [T]
+    // the norm of the finished row (k_moe_combine_norm): times w, to h [T, E]
+    const void* norm_w;
+    int norm_w_bf16, centred;
+    float eps;
+    bf16_t* h;
+};
+__global__ void k_moe_combine(CombineArgs a, size_t n) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
-    const size_t t = i / E;
-    const int c = (int)(i - t * E);
+    const size_t t = i / a.E;
+    const int c = (int)(i - t * a.E);
     float s = 0.f;
-    for (int j = 0; j < top; ++j) s += wts[t * top + j] * yz[(t * top + j) * E + c];
-    if (y_side) s = fmaf(g_side[t], y_side[i], s);
-    float* o = y + t * ld_y + c;
-    *o = accumulate ? *o + s : s;
+    for (int j = 0; j < a.top; ++j) s += a.wts[t * a.top + j] * a.yz[(t * a.top + j) * a.E + c];
+    if (a.y_side) s = fmaf(a.g_side[t], a.y_side[i], s);
+    float* o = a.y + t * a.ld_y + c;
+    *o = a.accumulate ? *o + s : s;
 }
+
+// The same with 4 columns a thread, a workgroup a row, and behind it, if asked for, the RMS or layer norm (`centred`) of
+// the row as it then stands, which the workgroup holds in registers (NV float4 a thread).
+__device__ inline float combine_block_sum(float v, float* part) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return part[0] + part[1] + part[2] + part[3];
+}
+template <int NV>
+__global__ __launch_bounds__(256) void k_moe_combine_norm(CombineArgs a) {
+    __shared__ float part[4];
+    const size_t t = blockIdx.x;
+    const int n4 = a.E >> 2;
+    float4 v[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    for (int j = 0; j < a.top; ++j) {
+        const float w = a.wts[t * a.top + j];
+        const float4* r = reinterpret_cast<const float4*>(a.yz + (t * a.top + j) * a.E);
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int c = threadIdx.x + i * 256;
+            if (c >= n4) continue;
+            const float4 x = r[c];
+            v[i].x += w * x.x; v[i].y += w * x.y; v[i].z += w * x.z; v[i].w += w * x.w;
+        }
+    }
+    float4* y = reinterpret_cast<float4*>(a.y + t * a.ld_y);
+    const float gs = a.y_side ? a.g_side[t] : 0.f;
+    const float4* side = reinterpret_cast<const float4*>(a.y_side + (a.y_side ? t * a.E : 0));
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = threadIdx.x + i * 256;
+        if (c >= n4) continue;
+        if (a.y_side) {
+            const float4 x = side[c];
+            v[i].x = fmaf(gs, x.x, v[i].x); v[i].y = fmaf(gs, x.y, v[i].y); v[i].z = fmaf(gs, x.z, v[i].z); v[i].w = fmaf(gs, x.w, v[i].w);
+        }
+        if (a.accumulate) {
+            const float4 x = y[c];
+            v[i].x += x.x; v[i].y += x.y; v[i].z += x.z; v[i].w += x.w;
+        }
+        y[c] = v[i];
+        s += a.centred ? v[i].x + v[i].y + v[i].z + v[i].w : v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+    }
+    if (!a.h) return;
+    float ss = combine_block_sum(s, part);
+    if (a.centred) {
+        const float mean = ss / (float)a.E;
+        s = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            if (threadIdx.x + i * 256 >= n4) continue;
+            v[i].x -= mean; v[i].y -= mean; v[i].z -= mean; v[i].w -= mean;
+            s += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+        }
+        ss = combine_block_sum(s, part);
+    }
+    const float rinv = 1.0f / sqrtf(ss / (float)a.E + a.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = threadIdx.x + i * 256;
+        if (c >= n4) continue;
+        float w[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) w[e] = a.norm_w_bf16 ? bf16_to_f32(((const bf16_t*)a.norm_w)[4 * c + e]) : ((const float*)a.norm_w)[4 * c + e];
+        *reinterpret_cast<uint2*>(a.h + t * a.E + 4 * c) = make_uint2(pack_bf16x2(v[i].x * rinv * w[0], v[i].y * rinv * w[1]),
+                                                                     pack_bf16x2(v[i].z * rinv * w[2], v[i].w * rinv * w[3]));
+    }
+}
+#define COMBINE_MAX_E (4 * 256 * 8)
 
 // The routed experts over many rows: sort, z = relu(up)^2 by expert, yz = down by expert, y = the weighted sum.
 // scratch: ints [A + 3 * (ceil(A / 16) + n) + 1]; z: bf16 [A, F]; yz: float [A, E].
-// Gated experts (`gu` given: float [A, 2F]; w_up [n, 2F, E], an expert's gate rows before its up rows): the first
-// product leaves both branches in 32 bits and the gate's own kernel makes z of them (`gate`: its code, `param` its number).
+// Gated experts (`gated`; w_up [n, 2F, E], an expert's gate rows before its up rows): the first product applies the gate
+// (its code `gate`, its number `param`) to its own two branches.
 // y_side / g_side: rows [T, E] that enter the sum with one weight a row, or null.
-extern "C" int xr_gate_mul(void* out, const void* gu, int T, int F, int ld_gu, int dtype, int out_dtype, int act, float param,
-                           hipStream_t stream);
+// `norm` given: the norm of the updated rows y goes to norm->h (with its weight and eps); widths up to COMBINE_MAX_E that
+// are multiples of 4.
+struct XrRowNorm {
+    const void* w;
+    int w_bf16, centred;
+    float eps;
+    void* h;
+};
 extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch, const void* h, const void* w_up,
                                       const void* w_down, const int* idx, const float* wts, int T, int E, int F, int ld_h,
-                                      int ld_y, int n, int top, int accumulate, float* gu, int gate, float param, const float* y_side,
-                                      const float* g_side, hipStream_t stream) {
+                                      int ld_y, int n, int top, int accumulate, int gated, int gate, float param, const float* y_side,
+                                      const float* g_side, const XrRowNorm* norm, hipStream_t stream) {
     XR_REQUIRE(gate >= 0 && gate < XR_ACT_COUNT, "moe_experts_grouped: unknown gate %d", gate);
     XR_REQUIRE(!y_side == !g_side, "moe_experts_grouped: rows beside the experts come with a weight a row");
     XR_REQUIRE(T >= 0 && E > 0 && F > 0 && ld_h >= E && ld_y >= E, "moe_experts_grouped: bad sizes T=%d E=%d F=%d", T, E, F);
     XR_REQUIRE(n >= 1 && n <= SORT_MAX_EXPERTS && top >= 1 && top <= n, "moe_experts_grouped: %d experts (at most %d), %d chosen", n,
                SORT_MAX_EXPERTS, top);
     XR_REQUIRE((long long)T * top <= (1 << 24), "moe_experts_grouped: too many rows");
-    const int Fu = gu ? 2 * F : F;          // rows of an expert's first matrix
+    const int Fu = gated ? 2 * F : F;          // rows of an expert's first matrix
     XR_REQUIRE(grouped_operands_ok(h, w_up, E, ld_h, 0, (long long)Fu * E) && grouped_operands_ok(z, w_down, F, F, 0, (long long)E * F),
                "moe_experts_grouped: widths and row strides must be multiples of 8 and the operands 16-byte aligned");
+    const bool rows4 = E % 4 == 0 && ld_y % 4 == 0 && E <= COMBINE_MAX_E && ((uintptr_t)y % 16) == 0 && ((uintptr_t)yz % 16) == 0 &&
+                       ((uintptr_t)y_side % 16) == 0;
+    XR_REQUIRE(!norm || (rows4 && norm->w && norm->h), "moe_experts_grouped: the norm behind the sum takes widths that are multiples of 4 up to %d, got %d",
+               COMBINE_MAX_E, E);
     if (T == 0) return XR_OK;
     const int A = T * top, avg = A / n;
     // rows of a tile: what an expert has on average, so that few rows do not idle most of a tile's lanes and the
@@ -429,19 +542,21 @@ extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch
     g.a_group_stride = 0; g.o_group_stride = 0;
     // up: rows of h by token, results by choice
     g.a = (const bf16_t*)h; g.lda = ld_h; g.w = (const bf16_t*)w_up; g.w_group_stride = (long long)Fu * E;
-    g.out = gu ? (void*)gu : z; g.ldo = Fu;
-    g.N = Fu; g.K = E; g.out_bf16 = gu ? 0 : 1; g.act = gu ? GM_ACT_NONE : GM_ACT_RELU2; g.gather_div = top;
+    g.out = z; g.ldo = F; g.N = F; g.K = E; g.out_bf16 = 1; g.act = gated ? GM_ACT_GATED : GM_ACT_RELU2; g.gate = gate; g.gate_param = param;
+    g.gather_div = top;
     launch_grouped(g, max_tiles, bm, stream);
-    if (gu) {
-        const int rc = xr_gate_mul(z, gu, A, F, 2 * F, XR_F32, XR_BF16, gate, param, stream);
-        if (rc != XR_OK) return rc;
-    }
     // down: rows of z by choice, results by choice
     g.a = (const bf16_t*)z; g.lda = F; g.w = (const bf16_t*)w_down; g.w_group_stride = (long long)E * F; g.out = yz; g.ldo = E;
     g.N = E; g.K = F; g.out_bf16 = 0; g.act = GM_ACT_NONE; g.gather_div = 1;
     launch_grouped(g, max_tiles, bm, stream);
-    const size_t cnt = (size_t)T * E;
-    k_moe_combine<<<(unsigned)((cnt + 255) / 256), 256, 0, stream>>>(y, yz, wts, E, ld_y, top, cnt, accumulate, y_side, g_side);
+    CombineArgs c{y, yz, wts, E, ld_y, top, accumulate, y_side, g_side, nullptr, 0, 0, 0.f, nullptr};
+    if (norm) { c.norm_w = norm->w; c.norm_w_bf16 = norm->w_bf16; c.centred = norm->centred; c.eps = norm->eps; c.h = (bf16_t*)norm->h; }
+    if (!rows4) {
+        const size_t cnt = (size_t)T * E;
+        k_moe_combine<<<(unsigned)((cnt + 255) / 256), 256, 0, stream>>>(c, cnt);
+    } else if (E <= 4 * 256 * 2) k_moe_combine_norm<2><<<T, 256, 0, stream>>>(c);
+    else if (E <= 4 * 256 * 4) k_moe_combine_norm<4><<<T, 256, 0, stream>>>(c);
+    else k_moe_combine_norm<8><<<T, 256, 0, stream>>>(c);
     XR_CHECK_LAUNCH("moe_experts_grouped");
     return XR_OK;
 }

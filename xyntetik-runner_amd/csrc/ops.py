@@ -57,6 +57,7 @@ _PROTOS = {
     "xr_embedding": [_p, _p, _p, _i, _i, _i, _f, _i, _i, _p],
     "xr_rmsnorm": [_p, _p, _p, _p, _i, _i, _i, _f, _i, _i, _p],
     "xr_rope_kv_write": [_p, _p, _p, _i, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p],
+    "xr_row_norm_rope_write": [_p, _p, _p, _i, _p, _p, _f, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p],
     "xr_gate_mul": [_p, _p, _i, _i, _i, _i, _i, _i, _f, _p],
     "xr_add": [_p, _p, _sz, _i, _f, _p],
     "xr_fill_rows": [_p, _p, _i, _sz, _u32, _p],
@@ -92,7 +93,7 @@ _PROTOS = {
     "xr_streams_step": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _f, _i, _p],
     "xr_latent_prepare": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p],
     "xr_moe_route": [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _p],
-    "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p, _i, _f, _p, _p, _p],
+    "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p, _p],
     "xr_heads_gemm_bf16": [_p, _p, _p, _i, _i, _i, _i, _i, C.c_longlong, _i, C.c_longlong, _i, _p],
     "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p],
     "xr_delta_prepare": [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _p],
@@ -171,7 +172,12 @@ class UnscaledRows:
 class _GemmNorm(C.Structure):
     """XrGemmNorm of the library."""
     _fields_ = [("ss_in", _p), ("n_ss", _i), ("ss_inv_width", _f), ("ss_eps", _f), ("norm_w", _p),
-                ("norm_w_bf16", _i), ("xg", _p), ("ss_out", _p), ("ss_out_rows", _i)]
+                ("norm_w_bf16", _i), ("xg", _p), ("ss_out", _p), ("ss_out_rows", _i), ("centred", _i)]
+
+
+class _RowNorm(C.Structure):
+    """XrRowNorm of the library."""
+    _fields_ = [("w", _p), ("w_bf16", _i), ("centred", _i), ("eps", _f), ("h", _p)]
 
 
 class _GemmRope(C.Structure):
@@ -439,8 +445,10 @@ class Ops:
         return norm, a.data
 
     def linear_add_rmsnorm(self, a, w, residual: torch.Tensor, norm_weight: Optional[torch.Tensor], eps: float,
-                           out_dtype: torch.dtype, bias: Optional[torch.Tensor] = None, defer: bool = False):
-        """``residual += a @ w^T (+ bias)``, then the RMSNorm of the updated rows.
+                           out_dtype: torch.dtype, bias: Optional[torch.Tensor] = None, defer: bool = False,
+                           centred: bool = False):
+        """``residual += a @ w^T (+ bias)``, then the RMSNorm of the updated rows (``centred``: the layer norm, whose
+        weight is 32-bit; it is never deferred).
 
         With ``defer`` the caller says that what reads the result is a ``linear`` or
         ``linear_gated``: for at most 16 bfloat16 rows the product's kernel then also writes the
@@ -455,7 +463,8 @@ class Ops:
         fits = (self.fold_norms and out_dtype == torch.bfloat16 and norm_weight is not None
                 and N % 8 == 0 and norm_weight.numel() == N and norm_weight.is_contiguous()
                 and residual.dtype == torch.float32 and self._mfma_ok(rows, wt))
-        deferred = fits and defer and M <= UnscaledRows.MAX_ROWS
+        deferred = fits and defer and M <= UnscaledRows.MAX_ROWS and not centred
+        normed = self.layernorm if centred else self.rmsnorm
         # More rows: where the product is split over K (always from 17 to 64 rows, above that when
         # its tiles are too few for the chip), the kernel that adds the parts up takes whole rows and
         # writes the finished norm; the library says whether it did.
@@ -468,15 +477,15 @@ class Ops:
             sumsq = torch.empty((parts, 16), dtype=torch.float32, device=rows.device) if deferred else None
             then.norm_w, then.norm_w_bf16 = norm_weight.data_ptr(), dtype_code(norm_weight.dtype)
             then.xg, then.ss_out, then.ss_out_rows = xg.data_ptr(), _ptr(sumsq), parts
-            then.ss_inv_width, then.ss_eps = 1.0 / N, float(eps)
+            then.ss_inv_width, then.ss_eps, then.centred = 1.0 / N, float(eps), 1 if centred else 0
             self.linear(a, w, bias=bias, out=residual, accumulate=True, _then=then)
             if then.ss_out_rows < 0:
                 return xg                                   # the finished norm
             if deferred:
                 return UnscaledRows(xg, sumsq[:then.ss_out_rows], eps)
-            return self.rmsnorm(residual, norm_weight, eps, out_dtype)      # the library declined
+            return normed(residual, norm_weight, eps, out_dtype)            # the library declined
         self.linear(a, w, bias=bias, out=residual, accumulate=True)
-        return self.rmsnorm(residual, norm_weight, eps, out_dtype)
+        return normed(residual, norm_weight, eps, out_dtype)
 
     def linear_gated(self, a: torch.Tensor, w, bias: Optional[torch.Tensor] = None, activation: str = "silu",
                      variant: int = 0, param: float = 0.0) -> torch.Tensor:
@@ -543,6 +552,37 @@ class Ops:
             block_table.stride(0) if block_table is not None else 0, _ptr(inv_freq), T, H, Hk, D, rot,
             1 if interleaved else 0, float(mscale), page_size, dtype_code(store.dtype), 1 if paired else 0,
             _stream()))
+
+    def row_norm_rope_write(self, q_in, k_in, v_in, w_q, w_k, eps: float, k_cache, v_cache, ctx, group: int, inv_freq, H: int,
+                            Hk: int, D: int, rot: int, interleaved: bool, mscale: float, page_size: int, out_dtype) -> torch.Tensor:
+        """Queries and keys over the root mean square of all their heads together (eps inside the root) times ``w_q [H * D]``
+        and ``w_k [Hk * D]``, then rotated; queries come back ``[T, H * D]`` in ``out_dtype``, keys and the values ``v_in`` (which
+        may be ``k_in``: the keys as projected) go to their pages.  Inputs are 32-bit views with one row stride; ``k_in`` None:
+        queries alone."""
+        self._dev(q_in, k_in, v_in, w_q, w_k, k_cache, v_cache, inv_freq)
+        views = [t for t in (q_in, k_in, v_in) if t is not None]
+        T = q_in.shape[0]
+        if any(t.dtype != torch.float32 or t.stride(1) != 1 for t in views) or (T > 1 and len({t.stride(0) for t in views}) != 1):
+            raise KernelError("row_norm_rope_write: q, k and v must be float32 views with one row stride")
+        Hk = Hk if k_in is not None else 0
+        if tuple(q_in.shape) != (T, H * D) or any(tuple(t.shape) != (T, Hk * D) for t in views[1:]) or (k_in is None) != (v_in is None):
+            raise KernelError("row_norm_rope_write: view widths do not fit the heads")
+        for w, n in ((w_q, H * D), (w_k, Hk * D)):
+            if n and (w is None or w.dtype != torch.float32 or w.numel() != n or not w.is_contiguous()):
+                raise KernelError(f"row_norm_rope_write: a weight must be float32 [{n}]")
+        if Hk and (k_cache.dtype != out_dtype or v_cache.dtype != out_dtype or tuple(k_cache.shape[1:]) != (Hk, page_size, D)
+                   or tuple(v_cache.shape[1:]) != (Hk, D, page_size)):
+            raise KernelError("row_norm_rope_write: the cache does not fit the heads")
+        if rot and (inv_freq is None or inv_freq.dtype != torch.float32 or inv_freq.numel() != rot // 2):
+            raise KernelError(f"row_norm_rope_write: {rot // 2} 32-bit frequencies are needed")
+        table = ctx.block_table(group)
+        q = torch.empty((T, H * D), dtype=out_dtype, device=q_in.device)
+        self.lib.check(self.lib.xr_row_norm_rope_write(
+            q_in.data_ptr(), _ptr(k_in), _ptr(v_in), q_in.stride(0), w_q.data_ptr(), _ptr(w_k) if Hk else None, float(eps), q.data_ptr(),
+            _ptr(k_cache) if Hk else None, _ptr(v_cache) if Hk else None, ctx.positions.data_ptr(), ctx.req_of_token.data_ptr(),
+            table.data_ptr(), table.stride(0), _ptr(inv_freq), T, H, Hk, D, int(rot), 1 if interleaved else 0, float(mscale),
+            page_size, dtype_code(out_dtype), _stream()))
+        return q
 
     def rope_table(self, positions: torch.Tensor, inv_freq: torch.Tensor, mscale: float = 1.0) -> torch.Tensor:
         """``[T, rot/2, 2]`` float32: cosine and sine (times ``mscale``) of every row's angles, as
@@ -1169,15 +1209,17 @@ class Ops:
 
     def moe_experts(self, h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor,
                     out: Optional[torch.Tensor] = None, accumulate: bool = False, activation: str = "relu2", param: float = 0.0,
-                    beside=None) -> torch.Tensor:
+                    beside=None, norm=None):
         """``out[t] (+)= sum_j wts[t, j] * w_down[e] @ relu(w_up[e] @ h[t])^2`` with ``e = idx[t, j]``, as 32-bit
         rows; ``w_up [n, F, E]`` and ``w_down [n, E, F]`` in ``h``'s dtype.  ``activation`` "swiglu": gated experts,
         ``w_down[e] @ (silu(g) * u)`` with ``[g; u] = w_up[e] @ h[t]`` for ``w_up [n, 2F, E]`` (an expert's gate rows
         before its up rows); "clamped_swish" and "gelu_tanh" likewise with that gate (its number ``param``).  ``beside`` =
-        (32-bit rows ``[T, E]``, one weight a row ``[T]``): these rows enter the sum too.  A few choices stream the chosen
+        (32-bit rows ``[T, E]``, one weight a row ``[T]``): these rows enter the sum too.  ``norm`` = (weight, eps,
+        centred), the norm of the updated rows (an RMS norm, or with ``centred`` the layer norm with a 32-bit weight): its
+        result in ``h``'s dtype comes back instead of the rows.  A few choices stream the chosen
         experts' weights, a wave an output column; from ``GROUPED_EXPERTS_FROM`` choices on (bfloat16, widths
         that are multiples of 8) the rows are sorted by expert on the device, both products run on the matrix
-        cores and a last kernel adds a token's experts up in the order of its choice."""
+        cores and a last kernel adds a token's experts up in the order of its choice (and writes the norm)."""
         self._dev(h, w_up, w_down, idx, wts, out)
         T, E = h.shape
         if activation not in EXPERT_ACTIVATIONS:
@@ -1212,18 +1254,28 @@ class Ops:
             A = T * top
             yz = torch.empty((A, E), dtype=torch.float32, device=h.device)
             scratch = torch.empty((A + 3 * (-(-A // 16) + n) + 1,), dtype=torch.int32, device=h.device)
-            gu = torch.empty((A, 2 * F), dtype=torch.float32, device=h.device) if gated else None
+            rn = normed = None
+            if norm is not None and E % 4 == 0 and E <= 8192 and out.stride(0) % 4 == 0 and out.data_ptr() % 16 == 0:
+                self._dev(norm[0])
+                normed = torch.empty((T, E), dtype=h.dtype, device=h.device)
+                rn = _RowNorm(norm[0].data_ptr(), dtype_code(norm[0].dtype), 1 if norm[2] else 0, float(norm[1]), normed.data_ptr())
             self.lib.check(self.lib.xr_moe_experts_grouped(out.data_ptr(), z.data_ptr(), yz.data_ptr(), scratch.data_ptr(),
                                                            h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(), idx.data_ptr(),
                                                            wts.data_ptr(), T, E, F, h.stride(0), out.stride(0), n, top,
-                                                           1 if accumulate else 0, _ptr(gu), gate, float(param), _ptr(y_beside),
-                                                           _ptr(g_beside), _stream()))
-            return out
+                                                           1 if accumulate else 0, form, gate, float(param), _ptr(y_beside),
+                                                           _ptr(g_beside), C.addressof(rn) if rn is not None else None, _stream()))
+            return normed if normed is not None else self._then_norm(out, norm, h.dtype)
         self.lib.check(self.lib.xr_moe_experts(out.data_ptr(), z.data_ptr(), h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(),
                                                idx.data_ptr(), wts.data_ptr(), T, E, F, h.stride(0), out.stride(0), n, top,
                                                1 if accumulate else 0, dtype_code(h.dtype), form, gate, float(param),
                                                _ptr(y_beside), _ptr(g_beside), _stream()))
-        return out
+        return self._then_norm(out, norm, h.dtype)
+
+    def _then_norm(self, rows: torch.Tensor, norm, dtype: torch.dtype):
+        """``rows``, or their norm (weight, eps, centred) by its own kernel."""
+        if norm is None:
+            return rows
+        return (self.layernorm if norm[2] else self.rmsnorm)(rows, norm[0], norm[1], dtype)
 
     def delta_prepare_(self, q, k, b, a, a_log, dt_bias, G: int, H: int, D: int, q_scale: float, unit_eps: float) -> None:
         """In place on 32-bit views (``q`` and ``k`` with one row stride, ``b`` and ``a`` with one):

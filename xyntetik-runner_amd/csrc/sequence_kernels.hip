@@ -45,6 +45,51 @@ __global__ __launch_bounds__(64 * NW) void k_layernorm(TO* __restrict__ out, con
     for (int i = threadIdx.x; i < E; i += 64 * NW) st<TO>(o, i, (xr[i] - mean) * rinv * (w ? w[i] : 1.f));
 }
 
+// Rows whose width is a multiple of 4 (up to 4 * 64 NW * NV): a thread keeps its float4 pieces in registers from the sum
+// to the scaling, so that a row is read once.
+template <typename TO> __device__ inline void ln_put4(TO* p, float a, float b, float c, float d);
+template <> __device__ inline void ln_put4<float>(float* p, float a, float b, float c, float d) {
+    *reinterpret_cast<float4*>(p) = make_float4(a, b, c, d);
+}
+template <> __device__ inline void ln_put4<bf16_t>(bf16_t* p, float a, float b, float c, float d) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(c, d));
+}
+template <typename TO, int NW, int NV>
+__global__ __launch_bounds__(64 * NW) void k_layernorm_v4(TO* __restrict__ out, const float* __restrict__ x,
+                                                         const float* __restrict__ w, const int* __restrict__ rows,
+                                                         int E, int ldx, float eps) {
+    __shared__ float part[NW];
+    const int r = blockIdx.x;
+    const int src = rows ? rows[r] : r;
+    const float4* xr = reinterpret_cast<const float4*>(x + (size_t)src * ldx);
+    const float4* w4 = reinterpret_cast<const float4*>(w);
+    const int n4 = E >> 2;
+    float4 v[NV], g[NV];
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = threadIdx.x + i * 64 * NW;
+        v[i] = c < n4 ? xr[c] : make_float4(0.f, 0.f, 0.f, 0.f);
+        g[i] = (w && c < n4) ? w4[c] : make_float4(1.f, 1.f, 1.f, 1.f);
+        s += v[i].x + v[i].y + v[i].z + v[i].w;
+    }
+    const float mean = block_sum<NW>(s, part) / (float)E;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        if (threadIdx.x + i * 64 * NW >= n4) continue;
+        v[i].x -= mean; v[i].y -= mean; v[i].z -= mean; v[i].w -= mean;
+        ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+    }
+    const float rinv = 1.0f / sqrtf(block_sum<NW>(ss, part) / (float)E + eps);
+    TO* o = out + (size_t)r * E;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = threadIdx.x + i * 64 * NW;
+        if (c < n4) ln_put4<TO>(o + 4 * c, v[i].x * rinv * g[i].x, v[i].y * rinv * g[i].y, v[i].z * rinv * g[i].z, v[i].w * rinv * g[i].w);
+    }
+}
+
 extern "C" int xr_layernorm(void* out, const float* x, const float* w, const int* rows, int R, int E, int ldx,
                             float eps, int out_dtype, hipStream_t stream) {
     XR_REQUIRE(R >= 0 && E > 0 && ldx >= E, "layernorm: bad sizes R=%d E=%d ldx=%d", R, E, ldx);
@@ -52,7 +97,21 @@ extern "C" int xr_layernorm(void* out, const float* x, const float* w, const int
     XR_REQUIRE(out_dtype == XR_F32 || out_dtype == XR_BF16, "layernorm: bad dtype %d", out_dtype);
     if (R == 0) return XR_OK;
     const bool few = R <= FEW_ROWS && E >= 1024;
-    if (out_dtype == XR_F32) {
+    const bool vec = E % 4 == 0 && ldx % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)w % 16) == 0 &&
+                     E <= 4 * 256 * 8;
+    if (vec) {
+#define LN(TO)                                                                                                        \
+    do {                                                                                                              \
+        if (few && E <= 4096) k_layernorm_v4<TO, 16, 1><<<R, 1024, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps);    \
+        else if (few) k_layernorm_v4<TO, 16, 2><<<R, 1024, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps);            \
+        else if (E <= 4 * 256 * 2) k_layernorm_v4<TO, 4, 2><<<R, 256, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps); \
+        else if (E <= 4 * 256 * 4) k_layernorm_v4<TO, 4, 4><<<R, 256, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps); \
+        else k_layernorm_v4<TO, 4, 8><<<R, 256, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps);                       \
+    } while (0)
+        if (out_dtype == XR_F32) LN(float);
+        else LN(bf16_t);
+#undef LN
+    } else if (out_dtype == XR_F32) {
         if (few) k_layernorm<float, 16><<<R, 1024, 0, stream>>>((float*)out, x, w, rows, E, ldx, eps);
         else k_layernorm<float, 4><<<R, 256, 0, stream>>>((float*)out, x, w, rows, E, ldx, eps);
     } else {

@@ -31,7 +31,7 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import KVSpec, Mixer, ParamSpec, make_part, register_mixer
+from .base import KVSpec, Mixer, ParamSpec, PositionEncoding, make_part, register_mixer
 
 MAX_HEAD_DIM = 256      # the attention and rotation kernels keep a head's channels in registers up to this size
 
@@ -92,6 +92,10 @@ class PagedAttention(Mixer):
         # applied to the 32-bit projections before the position encoding; with one, the projections
         # are written out and the kernels that rotate and cache their own result are not used
         self.qk_transform = make_part("qk_transform", qk_transform) if qk_transform is not None else None
+        # a norm over all heads of a row that the rotation-and-cache kernel applies itself; that kernel takes the values from
+        # any rows, so keys that are the values stand once in the input matrix
+        self.row_normed = (self.qk_transform is not None and hasattr(self.qk_transform, "row_norm") and self.v_head_dim == self.head_dim
+                           and (self.position is None or type(self.position).rotary is not PositionEncoding.rotary))
         self.q_size = self.num_heads * self.head_dim
         self.kv_size = self.num_kv_heads * self.head_dim
         self.v_size = self.num_kv_heads * self.v_head_dim
@@ -146,18 +150,16 @@ class PagedAttention(Mixer):
         q, k, v, o = self.names
         H, Hk, D = self.num_heads, self.num_kv_heads, self.head_dim
         ws, bsf = self.w_sfx, self.b_sfx
-        if self.values_are_keys:        # the value projection is the key projection: its rows stand twice in the one matrix
-            v = k
-        mats = [tensors[f"{q}{ws}"]]
-        if not self.kv_shared:
-            mats += [tensors[f"{k}{ws}"], tensors[f"{v}{ws}"]]
+        # the value projection is the key projection: its rows stand twice in the one matrix, or once where the kernel
+        # behind the product takes both from the same columns
+        inputs = [q] if self.kv_shared else [q, k, k if self.values_are_keys else v]
+        if self.row_normed and self.values_are_keys and not self.kv_shared:
+            inputs = [q, k]
+        mats = [tensors[f"{n}{ws}"] for n in inputs]
         w_in = torch.cat(mats, dim=0).contiguous() if len(mats) > 1 else mats[0]
         b_in = None
         if self.bias:
-            bs = [tensors[f"{q}{bsf}"]]
-            if not self.kv_shared:
-                bs += [tensors[f"{k}{bsf}"], tensors[f"{v}{bsf}"]]
-            b_in = torch.cat([b.float() for b in bs]).contiguous()
+            b_in = torch.cat([tensors[f"{n}{bsf}"].float() for n in inputs]).contiguous()
         if self.slope_values is not None:
             self.slopes = torch.tensor(self.slope_values, dtype=torch.float32, device=rt.device)
         if self.sink == "learned":
@@ -214,6 +216,15 @@ class PagedAttention(Mixer):
                 if writes:
                     ops.rotate_rows_(k_in, ctx.positions, rot.inv_freq, Hk, D, rot.rotary_dim, 1.0)
             q = ops.qkv_store(q_in, k_in, v_in, cache.k, cache.v, ctx, cache.group, H, Hk, D, Dv, cache.page_size, rt.dtype)
+        elif self.row_normed:
+            # norm over all heads, rotation and cache write in one kernel behind the product
+            proj = ops.linear(h, self.w_in, bias=self.b_in, out_dtype=torch.float32)
+            k_in = proj[:, Q:Q + K] if writes else None
+            v_in = k_in if self.values_are_keys or not writes else proj[:, Q + K:Q + 2 * K]
+            w_q, w_k, eps = self.qk_transform.row_norm()
+            q = ops.row_norm_rope_write(proj[:, :Q], k_in, v_in, w_q, w_k, eps, cache.k, cache.v, ctx, cache.group,
+                                        rot.inv_freq if rot else None, H, Hk, D, rot.rotary_dim if rot else 0,
+                                        rot.interleaved if rot else False, rot.mscale if rot else 1.0, cache.page_size, rt.dtype)
         elif (self.position is None or rot is not None) and writes == (not self.kv_shared) and self.qk_transform is None:
             q = ops.project_rope_kv_write(
                 h, self.w_in, self.b_in, cache.k if writes else None, cache.v if writes else None, ctx.positions,
@@ -266,11 +277,11 @@ class PagedAttention(Mixer):
         self.rt.ops.linear(self._attend(ctx, cache, h), self.w_out, bias=self.b_out, out=residual, accumulate=True)
 
     def forward_add_norm(self, ctx, cache, h, residual, norm, defer=False):
-        fold = norm.fold()
+        fold = norm.fold_row()
         if fold is None:
             return super().forward_add_norm(ctx, cache, h, residual, norm, defer)
         return self.rt.ops.linear_add_rmsnorm(self._attend(ctx, cache, h), self.w_out, residual, fold[0], fold[1],
-                                              self.rt.dtype, bias=self.b_out, defer=defer)
+                                              self.rt.dtype, bias=self.b_out, defer=defer, centred=fold[2])
 
 
 register_mixer("paged_attention", PagedAttention)

@@ -10,7 +10,8 @@ Families and what each must offer:
 * ``Norm``: ``forward(ctx, x, rows=None) -> h``.  ``x`` is the 32-bit residual
   stream ``[T, E]``; ``h`` is in the compute dtype.  ``rows`` (device int32)
   selects rows of ``x``.  ``fold()`` may return ``(weight, eps)`` if the norm is an
-  RMSNorm that the product before it may compute (see below).
+  RMSNorm that the product before it may compute (see below), ``fold_row()`` the same for a
+  layer norm too, for kernels that hold whole rows.
 * ``PositionEncoding``: ``rotary()`` returns the parameters of a rotation that
   the attention kernels apply themselves, or ``None``; then ``apply(ctx, q, k)``
   is called on the 32-bit queries and keys before they are cached.
@@ -140,6 +141,13 @@ class Norm(Part):
         """``(weight, eps)`` if this is ``x / sqrt(mean(x^2) + eps) * weight``, which the product
         that writes ``x`` may compute in its own kernel; None for any other norm."""
         return None
+
+    def fold_row(self) -> Optional[Tuple[torch.Tensor, float, bool]]:
+        """``(weight, eps, centred)`` of a norm that a kernel which holds whole rows of ``x`` may compute: the one of
+        ``fold()``, or with ``centred`` the layer norm ``(x - mean) / sqrt(var + eps) * weight`` with a 32-bit weight and a
+        result in the compute dtype; None for any other norm."""
+        f = self.fold()
+        return (f[0], f[1], False) if f is not None else None
 
 
 @dataclass(frozen=True)

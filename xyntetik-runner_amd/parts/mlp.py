@@ -91,11 +91,11 @@ class GatedMLP(FeedForward):
         self.rt.ops.linear(self._hidden(ctx, h), self.w_down, bias=self.b_down, out=residual, accumulate=True)
 
     def forward_add_norm(self, ctx, h, residual, norm, defer=False):
-        fold = norm.fold()
+        fold = norm.fold_row()
         if fold is None:
             return super().forward_add_norm(ctx, h, residual, norm, defer)
         return self.rt.ops.linear_add_rmsnorm(self._hidden(ctx, h), self.w_down, residual, fold[0], fold[1],
-                                              self.rt.dtype, bias=self.b_down, defer=defer)
+                                              self.rt.dtype, bias=self.b_down, defer=defer, centred=fold[2])
 
 
 class DenseMLP(FeedForward):
@@ -234,7 +234,7 @@ class RoutedExperts(FeedForward):
         if self.shared is not None:
             self.shared.bind({name: tensors[name] for name in self.shared.param_specs()}, rt)
 
-    def _run(self, ctx, h, out=None, accumulate=False):
+    def _run(self, ctx, h, out=None, accumulate=False, norm=None):
         ops = self.rt.ops
         beside = None
         if self.routing == "table":
@@ -245,7 +245,7 @@ class RoutedExperts(FeedForward):
             idx, wts, gate = ops.moe_route(h, self.router, self.correction, self.top, side_gate=True, **self.how)
             beside = (self.shared.forward_f32(ctx, h), gate)
         out = ops.moe_experts(h, self.w_up, self.w_down, idx, wts, out=out, accumulate=accumulate, activation=self.activation,
-                              param=self.activation_param, beside=beside)
+                              param=self.activation_param, beside=beside, norm=norm)
         if self.shared is not None and beside is None:
             self.shared.forward_add(ctx, h, out)
         return out
@@ -258,6 +258,12 @@ class RoutedExperts(FeedForward):
 
     def forward_add(self, ctx, h, residual) -> None:
         self._run(ctx, h, out=residual, accumulate=True)
+
+    def forward_add_norm(self, ctx, h, residual, norm, defer=False):
+        fold = norm.fold_row()
+        if fold is None or (self.shared is not None and self.shared_gate_name is None):      # (a shared expert without a gate adds to the rows afterwards)
+            return super().forward_add_norm(ctx, h, residual, norm, defer)
+        return self._run(ctx, h, out=residual, accumulate=True, norm=fold)
 
 
 register_feed_forward("gated_mlp", GatedMLP)

@@ -63,6 +63,9 @@ class LayerNorm(Norm):
         dt = torch.float32 if self.out_dtype == "float32" else self.rt.dtype
         return self.rt.ops.layernorm(x, self.weight, self.eps, dt, rows=rows)
 
+    def fold_row(self):
+        return (self.weight, self.eps, True) if self.weight is not None and self.out_dtype == "compute" else None
+
 
 class DynamicTanh(Norm):
     """Tensors: the weight ``[size]`` under ``weight_name``, and beside it ``<weight_name>.b`` (the bias) and
