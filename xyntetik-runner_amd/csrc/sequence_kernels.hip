@@ -45,17 +45,11 @@ __global__ __launch_bounds__(64 * NW) void k_layernorm(TO* __restrict__ out, con
     for (int i = threadIdx.x; i < E; i += 64 * NW) st<TO>(o, i, (xr[i] - mean) * rinv * (w ? w[i] : 1.f));
 }
 
-// Rows whose width is a multiple of 4 (up to 4 * 64 NW * NV): a thread keeps its float4 pieces in registers from the sum
-// to the scaling, so that a row is read once.
-template <typename TO> __device__ inline void ln_put4(TO* p, float a, float b, float c, float d);
-template <> __device__ inline void ln_put4<float>(float* p, float a, float b, float c, float d) {
-    *reinterpret_cast<float4*>(p) = make_float4(a, b, c, d);
-}
-template <> __device__ inline void ln_put4<bf16_t>(bf16_t* p, float a, float b, float c, float d) {
-    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(c, d));
-}
-template <typename TO, int NW, int NV>
-__global__ __launch_bounds__(64 * NW) void k_layernorm_v4(TO* __restrict__ out, const float* __restrict__ x,
+// Rows whose width is a multiple of 4 (up to 4 * 64 NW * NV), to bfloat16: a thread keeps its float4 pieces in registers
+// from the sum to the scaling, so that a row is read once.  (32-bit rows stay with the kernel above: k_layernorm_conv sums
+// in its order, and a step of single rows must give the same bits with and without it.)
+template <int NW, int NV>
+__global__ __launch_bounds__(64 * NW) void k_layernorm_v4(bf16_t* __restrict__ out, const float* __restrict__ x,
                                                          const float* __restrict__ w, const int* __restrict__ rows,
                                                          int E, int ldx, float eps) {
     __shared__ float part[NW];
@@ -82,11 +76,13 @@ __global__ __launch_bounds__(64 * NW) void k_layernorm_v4(TO* __restrict__ out, 
         ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
     }
     const float rinv = 1.0f / sqrtf(block_sum<NW>(ss, part) / (float)E + eps);
-    TO* o = out + (size_t)r * E;
+    bf16_t* o = out + (size_t)r * E;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
         const int c = threadIdx.x + i * 64 * NW;
-        if (c < n4) ln_put4<TO>(o + 4 * c, v[i].x * rinv * g[i].x, v[i].y * rinv * g[i].y, v[i].z * rinv * g[i].z, v[i].w * rinv * g[i].w);
+        if (c < n4)
+            *reinterpret_cast<uint2*>(o + 4 * c) = make_uint2(pack_bf16x2(v[i].x * rinv * g[i].x, v[i].y * rinv * g[i].y),
+                                                              pack_bf16x2(v[i].z * rinv * g[i].z, v[i].w * rinv * g[i].w));
     }
 }
 
@@ -99,18 +95,13 @@ extern "C" int xr_layernorm(void* out, const float* x, const float* w, const int
     const bool few = R <= FEW_ROWS && E >= 1024;
     const bool vec = E % 4 == 0 && ldx % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)w % 16) == 0 &&
                      E <= 4 * 256 * 8;
-    if (vec) {
-#define LN(TO)                                                                                                        \
-    do {                                                                                                              \
-        if (few && E <= 4096) k_layernorm_v4<TO, 16, 1><<<R, 1024, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps);    \
-        else if (few) k_layernorm_v4<TO, 16, 2><<<R, 1024, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps);            \
-        else if (E <= 4 * 256 * 2) k_layernorm_v4<TO, 4, 2><<<R, 256, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps); \
-        else if (E <= 4 * 256 * 4) k_layernorm_v4<TO, 4, 4><<<R, 256, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps); \
-        else k_layernorm_v4<TO, 4, 8><<<R, 256, 0, stream>>>((TO*)out, x, w, rows, E, ldx, eps);                       \
-    } while (0)
-        if (out_dtype == XR_F32) LN(float);
-        else LN(bf16_t);
-#undef LN
+    if (vec && out_dtype == XR_BF16) {
+        bf16_t* o = (bf16_t*)out;
+        if (few && E <= 4096) k_layernorm_v4<16, 1><<<R, 1024, 0, stream>>>(o, x, w, rows, E, ldx, eps);
+        else if (few) k_layernorm_v4<16, 2><<<R, 1024, 0, stream>>>(o, x, w, rows, E, ldx, eps);
+        else if (E <= 4 * 256 * 2) k_layernorm_v4<4, 2><<<R, 256, 0, stream>>>(o, x, w, rows, E, ldx, eps);
+        else if (E <= 4 * 256 * 4) k_layernorm_v4<4, 4><<<R, 256, 0, stream>>>(o, x, w, rows, E, ldx, eps);
+        else k_layernorm_v4<4, 8><<<R, 256, 0, stream>>>(o, x, w, rows, E, ldx, eps);
     } else if (out_dtype == XR_F32) {
         if (few) k_layernorm<float, 16><<<R, 1024, 0, stream>>>((float*)out, x, w, rows, E, ldx, eps);
         else k_layernorm<float, 4><<<R, 256, 0, stream>>>((float*)out, x, w, rows, E, ldx, eps);
