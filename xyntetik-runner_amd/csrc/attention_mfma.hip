@@ -1,6 +1,7 @@
 // Paged grouped-query attention on the gfx950 matrix cores, bfloat16 storage, for prompt
 // portions and decoded tokens in one launch.  Compiled once per head size (XR_HEAD_DIM,
-// a multiple of 16 up to 256).
+// a multiple of 16 up to 256) and, where values are of another size than keys, per size of a value
+// (XR_VALUE_DIM, a multiple of 16 up to 256 too).
 //
 // The formulas are the reference's (src/model.c:3548-3589: scores (q.k)*scale
 // over the keys a position may see, softmax with the maximum taken out, weighted values;
@@ -39,10 +40,16 @@
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 
+#ifndef XR_VALUE_DIM
+#define XR_VALUE_DIM XR_HEAD_DIM
+#endif
+
 constexpr int HD = XR_HEAD_DIM;
+constexpr int HV = XR_VALUE_DIM;     // channels of a value, and of a head's output
 constexpr int KD = HD / 16;          // k-steps of the score product
-constexpr int DB = (HD + 31) / 32;   // 32-row blocks of O^T
+constexpr int DB = (HV + 31) / 32;   // 32-row blocks of O^T
 static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head size must be a multiple of 16 up to 256");
+static_assert(HV % 16 == 0 && HV >= 16 && HV <= 256, "value size must be a multiple of 16 up to 256");
 
 #define ITEM_INTS 8                   // req, row0, k_begin, k_end, slot (-1: final), q0, q_len, start
 #define ROWS 32
@@ -51,15 +58,15 @@ static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head size must be a multip
 struct AttnArgs {
     const bf16_t* q;        // [T, H, HD]
     const bf16_t* kc;       // [pages, Hk, page_size, HD]
-    const bf16_t* vc;       // [pages, Hk, HD, page_size]
-    bf16_t* out;            // [T, H, HD]
+    const bf16_t* vc;       // [pages, Hk, HV, page_size]
+    bf16_t* out;            // [T, H, HV], rows ld_out apart
     const int* items;       // [n_items, ITEM_INTS]; q0: the request's first row, start: its first position
     const int* cta_items;   // [n_cta_items, ITEM_INTS]: the same for 128-row blocks that a whole workgroup takes
     const int* cu_q;        // [B + 1] first row (token) of each request in this step
     const int* starts;      // [B] position of each request's first token of this step
     const int* block_table; // [B, table_stride]
     int table_stride;
-    float* part_o;          // [slots, Hk, ROWS, HD]
+    float* part_o;          // [slots, Hk, ROWS, HV]
     float* part_ml;         // [slots, Hk, ROWS, 2]
     int n_items, n_cta_items, H, Hk, page_shift, page_mask, page_size;
     float scale;
@@ -69,7 +76,17 @@ struct AttnArgs {
     float cap;              // > 0: a scaled score s counts as cap * tanh(s / cap) (no slopes then)
     const float* sinks;     // [H], or null: the softmax's denominator also holds exp(sinks[h]), an entry without key or value;
                             // it is added where a row's result is finished: by the item that writes the output, or by the merge
+    // What a finished row is multiplied by before it is rounded: out_scale, and with `gate` the sigmoid of the
+    // token's and head's number gate[t * ld_gate + h].
+    const float* gate;
+    int ld_gate;
+    float out_scale;
+    int ld_out;
 };
+
+__device__ inline float row_factor(const float* gate, int ld_gate, float out_scale, int t, int h) {
+    return gate ? out_scale / (1.0f + expf(-gate[(size_t)t * ld_gate + h])) : out_scale;
+}
 
 // a finished row's sum with the sink's share: the sums are in units of 2^m (m the row's reference in units of log2)
 __device__ inline float with_sink(const float* sinks, int h, float m, float l) {
@@ -240,7 +257,7 @@ struct CtaShape {
     static constexpr int SETS = 2 * CTA_STAGES * STAGE * 16 <= 144 * 1024 ? 2 : 1;
     static constexpr int THREADS = SET_THREADS * SETS;
     static constexpr int RING_BYTES = SETS * CTA_STAGES * STAGE * 16;
-    static constexpr int COMBINE_BYTES = SETS == 2 ? 4 * ROWS * (HD + 4 + 2) * 4 : 0;
+    static constexpr int COMBINE_BYTES = SETS == 2 ? 4 * ROWS * (HV + 4 + 2) * 4 : 0;
     static constexpr int LDS_BYTES = RING_BYTES > COMBINE_BYTES ? RING_BYTES : COMBINE_BYTES;
     static_assert(LDS_BYTES <= 160 * 1024, "the tiles do not fit into LDS");
 };
@@ -250,15 +267,16 @@ __device__ inline void cta_write_out(const AttnArgs& a, const f32x16 (&o)[DB], f
                                      int kvh, int lr, int lg, int slot) {
     if (!row_ok) return;
     if (slot < 0) l = with_sink(a.sinks, h, m, l);
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float inv = l > 0.f ? 1.0f / l : 0.f;
     if (slot < 0) {
-        bf16_t* op = a.out + ((size_t)t * a.H + h) * HD;
+        inv *= row_factor(a.gate, a.ld_gate, a.out_scale, t, h);
+        bf16_t* op = a.out + (size_t)t * a.ld_out + h * HV;
 #pragma unroll
         for (int d = 0; d < DB; ++d)
 #pragma unroll
             for (int e4 = 0; e4 < 4; ++e4) {
                 const int dd = d * 32 + e4 * 8 + lg * 4;
-                if (dd < HD) {
+                if (dd < HV) {
                     uint2 w = make_uint2(pack2(o[d][e4 * 4 + 0] * inv, o[d][e4 * 4 + 1] * inv),
                                          pack2(o[d][e4 * 4 + 2] * inv, o[d][e4 * 4 + 3] * inv));
                     *reinterpret_cast<uint2*>(op + dd) = w;
@@ -266,13 +284,13 @@ __device__ inline void cta_write_out(const AttnArgs& a, const f32x16 (&o)[DB], f
             }
         return;
     }
-    float* po = a.part_o + (((size_t)slot * a.Hk + kvh) * ROWS + lr) * HD;
+    float* po = a.part_o + (((size_t)slot * a.Hk + kvh) * ROWS + lr) * HV;
 #pragma unroll
     for (int d = 0; d < DB; ++d)
 #pragma unroll
         for (int e4 = 0; e4 < 4; ++e4) {
             const int dd = d * 32 + e4 * 8 + lg * 4;
-            if (dd < HD)
+            if (dd < HV)
                 *reinterpret_cast<float4*>(po + dd) = make_float4(o[d][e4 * 4 + 0] * inv, o[d][e4 * 4 + 1] * inv,
                                                                   o[d][e4 * 4 + 2] * inv, o[d][e4 * 4 + 3] * inv);
         }
@@ -538,7 +556,7 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
     // whole tile and a copy instruction brings pieces of keys only or of values only (head sizes 64, 128
     // and 256), a whole tile of an existing page is copied from two bases that all lanes share, each
     // lane adding a fixed 32-bit offset.
-    constexpr bool CTA_FAST = CK_POW2 && NKC % SET_THREADS == 0 && NVC % SET_THREADS == 0 && HD % 32 == 0;
+    constexpr bool CTA_FAST = CK_POW2 && NKC % SET_THREADS == 0 && NVC % SET_THREADS == 0 && HV % 32 == 0;
     auto piece = [&](int i, int tid_, int& off, int& key, bool& is_k) {
         const int q = i * SET_THREADS + tid_;
         is_k = q < NKC;
@@ -550,7 +568,7 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
         } else {
             const int vv = q - NKC, d = vv >> 2, c = (vv & 3) ^ ((d >> 2) & 3);
             off = d * a.page_size + c * 8;
-            key = (vv < NVC && d < HD) ? c * 8 : (1 << 30);
+            key = (vv < NVC && d < HV) ? c * 8 : (1 << 30);
         }
     };
     constexpr int N_OFF = CTA_FAST ? LOADS : 1;
@@ -567,9 +585,9 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
     const bf16_t* __restrict__ kc = a.kc;
     const bf16_t* __restrict__ vc = a.vc;
     // a page's bytes (of all its key/value heads), and this head's part of page 0
-    const uint32_t page_bytes = (uint32_t)a.Hk * (uint32_t)a.page_size * (HD * 2);
+    const uint32_t page_bytes = (uint32_t)a.Hk * (uint32_t)a.page_size * (HD * 2), v_page_bytes = (uint32_t)a.Hk * (uint32_t)a.page_size * (HV * 2);
     const char* const kc_head = reinterpret_cast<const char*>(kc) + (size_t)kvh * a.page_size * (HD * 2);
-    const char* const vc_head = reinterpret_cast<const char*>(vc) + (size_t)kvh * a.page_size * (HD * 2);
+    const char* const vc_head = reinterpret_cast<const char*>(vc) + (size_t)kvh * a.page_size * (HV * 2);
     const bf16_t* zero_src = reinterpret_cast<const bf16_t*>(xr_zero_chunk);
 
     // page numbers of the item's keys, one per lane, 64 pages at a time, from the page of the older of
@@ -616,7 +634,7 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
             }                                                                                            \
             if (v_there_) {                                                                              \
                 const int pg_ = __builtin_amdgcn_readlane(my_page, (ktv_ >> a.page_shift) - pages_base); \
-                const char* vb_ = vc_head + (size_t)(uint32_t)max(pg_, 0) * page_bytes + (uint32_t)(ktv_ & a.page_mask) * 2; \
+                const char* vb_ = vc_head + (size_t)(uint32_t)max(pg_, 0) * v_page_bytes + (uint32_t)(ktv_ & a.page_mask) * 2; \
                 _Pragma("unroll") for (int i = 0; i < LOADS; ++i)                                        \
                     if (i * SET_THREADS >= NKC) lds_dma16_base(vb_, fast_off[i % N_OFF], dst_ + i * SET_THREADS * 16); \
             }                                                                                            \
@@ -626,7 +644,7 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
             const size_t pbk_ = (size_t)(pgk_ < 0 ? 0 : pgk_) * a.Hk + kvh;                              \
             const size_t pbv_ = (size_t)(pgv_ < 0 ? 0 : pgv_) * a.Hk + kvh;                              \
             const bf16_t* kb_ = kc + (pbk_ * a.page_size + (ktk_ & a.page_mask)) * HD;                   \
-            const bf16_t* vb_ = vc + pbv_ * HD * a.page_size + (ktv_ & a.page_mask);                     \
+            const bf16_t* vb_ = vc + pbv_ * HV * a.page_size + (ktv_ & a.page_mask);                     \
             _Pragma("unroll") for (int i = 0; i < LOADS; ++i) {                                          \
                 int tid_ = tid, off_, key_;                                                              \
                 bool isk_;                                                                               \
@@ -729,16 +747,16 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
     if (SETS == 2) {
         // the second set hands its rows' maxima, sums and unnormalised outputs to the first
         __syncthreads();                                 // the rings are free
-        float* xo = reinterpret_cast<float*>(lds_all);   // [4 row blocks][ROWS][HD + 4]
-        float* xml = xo + 4 * ROWS * (HD + 4);           // [4 row blocks][ROWS][2]
-        float* mine = xo + (wave * ROWS + lr) * (HD + 4);
+        float* xo = reinterpret_cast<float*>(lds_all);   // [4 row blocks][ROWS][HV + 4]
+        float* xml = xo + 4 * ROWS * (HV + 4);           // [4 row blocks][ROWS][2]
+        float* mine = xo + (wave * ROWS + lr) * (HV + 4);
         if (set == 1) {
 #pragma unroll
             for (int d = 0; d < DB; ++d)
 #pragma unroll
                 for (int e4 = 0; e4 < 4; ++e4) {
                     const int dd = d * 32 + e4 * 8 + lg * 4;
-                    if (dd < HD)
+                    if (dd < HV)
                         *reinterpret_cast<float4*>(mine + dd) = make_float4(o[d][e4 * 4 + 0], o[d][e4 * 4 + 1], o[d][e4 * 4 + 2], o[d][e4 * 4 + 3]);
                 }
             if (lg == 0) {
@@ -759,7 +777,7 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
 #pragma unroll
             for (int e4 = 0; e4 < 4; ++e4) {
                 const int dd = d * 32 + e4 * 8 + lg * 4;
-                if (dd < HD) {
+                if (dd < HV) {
                     const float4 x = *reinterpret_cast<const float4*>(mine + dd);
                     o[d][e4 * 4 + 0] = o[d][e4 * 4 + 0] * f0 + x.x * f1;
                     o[d][e4 * 4 + 1] = o[d][e4 * 4 + 1] * f0 + x.y * f1;
@@ -779,13 +797,13 @@ __global__ __launch_bounds__(CtaShape::THREADS, 1) void k_attn_cta(AttnArgs a) {
 // 64 bytes of V^T per lane group, instead of 32 bytes from 32 places per load instruction)
 // and reads its fragments from there, so the main loop has no barrier at all.  At the end
 // the waves' results are combined through LDS and written as the output or as one partial.
-constexpr int STREAM_WAVES = HD <= 128 ? 4 : 2;
+constexpr int STREAM_WAVES = HD <= 128 && HV <= 128 ? 4 : 2;
 constexpr int W_LOADS = (NKC + NVC + 63) / 64;              // copies per lane and tile
 constexpr int W_STAGE = W_LOADS * 64;                       // chunks of a wave's tile
 // (measured at head size 128, batches of 1 to 64 and contexts of 2k and 8k: 4 waves with 2 tiles
 // each, 3 with 3, 2 with 2 to 4 and 1 with 3 or 4 are all within 5% of each other)
 constexpr int STREAM_STAGES = W_STAGE * 16 * STREAM_WAVES * 3 <= 96 * 1024 ? 3 : 2;
-constexpr int MERGE_STRIDE = HD + 4;                        // floats between rows of the combining buffer
+constexpr int MERGE_STRIDE = HV + 4;                        // floats between rows of the combining buffer
 constexpr int STREAM_RING_BYTES = STREAM_WAVES * STREAM_STAGES * W_STAGE * 16;
 constexpr int STREAM_MERGE_BYTES = STREAM_WAVES * ROWS * (MERGE_STRIDE + 2) * 4;
 constexpr int STREAM_LDS_BYTES = STREAM_RING_BYTES > STREAM_MERGE_BYTES ? STREAM_RING_BYTES : STREAM_MERGE_BYTES;
@@ -844,7 +862,7 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
         } else {
             const int v = q - NKC, d = v >> 2, c = (v & 3) ^ ((d >> 2) & 3);
             src_off[i] = d * a.page_size;
-            src_key[i] = (v < NVC && d < HD) ? c * 8 : (1 << 30);
+            src_key[i] = (v < NVC && d < HV) ? c * 8 : (1 << 30);
         }
     }
     const bf16_t* __restrict__ kc = a.kc;
@@ -885,7 +903,7 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
             const size_t pb_ = (size_t)(pg_ < 0 ? 0 : pg_) * a.Hk + kvh;                                 \
             const int ko_ = kt_ & a.page_mask;                                                           \
             const bf16_t* kb_ = kc + (pb_ * a.page_size + ko_) * HD;                                     \
-            const bf16_t* vb_ = vc + pb_ * HD * a.page_size + ko_;                                       \
+            const bf16_t* vb_ = vc + pb_ * HV * a.page_size + ko_;                                       \
             _Pragma("unroll") for (int i = 0; i < W_LOADS; ++i) {                                        \
                 const bool ok_ = pg_ >= 0 && kt_ + src_key[i] < seq_len;                                 \
                 const bf16_t* p_ = ok_ ? (src_is_k[i] ? kb_ + src_key[i] * HD : vb_ + src_key[i]) + src_off[i] : zero_src; \
@@ -900,7 +918,7 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
                 const size_t pb_ = (size_t)(ok_ ? pg_ : 0) * a.Hk + kvh;                                 \
                 const int ko_ = key_ & a.page_mask;                                                      \
                 const bf16_t* p_ = src_is_k[i] ? kc + (pb_ * a.page_size + ko_) * HD + src_off[i]        \
-                                               : vc + pb_ * HD * a.page_size + src_off[i] + ko_;         \
+                                               : vc + pb_ * HV * a.page_size + src_off[i] + ko_;         \
                 lds_dma16(ok_ ? p_ : zero_src, dst_ + i * 64 * 16);                                      \
             }                                                                                            \
         }                                                                                                \
@@ -989,7 +1007,7 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
 #pragma unroll
             for (int e4 = 0; e4 < 4; ++e4) {
                 const int dd = d * 32 + e4 * 8 + lg * 4;
-                if (dd < HD)
+                if (dd < HV)
                     *reinterpret_cast<float4*>(dst + dd) = make_float4(o[d][e4 * 4 + 0], o[d][e4 * 4 + 1],
                                                                        o[d][e4 * 4 + 2], o[d][e4 * 4 + 3]);
             }
@@ -1001,8 +1019,8 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
     __syncthreads();
     const int rows_left = q_len * G - row0;
     const int n_rows = rows_left < ROWS ? rows_left : ROWS;
-    for (int idx = tid; idx < n_rows * (HD / 4); idx += 64 * STREAM_WAVES) {
-        const int r = idx / (HD / 4), d4 = (idx - r * (HD / 4)) * 4;
+    for (int idx = tid; idx < n_rows * (HV / 4); idx += 64 * STREAM_WAVES) {
+        const int r = idx / (HV / 4), d4 = (idx - r * (HV / 4)) * 4;
         float mx = -INFINITY;
 #pragma unroll
         for (int w = 0; w < STREAM_WAVES; ++w) mx = fmaxf(mx, mml[(w * ROWS + r) * 2]);
@@ -1018,12 +1036,13 @@ __global__ __launch_bounds__(64 * STREAM_WAVES) void k_attn_stream(AttnArgs a) {
         }
         const int rr = row0 + r, tk = rr / G, hh = kvh * G + (rr - tk * G);
         if (slot < 0) lsum = with_sink(a.sinks, hh, mx, lsum);
-        const float inv = lsum > 0.f ? 1.0f / lsum : 0.f;
+        float inv = lsum > 0.f ? 1.0f / lsum : 0.f;
         if (slot < 0) {
-            bf16_t* op = a.out + ((size_t)(q0 + tk) * a.H + hh) * HD + d4;
+            inv *= row_factor(a.gate, a.ld_gate, a.out_scale, q0 + tk, hh);
+            bf16_t* op = a.out + (size_t)(q0 + tk) * a.ld_out + hh * HV + d4;
             *reinterpret_cast<uint2*>(op) = make_uint2(pack2(acc.x * inv, acc.y * inv), pack2(acc.z * inv, acc.w * inv));
         } else {
-            float* po = a.part_o + (((size_t)slot * a.Hk + kvh) * ROWS + r) * HD + d4;
+            float* po = a.part_o + (((size_t)slot * a.Hk + kvh) * ROWS + r) * HV + d4;
             *reinterpret_cast<float4*>(po) = make_float4(acc.x * inv, acc.y * inv, acc.z * inv, acc.w * inv);
             if (d4 == 0) {
                 float* pm = a.part_ml + (((size_t)slot * a.Hk + kvh) * ROWS + r) * 2;
@@ -1045,6 +1064,10 @@ struct MergeArgs {
     bf16_t* out;
     int H, Hk;
     const float* sinks;     // as in AttnArgs
+    const float* gate;
+    int ld_gate;
+    float out_scale;
+    int ld_out;
 };
 
 __global__ __launch_bounds__(256) void k_attn_merge(MergeArgs a) {
@@ -1054,13 +1077,13 @@ __global__ __launch_bounds__(256) void k_attn_merge(MergeArgs a) {
     const int G = a.H / a.Hk;
     const int q0 = job[5], q_len = job[6];          // (with the job: one dependent read less before the partial results)
     const int n_rows = (q_len * G - row0) < ROWS ? (q_len * G - row0) : ROWS;      // rows of this block that exist
-    for (int idx = threadIdx.x; idx < n_rows * (HD / 4); idx += 256) {
-        const int r = idx / (HD / 4), d4 = (idx % (HD / 4)) * 4;
+    for (int idx = threadIdx.x; idx < n_rows * (HV / 4); idx += 256) {
+        const int r = idx / (HV / 4), d4 = (idx % (HV / 4)) * 4;
         const int rho = row0 + r;
         const int tok = rho / G, hg = rho - tok * G;
         const float* ml = a.part_ml + (((size_t)s0 * a.Hk + kvh) * ROWS + r) * 2;
-        const float* po = a.part_o + (((size_t)s0 * a.Hk + kvh) * ROWS + r) * HD + d4;
-        const size_t ml_step = (size_t)stride * a.Hk * ROWS * 2, po_step = (size_t)stride * a.Hk * ROWS * HD;
+        const float* po = a.part_o + (((size_t)s0 * a.Hk + kvh) * ROWS + r) * HV + d4;
+        const size_t ml_step = (size_t)stride * a.Hk * ROWS * 2, po_step = (size_t)stride * a.Hk * ROWS * HV;
         // 16 slots at a time, all their loads on their way before the first is used (a thread that
         // took the maxima first and then the outputs, four loads at a time, waited out eight memory
         // latencies for the 14 slots of a lone request: 8 us, as long as the attention itself)
@@ -1093,8 +1116,8 @@ __global__ __launch_bounds__(256) void k_attn_merge(MergeArgs a) {
             }
         }
         wsum = with_sink(a.sinks, kvh * G + hg, mx, wsum);
-        const float inv = wsum > 0.f ? 1.0f / wsum : 0.f;
-        bf16_t* op = a.out + ((size_t)(q0 + tok) * a.H + kvh * G + hg) * HD + d4;
+        const float inv = (wsum > 0.f ? 1.0f / wsum : 0.f) * row_factor(a.gate, a.ld_gate, a.out_scale, q0 + tok, kvh * G + hg);
+        bf16_t* op = a.out + (size_t)(q0 + tok) * a.ld_out + (kvh * G + hg) * HV + d4;
         *reinterpret_cast<uint2*>(op) = make_uint2(pack2(acc.x * inv, acc.y * inv), pack2(acc.z * inv, acc.w * inv));
     }
 }
@@ -1127,6 +1150,7 @@ static int launch_mode(const AttnArgs& a, const int* jobs, int n_jobs, const int
         MergeArgs mg;
         mg.jobs = jobs; mg.cu_q = cu_q; mg.part_o = a.part_o; mg.part_ml = a.part_ml; mg.out = a.out;
         mg.H = a.H; mg.Hk = a.Hk; mg.sinks = a.sinks;
+        mg.gate = a.gate; mg.ld_gate = a.ld_gate; mg.out_scale = a.out_scale; mg.ld_out = a.ld_out;
         k_attn_merge<<<dim3(n_jobs, a.Hk), 256, 0, stream>>>(mg);
         XR_CHECK_LAUNCH("attention_merge");
     }
@@ -1139,9 +1163,12 @@ extern "C" int xr_attention_mfma(void* out, const void* q, const void* k_cache, 
                                  const int* items, int n_items, int n_cta_items, const int* jobs, int n_jobs,
                                  const int* cu_q,
                                  const int* starts, const int* block_table, int table_stride, float* part_o,
-                                 float* part_ml, int H, int Hk, int D, int page_size, float scale, int window,
-                                 int chunk, const float* slopes, const float* sinks, float cap, hipStream_t stream) {
-    XR_REQUIRE(D == HD, "attention: this library is compiled for head size %d, got %d", HD, D);
+                                 float* part_ml, int H, int Hk, int D, int Dv, int page_size, float scale, int window,
+                                 int chunk, const float* slopes, const float* sinks, float cap, const float* gate, int ld_gate,
+                                 float out_scale, int ld_out, hipStream_t stream) {
+    XR_REQUIRE(D == HD && Dv == HV, "attention: this library is compiled for head size %d and value size %d, got %d and %d", HD, HV, D, Dv);
+    XR_REQUIRE(ld_out >= H * HV && ld_out % 4 == 0 && ((uintptr_t)out % 8) == 0, "attention: output rows %d apart (at least %d, a multiple of 4)", ld_out, H * HV);
+    XR_REQUIRE(!gate || ld_gate >= H, "attention: a gate of %d heads in rows %d apart", H, ld_gate);
     XR_REQUIRE(H > 0 && Hk > 0 && H % Hk == 0, "attention: %d query heads are not a multiple of %d key/value heads", H, Hk);
     int shift = ilog2_exact(page_size);
     XR_REQUIRE(shift >= 4, "attention: the MFMA kernel needs a page size that is a power of two of at least 16, got %d", page_size);
@@ -1160,6 +1187,7 @@ extern "C" int xr_attention_mfma(void* out, const void* q, const void* k_cache, 
     a.slopes = slopes;
     a.sinks = sinks;        // (an item that writes the output adds it; rows of split work are finished by the merge, which adds it there)
     a.cap = cap;
+    a.gate = gate; a.ld_gate = ld_gate; a.out_scale = out_scale; a.ld_out = ld_out;
     XR_REQUIRE(cap >= 0.f && (cap == 0.f || (scale > 0.f && !slopes)), "attention: a soft cap %g of the scores needs a positive scale and no slopes", (double)cap);
     XR_REQUIRE(!slopes || scale > 0.f, "attention: distance slopes need a positive scale, got %g", (double)scale);
     if (cap > 0.f) return launch_mode<MODE_CAP>(a, jobs, n_jobs, cu_q, stream);

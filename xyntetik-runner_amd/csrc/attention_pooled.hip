@@ -13,6 +13,7 @@
 #include "common.h"
 
 #define AP_MAX_D 512
+#define AP_WIDE_D 1024       // the largest row of all, by a second instance of the attention kernel
 
 // ---------------------------------------------------------------- queries out, keys and values into their pages
 template <typename T>
@@ -188,7 +189,7 @@ __device__ inline void unpack8(uint4 w, float* f) {
     f[6] = __uint_as_float(w.w << 16); f[7] = __uint_as_float(w.w & 0xffff0000u);
 }
 
-template <typename T, bool VEC>
+template <typename T, bool VEC, int MAXD = AP_MAX_D>
 __device__ inline void attend_range(const T* __restrict__ kc, const T* __restrict__ vc, const int* __restrict__ bt, int lo,
                                     int hi, const float* qs, int kvh, const PoolAttnArgs& a, float& m, float& l,
                                     float* acc, int lane) {
@@ -216,7 +217,7 @@ __device__ inline void attend_range(const T* __restrict__ kc, const T* __restric
         const float corr = mn == -INFINITY ? 1.f : expf(m - mn);
         l = l * corr + wave_sum(p);
 #pragma unroll
-        for (int dd = 0; dd < AP_MAX_D / 64; ++dd) acc[dd] *= corr;
+        for (int dd = 0; dd < MAXD / 64; ++dd) acc[dd] *= corr;
         const int nk = hi - k0 < 64 ? hi - k0 : 64;
         if (VEC) {
             for (int j0 = 0; j0 < nk; j0 += 8) {
@@ -227,7 +228,7 @@ __device__ inline void attend_range(const T* __restrict__ kc, const T* __restric
                 for (int i = 0; i < 8; ++i) pj[i] = __shfl(p, j0 + i, 64);
                 const T* vb = vc + ((size_t)bt[kj >> a.page_shift] * a.Hk + kvh) * a.Dv * a.page_size + (kj & a.page_mask);
 #pragma unroll
-                for (int dd = 0; dd < AP_MAX_D / 64; ++dd) {
+                for (int dd = 0; dd < MAXD / 64; ++dd) {
                     const int d = lane + 64 * dd;
                     if (d < a.Dv) {
                         float f[8];
@@ -244,7 +245,7 @@ __device__ inline void attend_range(const T* __restrict__ kc, const T* __restric
                 const int kj = k0 + j;
                 const T* vb = vc + ((size_t)bt[kj >> a.page_shift] * a.Hk + kvh) * a.Dv * a.page_size + (kj & a.page_mask);
 #pragma unroll
-                for (int dd = 0; dd < AP_MAX_D / 64; ++dd) {
+                for (int dd = 0; dd < MAXD / 64; ++dd) {
                     const int d = lane + 64 * dd;
                     if (d < a.Dv) acc[dd] = fmaf(pj, ld<T>(vb, (size_t)d * a.page_size), acc[dd]);
                 }
@@ -254,11 +255,11 @@ __device__ inline void attend_range(const T* __restrict__ kc, const T* __restric
     }
 }
 
-template <typename T, bool VEC>
+template <typename T, bool VEC, int MAXD = AP_MAX_D>
 __global__ __launch_bounds__(64) void k_attention_pooled(T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ kc,
                                                          const T* __restrict__ vc, const T* __restrict__ pk,
                                                          const T* __restrict__ pv, PoolAttnArgs a) {
-    __shared__ float qs[AP_MAX_D];
+    __shared__ float qs[MAXD];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = a.positions[t], req = a.req_of_token[t];
     const int kvh = h / (a.H / a.Hk);
@@ -266,18 +267,18 @@ __global__ __launch_bounds__(64) void k_attention_pooled(T* __restrict__ out, co
     for (int d = lane; d < a.D; d += 64) qs[d] = ld<T>(qrow, d);
     __syncthreads();
     float m = -INFINITY, l = 0.f;
-    float acc[AP_MAX_D / 64];
+    float acc[MAXD / 64];
 #pragma unroll
-    for (int dd = 0; dd < AP_MAX_D / 64; ++dd) acc[dd] = 0.f;
+    for (int dd = 0; dd < MAXD / 64; ++dd) acc[dd] = 0.f;
     const int lo = pos - a.size + 1 > 0 ? pos - a.size + 1 : 0;
     // blocks b with b P + P - 1 <= pos - size, i.e. b < (pos - size + 1) / P
     const int n_blocks = (a.P > 0 && pos - a.size + 1 > 0) ? (pos - a.size + 1) / a.P : 0;
     if (n_blocks > 0)
-        attend_range<T, VEC>(pk, pv, a.pool_table + (size_t)req * a.pool_stride, 0, n_blocks, qs, kvh, a, m, l, acc, lane);
-    attend_range<T, VEC>(kc, vc, a.block_table + (size_t)req * a.table_stride, lo, pos + 1, qs, kvh, a, m, l, acc, lane);
+        attend_range<T, VEC, MAXD>(pk, pv, a.pool_table + (size_t)req * a.pool_stride, 0, n_blocks, qs, kvh, a, m, l, acc, lane);
+    attend_range<T, VEC, MAXD>(kc, vc, a.block_table + (size_t)req * a.table_stride, lo, pos + 1, qs, kvh, a, m, l, acc, lane);
     T* orow = out + ((size_t)t * a.H + h) * a.Dv;
 #pragma unroll
-    for (int dd = 0; dd < AP_MAX_D / 64; ++dd) {
+    for (int dd = 0; dd < MAXD / 64; ++dd) {
         const int d = lane + 64 * dd;
         if (d < a.Dv) st<T>(orow, d, acc[dd] / l);
     }
@@ -359,7 +360,7 @@ extern "C" int xr_attention_pooled(void* out, const void* q, const void* k_cache
                                    int table_stride, const int* pool_table, int pool_stride, int T, int H, int Hk, int D,
                                    int Dv, int page_size, float scale, int size, int P, int dtype, hipStream_t stream) {
     XR_REQUIRE(T >= 0 && H > 0 && Hk > 0 && H % Hk == 0, "pooled attention: %d query heads over %d key/value heads", H, Hk);
-    XR_REQUIRE(D > 0 && D <= AP_MAX_D && Dv > 0 && Dv <= AP_MAX_D, "pooled attention: key size %d, value size %d (1 to %d)", D, Dv, AP_MAX_D);
+    XR_REQUIRE(D > 0 && D <= AP_WIDE_D && Dv > 0 && Dv <= AP_WIDE_D, "pooled attention: key size %d, value size %d (1 to %d)", D, Dv, AP_WIDE_D);
     const int shift = ilog2_exact(page_size);
     XR_REQUIRE(shift >= 0, "pooled attention: page size %d is not a power of two", page_size);
     XR_REQUIRE(size >= 1 && P >= 0, "pooled attention: window %d, block %d", size, P);
@@ -369,16 +370,20 @@ extern "C" int xr_attention_pooled(void* out, const void* q, const void* k_cache
                    page_size - 1, page_size, scale, size, P};
     dim3 grid(T, H);
     const bool vec = dtype == XR_BF16 && D % 8 == 0 && page_size >= 8;
-    if (dtype == XR_F32)
-        k_attention_pooled<float, false><<<grid, 64, 0, stream>>>((float*)out, (const float*)q, (const float*)k_cache,
-                                                                  (const float*)v_cache, (const float*)pk, (const float*)pv, a);
-    else if (dtype == XR_BF16 && vec)
-        k_attention_pooled<bf16_t, true><<<grid, 64, 0, stream>>>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k_cache,
-                                                                  (const bf16_t*)v_cache, (const bf16_t*)pk, (const bf16_t*)pv, a);
-    else if (dtype == XR_BF16)
-        k_attention_pooled<bf16_t, false><<<grid, 64, 0, stream>>>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k_cache,
-                                                                   (const bf16_t*)v_cache, (const bf16_t*)pk, (const bf16_t*)pv, a);
+#define AP(T, VEC)                                                                                                          \
+    do {                                                                                                                    \
+        if (D <= AP_MAX_D && Dv <= AP_MAX_D)                                                                                \
+            k_attention_pooled<T, VEC><<<grid, 64, 0, stream>>>((T*)out, (const T*)q, (const T*)k_cache, (const T*)v_cache,  \
+                                                                (const T*)pk, (const T*)pv, a);                             \
+        else                                                                                                                \
+            k_attention_pooled<T, VEC, AP_WIDE_D><<<grid, 64, 0, stream>>>((T*)out, (const T*)q, (const T*)k_cache,          \
+                                                                           (const T*)v_cache, (const T*)pk, (const T*)pv, a); \
+    } while (0)
+    if (dtype == XR_F32) AP(float, false);
+    else if (dtype == XR_BF16 && vec) AP(bf16_t, true);
+    else if (dtype == XR_BF16) AP(bf16_t, false);
     else { xr_set_error("pooled attention: bad dtype %d", dtype); return XR_BAD_ARG; }
+#undef AP
     XR_CHECK_LAUNCH("attention_pooled");
     return XR_OK;
 }

@@ -14,7 +14,8 @@
 // `keep` > 0: the keys [0, keep) are read as well wherever lo lies.  `sinks` (one number a query head): the
 // softmax's denominator also holds exp(sink_h) (of the sink as it is: no scale, no cap), an entry that has no key and no value.  Values may have another
 // size than keys (Dv; cache layout K [page][kv_head][slot][D], V [page][kv_head][Dv][slot]).
-// With `cap` > 0 a scaled score s counts as cap * tanh(s / cap), before a slope's bias.
+// With `cap` > 0 a scaled score s counts as cap * tanh(s / cap), before a slope's bias.  A head's output is multiplied by
+// `out_scale` and, with `gate` (a number a token and head), by sigmoid(gate); output rows are ld_out apart.
 #include "common.h"
 
 #define AR_MAX_D 256
@@ -25,7 +26,7 @@ __global__ __launch_bounds__(64) void k_attention_ref(
     const int* __restrict__ positions, const int* __restrict__ req_of_token,
     const int* __restrict__ block_table, int table_stride, int H, int Hk, int D, int Dv, int page_shift,
     int page_mask, int page_size, float scale, int window, int chunk, int keep, const float* __restrict__ slopes,
-    const float* __restrict__ sinks, float cap) {
+    const float* __restrict__ sinks, float cap, const float* __restrict__ gate, int ld_gate, float out_scale, int ld_out) {
     __shared__ float qs[AR_MAX_D];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = positions[t];
@@ -88,11 +89,12 @@ __global__ __launch_bounds__(64) void k_attention_ref(
 #pragma unroll
         for (int dd = 0; dd < AR_MAX_D / 64; ++dd) acc[dd] *= corr;
     }
-    T* orow = out + ((size_t)t * H + h) * Dv;
+    T* orow = out + (size_t)t * ld_out + (size_t)h * Dv;
+    const float f = gate ? out_scale / (1.0f + expf(-gate[(size_t)t * ld_gate + h])) : out_scale;
 #pragma unroll
     for (int dd = 0; dd < AR_MAX_D / 64; ++dd) {
         const int d = lane + 64 * dd;
-        if (d < Dv) st<T>(orow, d, acc[dd] / l);
+        if (d < Dv) st<T>(orow, d, acc[dd] / l * f);
     }
 }
 
@@ -100,7 +102,8 @@ extern "C" int xr_attention_ref(void* out, const void* q, const void* k_cache, c
                                 const int* positions, const int* req_of_token, const int* block_table,
                                 int table_stride, int T, int H, int Hk, int D, int Dv, int page_size, float scale,
                                 int window, int chunk, int keep, int dtype, const float* slopes, const float* sinks,
-                                float cap, hipStream_t stream) {
+                                float cap, const float* gate, int ld_gate, float out_scale, int ld_out, hipStream_t stream) {
+    XR_REQUIRE(ld_out >= H * Dv && (!gate || ld_gate >= H), "attention: output rows %d apart, gate rows %d apart for %d heads of %d", ld_out, ld_gate, H, Dv);
     XR_REQUIRE(cap >= 0.f, "attention: soft cap %g of the scores is negative", (double)cap);
     XR_REQUIRE(T >= 0 && H > 0 && Hk > 0 && D > 0, "attention: bad sizes T=%d H=%d Hk=%d D=%d", T, H, Hk, D);
     XR_REQUIRE(H % Hk == 0, "attention: %d query heads are not a multiple of %d key/value heads", H, Hk);
@@ -114,11 +117,11 @@ extern "C" int xr_attention_ref(void* out, const void* q, const void* k_cache, c
     if (dtype == XR_F32)
         k_attention_ref<float><<<grid, 64, 0, stream>>>((float*)out, (const float*)q, (const float*)k_cache,
                                                         (const float*)v_cache, positions, req_of_token, block_table,
-                                                        table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks, cap);
+                                                        table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks, cap, gate, ld_gate, out_scale, ld_out);
     else if (dtype == XR_BF16)
         k_attention_ref<bf16_t><<<grid, 64, 0, stream>>>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k_cache,
                                                          (const bf16_t*)v_cache, positions, req_of_token, block_table,
-                                                         table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks, cap);
+                                                         table_stride, H, Hk, D, Dv, shift, page_size - 1, page_size, scale, window, chunk, keep, slopes, sinks, cap, gate, ld_gate, out_scale, ld_out);
     else { xr_set_error("attention: bad dtype %d", dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("attention_ref");
     return XR_OK;

@@ -603,6 +603,147 @@ extern "C" int xr_row_norm_rope_write(const float* q_in, const float* k_in, cons
     return XR_OK;
 }
 
+// The same head by head, for values of any size: every query and key head over its own root mean square (eps inside
+// the root) times a weight of its channels that the heads share (absent: none), before the rotation or behind it, or no
+// norm at all.  Queries go out, keys and values (Dv channels a head) to their pages.  A workgroup a token, a wave a head at
+// a time: its lanes hold channels lane, lane + 64, .. and read a pair's other channel beside their own.
+struct HeadNormArgs {
+    RopeArgs r;
+    const float* wq;        // [D] or null
+    const float* wk;        // [D] or null
+    float eps;
+    int norm;               // HEAD_NORM_*
+    int Dv;
+};
+#define HEAD_NORM_NONE 0
+#define HEAD_NORM_BEFORE 1
+#define HEAD_NORM_AFTER 2
+#define HEAD_MAX_D 256
+template <typename T, int NW>
+__global__ __launch_bounds__(64 * NW) void k_head_norm_rope_write(HeadNormArgs n) {
+    constexpr int NT = 64 * NW, NC = HEAD_MAX_D / 64;
+    __shared__ float cs[2][HEAD_MAX_D / 2];
+    const RopeArgs& a = n.r;
+    const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int D = a.D, half = a.rot >> 1;
+    const int pos = a.positions[t];
+    for (int j = tid; j < half; j += NT) {
+        const float ang = (float)pos * a.inv_freq[j];
+        cs[0][j] = cosf(ang) * a.mscale;
+        cs[1][j] = sinf(ang) * a.mscale;
+    }
+    __syncthreads();
+    PageRef pr{0, 0};
+    int req = 0;
+    if (a.Hk) {
+        req = a.req_of_token[t];
+        pr = page_of(a.block_table, a.table_stride, req, pos, a.page_shift, a.page_mask);
+    }
+    for (int head = wave; head < a.H + a.Hk; head += NW) {
+        const bool is_q = head < a.H;
+        const float* src = (is_q ? a.q_in + (size_t)head * D : a.k_in + (size_t)(head - a.H) * D) + (size_t)t * a.in_stride;
+        const float* w = is_q ? n.wq : n.wk;
+        float x[NC], z[NC], wx[NC], wz[NC];
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+            const int d = lane + 64 * i;
+            const bool ok = d < D, turns = d < a.rot;
+            const int o = !turns ? d : a.interleaved ? d ^ 1 : (d < half ? d + half : d - half);      // the pair's other channel
+            x[i] = ok ? src[d] : 0.f;
+            z[i] = ok && turns ? src[o] : 0.f;
+            wx[i] = ok && w ? w[d] : 1.f;
+            wz[i] = ok && w && turns ? w[o] : 1.f;
+            ss = fmaf(x[i], x[i], ss);
+        }
+        if (n.norm == HEAD_NORM_BEFORE) {
+            const float f = 1.0f / sqrtf(wave_sum(ss) / (float)D + n.eps);
+#pragma unroll
+            for (int i = 0; i < NC; ++i) { x[i] *= f * wx[i]; z[i] *= f * wz[i]; }
+        }
+        ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+            const int d = lane + 64 * i;
+            if (d < a.rot) {
+                const int j = a.interleaved ? d >> 1 : (d < half ? d : d - half);
+                const bool first = a.interleaved ? (d & 1) == 0 : d < half;
+                const float c = cs[0][j], s = cs[1][j];
+                x[i] = first ? x[i] * c - z[i] * s : x[i] * c + z[i] * s;
+            }
+            ss = fmaf(x[i], x[i], ss);
+        }
+        if (n.norm == HEAD_NORM_AFTER) {
+            const float f = 1.0f / sqrtf(wave_sum(ss) / (float)D + n.eps);
+#pragma unroll
+            for (int i = 0; i < NC; ++i) x[i] *= f * wx[i];
+        }
+        T* dst = is_q ? (T*)a.q_out + ((size_t)t * a.H + head) * D
+                      : (T*)a.k_cache + (((size_t)pr.page * a.Hk + (head - a.H)) * a.page_size + pr.off) * D;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+            const int d = lane + 64 * i;
+            if (d < D) st<T>(dst, d, x[i]);
+        }
+    }
+    if (!a.Hk) return;
+    // values: see k_rope_kv_write
+    const int V = a.Hk * n.Dv;
+    const float* vr = a.v_in + (size_t)t * a.in_stride;
+    T* vpage = (T*)a.v_cache + (size_t)pr.page * V * a.page_size + pr.off;
+    const int lead = t - (pos & 7);
+    const bool whole = a.page_size >= 8 && lead >= 0 && lead + 7 < a.T && a.req_of_token[lead] == req &&
+                       a.req_of_token[lead + 7] == req && a.positions[lead] == pos - (pos & 7);
+    if (!whole) {
+        for (int i = tid; i < V; i += NT) st<T>(vpage, (size_t)i * a.page_size, vr[i]);
+    } else if ((pos & 7) == 0) {
+        for (int i = tid; i < V; i += NT) {
+            float v[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] = vr[(size_t)j * a.in_stride + i];
+            store8<T>(vpage + (size_t)i * a.page_size, v);
+        }
+    }
+}
+
+extern "C" int xr_head_norm_rope_write(const float* q_in, const float* k_in, const float* v_in, int in_stride, const float* wq,
+                                       const float* wk, float eps, int norm, void* q_out, void* k_cache, void* v_cache,
+                                       const int* positions, const int* req_of_token, const int* block_table,
+                                       int table_stride, const float* inv_freq, int T, int H, int Hk, int D, int Dv, int rot,
+                                       int interleaved, float mscale, int page_size, int dtype, hipStream_t stream) {
+    XR_REQUIRE(T >= 0 && H > 0 && Hk >= 0 && D > 0 && D <= HEAD_MAX_D && Dv > 0, "head_norm_rope_write: bad sizes T=%d H=%d Hk=%d D=%d Dv=%d", T, H, Hk, D, Dv);
+    XR_REQUIRE(rot >= 0 && rot <= D && (rot % 2) == 0, "head_norm_rope_write: rotary width %d must be even and at most head_dim %d", rot, D);
+    XR_REQUIRE(rot == 0 || inv_freq, "head_norm_rope_write: rotary width %d without a frequency table", rot);
+    XR_REQUIRE(eps >= 0.f && norm >= HEAD_NORM_NONE && norm <= HEAD_NORM_AFTER, "head_norm_rope_write: eps %g, norm %d", (double)eps, norm);
+    const int shift = ilog2_exact(page_size);
+    XR_REQUIRE(Hk == 0 || shift >= 0, "head_norm_rope_write: page size %d is not a power of two", page_size);
+    XR_REQUIRE(Hk == 0 || (k_in && v_in && k_cache && v_cache && block_table && req_of_token),
+               "head_norm_rope_write: keys and values to cache but a null operand");
+    XR_REQUIRE(q_in && q_out && positions, "head_norm_rope_write: an operand is missing");
+    XR_REQUIRE(dtype == XR_F32 || dtype == XR_BF16, "head_norm_rope_write: bad dtype %d", dtype);
+    if (T == 0) return XR_OK;
+    HeadNormArgs n;
+    RopeArgs& a = n.r;
+    a.q_in = q_in; a.k_in = k_in; a.v_in = v_in; a.in_stride = in_stride;
+    a.q_out = q_out; a.k_cache = k_cache; a.v_cache = v_cache;
+    a.positions = positions; a.req_of_token = req_of_token;
+    a.block_table = block_table; a.table_stride = table_stride; a.inv_freq = inv_freq;
+    a.T = T; a.H = H; a.Hk = Hk; a.D = D; a.rot = rot; a.interleaved = interleaved; a.mscale = mscale;
+    a.page_shift = shift < 0 ? 0 : shift; a.page_mask = page_size - 1; a.page_size = page_size;
+    a.heads_per_block = 0; a.paired = 0;
+    n.wq = wq; n.wk = wk; n.eps = eps; n.norm = norm; n.Dv = Dv;
+    const bool few = T <= 128 && H + Hk > 4;
+    if (dtype == XR_F32) {
+        if (few) k_head_norm_rope_write<float, 16><<<T, 1024, 0, stream>>>(n);
+        else k_head_norm_rope_write<float, 4><<<T, 256, 0, stream>>>(n);
+    } else {
+        if (few) k_head_norm_rope_write<bf16_t, 16><<<T, 1024, 0, stream>>>(n);
+        else k_head_norm_rope_write<bf16_t, 4><<<T, 256, 0, stream>>>(n);
+    }
+    XR_CHECK_LAUNCH("head_norm_rope_write");
+    return XR_OK;
+}
+
 // ---------------------------------------------------------------- gate
 // h = act(g) * u; act = SiLU: g / (1 + exp(-g)) (src/model.c:4451-4452,
 // src/kernels.cu:2868-2874).  gu row = [gate(F) | up(F)].

@@ -2,8 +2,8 @@
 
 One shared object per *unit*: the unit "kernels" holds everything whose code does
 not depend on the model's sizes; a unit "attn_d<D>" holds the MFMA attention kernels
-specialised for head size D and is compiled when a model with that head size is
-first built.  Objects and libraries live beside the sources (``_build/`` and
+specialised for head size D ("attn_d<D>v<Dv>" with values of another size) and is compiled when a model with that head
+size is first built.  Objects and libraries live beside the sources (``_build/`` and
 ``lib*.so``); if that folder cannot be written, under ``$XR_BUILD_DIR`` or a
 per-user folder in the temporary directory.
 
@@ -51,9 +51,9 @@ class BuildError(RuntimeError):
 def unit_spec(unit: str) -> dict:
     if unit in UNITS:
         return UNITS[unit]
-    if unit.startswith("attn_d"):
-        d = int(unit[len("attn_d"):])
-        return {"sources": ATTN_SOURCES, "defines": [f"-DXR_HEAD_DIM={d}"]}
+    if unit.startswith("attn_d"):       # attn_d<D>, or attn_d<D>v<Dv> where values are of another size than keys
+        d, _, v = unit[len("attn_d"):].partition("v")
+        return {"sources": ATTN_SOURCES, "defines": [f"-DXR_HEAD_DIM={int(d)}"] + ([f"-DXR_VALUE_DIM={int(v)}"] if v else [])}
     raise BuildError(f"unknown kernel unit {unit!r}")
 
 

@@ -68,7 +68,7 @@ struct GemmArgs {
     int M, N, K, lda, ldo;
     int out_bf16;      // storage of out
     int epi;
-    int act;           // the gate's activation (XR_ACT_*), with EPI_GATED
+    int act;           // the gate's activation (XR_ACT_*), with EPI_GATED; with EPI_STORE what the results pass (XR_POST_*)
     float act_param;   // and its number, for a gate that takes one
     int m_fast;        // tile order of the asynchronous kernel: 1 = consecutive workgroups share a weight tile, 2 = by XCD
     int splits;        // > 1: K is cut into this many ranges, each workgroup writes raw sums to `partial`
@@ -92,6 +92,11 @@ struct GemmArgs {
     int norm_w_bf16;
     bf16_t* xg;
     float* ss_out;
+    // With norm_whole and EPI_STORE: the product itself is not written; row t of post_x becomes the norm of
+    // post_alpha * post_x[t] + the product's row, and xg its copy in bfloat16.
+    float* post_x;
+    int post_ld;
+    float post_alpha;
     RopeFuse rope;     // rotation and cache write in place of the output (on: rope.q_out not null)
 };
 
@@ -122,7 +127,18 @@ struct XrGemmNorm {
     float* ss_out;
     int ss_out_rows;   // in: partial rows that ss_out has room for; out: partial rows written
     int centred;       // the norm after the product is a layer norm (more than 16 rows, finished by k_gemm_finish_norm)
+    void* post_x;      // or null: the rows [M, post_ld] that become the norm of post_alpha x themselves + the product (EPI_STORE)
+    int post_ld;
+    float post_alpha;
 };
+
+// what a plain product's results pass before they are stored
+#define XR_POST_NONE 0
+#define XR_POST_RELU2 1
+__device__ inline float post_act(const GemmArgs& g, float v) {
+    if (g.epi == EPI_STORE && g.act == XR_POST_RELU2) { v = fmaxf(v, 0.f); v *= v; }
+    return v;
+}
 
 __device__ inline uint4 ldg16(const bf16_t* p) { return *reinterpret_cast<const uint4*>(p); }
 // streaming load: the weights of a decode step are read once and must not push the
@@ -143,6 +159,7 @@ __device__ inline uint4 keep_if(bool ok, uint4 v) {
 }
 __device__ inline void store_out(const GemmArgs& g, int m, int n, float v) {
     size_t o = (size_t)m * g.ldo + n;
+    v = post_act(g, v);
     if (g.epi == EPI_ACCUM) {
         float* p = (float*)g.out;
         p[o] = p[o] + v;
@@ -873,6 +890,10 @@ __device__ __forceinline__ void gemm_tile(const GemmArgs& g, const int item, uin
                 const float b = g.bias && col < g.N ? g.bias[col] : 0.f;
 #pragma unroll
                 for (int e = 0; e < 16; ++e) t[n][e] = acc[i][j + n][e] + b;
+                if (g.epi == EPI_STORE && g.act == XR_POST_RELU2) {
+#pragma unroll
+                    for (int e = 0; e < 16; ++e) { const float v = fmaxf(t[n][e], 0.f); t[n][e] = v * v; }
+                }
             }
             if (rotate)
                 rope_tiles<NTP>(stage, t, g.rope, m0 + wm0 + i * 32, g.M, bx * BN + wn0 + j * 32, g.N, lane);
@@ -956,7 +977,8 @@ __global__ __launch_bounds__(1024) void k_gemm_finish_norm(GemmArgs g) {
     __shared__ float rstd_s, mean_s;
     const int m = blockIdx.x, tid = threadIdx.x;
     const size_t step = (size_t)g.M * g.N;
-    float* xrow = (float*)g.out + (size_t)m * g.ldo;
+    float* xrow = g.post_x ? g.post_x + (size_t)m * g.post_ld : (float*)g.out + (size_t)m * g.ldo;
+    const float keep = g.post_x ? g.post_alpha : 1.0f;
     float sq = 0.f;
     for (int n = tid * 4; n < g.N; n += 1024 * 4) {
         const float* p = g.partial + (size_t)m * g.N + n;
@@ -971,7 +993,7 @@ __global__ __launch_bounds__(1024) void k_gemm_finish_norm(GemmArgs g) {
         }
         if (g.bias) { v.x += g.bias[n]; v.y += g.bias[n + 1]; v.z += g.bias[n + 2]; v.w += g.bias[n + 3]; }
         float4 x = *reinterpret_cast<const float4*>(xrow + n);
-        x.x += v.x; x.y += v.y; x.z += v.z; x.w += v.w;
+        x.x = fmaf(keep, x.x, v.x); x.y = fmaf(keep, x.y, v.y); x.z = fmaf(keep, x.z, v.z); x.w = fmaf(keep, x.w, v.w);
         *reinterpret_cast<float4*>(xrow + n) = x;
         sq += g.norm_centred ? x.x + x.y + x.z + x.w : x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
     }
@@ -1012,10 +1034,9 @@ __global__ __launch_bounds__(1024) void k_gemm_finish_norm(GemmArgs g) {
 #pragma unroll
         for (int i = 0; i < 4; ++i)
             w[i] = g.norm_w_bf16 ? bf16_to_f32(((const bf16_t*)g.norm_w)[n + i]) : ((const float*)g.norm_w)[n + i];
-        uint2 o;
-        o.x = pack_bf16x2((x.x - mean) * rstd * w[0], (x.y - mean) * rstd * w[1]);
-        o.y = pack_bf16x2((x.z - mean) * rstd * w[2], (x.w - mean) * rstd * w[3]);
-        *reinterpret_cast<uint2*>(g.xg + (size_t)m * g.N + n) = o;
+        const float4 y = make_float4((x.x - mean) * rstd * w[0], (x.y - mean) * rstd * w[1], (x.z - mean) * rstd * w[2], (x.w - mean) * rstd * w[3]);
+        if (g.post_x) *reinterpret_cast<float4*>(xrow + n) = y;
+        *reinterpret_cast<uint2*>(g.xg + (size_t)m * g.N + n) = make_uint2(pack_bf16x2(y.x, y.y), pack_bf16x2(y.z, y.w));
     }
 }
 
@@ -1404,6 +1425,7 @@ extern "C" int xr_gemm_bf16(void* out, const void* a, const void* w, const float
     XR_REQUIRE(((uintptr_t)a % 16) == 0 && ((uintptr_t)w % 16) == 0, "gemm: operands must be 16-byte aligned");
     XR_REQUIRE(epi >= 0 && epi <= 2, "gemm: unknown epilogue %d", epi);
     XR_REQUIRE(epi != EPI_GATED || (act >= 0 && act < XR_ACT_COUNT), "gemm: unknown activation code %d", act);
+    XR_REQUIRE(epi == EPI_GATED || act == XR_POST_NONE || (epi == EPI_STORE && act == XR_POST_RELU2 && !rope && !norm), "gemm: activation %d of a plain product", act);
     XR_REQUIRE(!(w_packed && epi == EPI_GATED && N % 16), "gemm: packed gate and up rows need a width that is a multiple of 16, got %d", N);
     XR_REQUIRE(epi != EPI_ACCUM || out_dtype == XR_F32, "gemm: accumulation needs a 32-bit output");
     XR_REQUIRE(out_dtype == XR_F32 || out_dtype == XR_BF16, "gemm: bad output dtype %d", out_dtype);
@@ -1416,6 +1438,7 @@ extern "C" int xr_gemm_bf16(void* out, const void* a, const void* w, const float
     bool want_whole_norm = false;      // a norm after a product of more than 16 rows is asked for and possible
     g.ss_in = nullptr; g.n_ss = 0; g.ss_inv_width = 0.f; g.ss_eps = 0.f;
     g.norm_w = nullptr; g.norm_w_bf16 = 0; g.xg = nullptr; g.ss_out = nullptr;
+    g.post_x = nullptr; g.post_ld = 0; g.post_alpha = 1.0f;
     if (norm) {
         XR_REQUIRE(variant == 0, "gemm: a norm is folded only into a product whose kernel the library chooses");
         XR_REQUIRE(M <= 16 || !norm->ss_in, "gemm: rows that lack their norm's scale: at most 16, got %d", M);
@@ -1424,7 +1447,13 @@ extern "C" int xr_gemm_bf16(void* out, const void* a, const void* w, const float
             g.ss_in = norm->ss_in; g.n_ss = norm->n_ss; g.ss_inv_width = norm->ss_inv_width; g.ss_eps = norm->ss_eps;
         }
         if (norm->xg) {
-            XR_REQUIRE(epi == EPI_ACCUM && norm->norm_w, "gemm: the norm after a product needs the accumulating epilogue and a weight");
+            XR_REQUIRE(epi == (norm->post_x ? EPI_STORE : EPI_ACCUM) && norm->norm_w,
+                       "gemm: the norm after a product needs the accumulating epilogue (or rows of its own to replace) and a weight");
+            if (norm->post_x) {
+                XR_REQUIRE(M > 16 && out_dtype == XR_F32 && !rope && norm->post_ld >= N && norm->post_ld % 4 == 0 && ((uintptr_t)norm->post_x % 16) == 0,
+                           "gemm: rows that become a norm: more than 16, 16-byte aligned, %d apart", norm->post_ld);
+                g.post_x = (float*)norm->post_x; g.post_ld = norm->post_ld; g.post_alpha = norm->post_alpha;
+            }
             XR_REQUIRE(M > 16 || (norm->ss_out && norm->ss_out_rows >= (N + 15) / 16),
                        "gemm: room for %d partial sums of squares, %d needed", norm->ss_out ? norm->ss_out_rows : 0, (N + 15) / 16);
             XR_REQUIRE(!norm->centred || M > 16, "gemm: a layer norm after a product of %d rows: from 17 rows on", M);

@@ -364,15 +364,19 @@ extern "C" int xr_heads_gemm_bf16(void* out, const void* a, const void* w, int T
 // ---------------------------------------------------------------- the experts' rows, sorted by expert
 // A = T * top choices idx[a] (a = token * top + j).  One workgroup: counts, offsets, the list `perm` of
 // the choices expert by expert (in any order inside an expert: a row's result does not depend on
-// its place), and the tiles of `bm` rows: tile_group / tile_start / tile_count, n_tiles[0] of them.
+// its place), and the tiles of `bm` rows: tile_group / tile_start / tile_count, n_tiles[0] of them.  Choices
+// n .. n + n_id - 1 (identity experts) have no product: they are in no list.
 #define SORT_MAX_EXPERTS 1024
-__global__ __launch_bounds__(1024) void k_moe_sort(const int* __restrict__ idx, int A, int n, int bm, int* __restrict__ perm,
+__global__ __launch_bounds__(1024) void k_moe_sort(const int* __restrict__ idx, int A, int n, int n_id, int bm, int* __restrict__ perm,
                                                     int* __restrict__ tile_group, int* __restrict__ tile_start,
                                                     int* __restrict__ tile_count, int* __restrict__ n_tiles) {
     __shared__ int count[SORT_MAX_EXPERTS], offset[SORT_MAX_EXPERTS], cursor[SORT_MAX_EXPERTS];
     for (int e = threadIdx.x; e < n; e += 1024) { count[e] = 0; cursor[e] = 0; }
     __syncthreads();
-    for (int a = threadIdx.x; a < A; a += 1024) atomicAdd(&count[min(max(idx[a], 0), n - 1)], 1);
+    for (int a = threadIdx.x; a < A; a += 1024) {
+        const int e = min(max(idx[a], 0), n + n_id - 1);
+        if (e < n) atomicAdd(&count[e], 1);
+    }
     __syncthreads();
     if (threadIdx.x == 0) {
         int at = 0, t = 0;
@@ -390,19 +394,25 @@ __global__ __launch_bounds__(1024) void k_moe_sort(const int* __restrict__ idx, 
     }
     __syncthreads();
     for (int a = threadIdx.x; a < A; a += 1024) {
-        const int e = min(max(idx[a], 0), n - 1);
-        perm[offset[e] + atomicAdd(&cursor[e], 1)] = a;
+        const int e = min(max(idx[a], 0), n + n_id - 1);
+        if (e < n) perm[offset[e] + atomicAdd(&cursor[e], 1)] = a;
     }
 }
 
-// y[t] (+)= sum_j wts[t][j] * yz[t * top + j], in the order of the choice  (+ g_side[t] * y_side[t])
+// y[t] (+)= sum_j wts[t][j] * yz[t * top + j], in the order of the choice  (+ g_side[t] * y_side[t]); an identity expert's
+// place takes the token's row h instead.  With `accumulate` the old y counts alpha times.
 struct CombineArgs {
     float* y;
     const float* yz;
     const float* wts;
     int E, ld_y, top, accumulate;
     const float* y_side;    // [T, E], or null
-    const float* g_side;    // [T]
+    const float* g_side;    // [T], or null (the rows beside count as they are)
+    float alpha;
+    const int* idx;         // the choice, where it may name an identity expert (n_exp and up); else null
+    const bf16_t* x;        // [T, ld_x]: the rows themselves
+    int n_exp, ld_x;
+    int replace;            // 1: the norm takes the rows' place in y as well
     // the norm of the finished row (k_moe_combine_norm): times w, to h [T, E]
     const void* norm_w;
     int norm_w_bf16, centred;
@@ -415,10 +425,13 @@ __global__ void k_moe_combine(CombineArgs a, size_t n) {
     const size_t t = i / a.E;
     const int c = (int)(i - t * a.E);
     float s = 0.f;
-    for (int j = 0; j < a.top; ++j) s += a.wts[t * a.top + j] * a.yz[(t * a.top + j) * a.E + c];
-    if (a.y_side) s = fmaf(a.g_side[t], a.y_side[i], s);
+    for (int j = 0; j < a.top; ++j) {
+        const bool self = a.idx && a.idx[t * a.top + j] >= a.n_exp;
+        s += a.wts[t * a.top + j] * (self ? bf16_to_f32(a.x[t * a.ld_x + c]) : a.yz[(t * a.top + j) * a.E + c]);
+    }
+    if (a.y_side) s = fmaf(a.g_side ? a.g_side[t] : 1.f, a.y_side[i], s);
     float* o = a.y + t * a.ld_y + c;
-    *o = a.accumulate ? *o + s : s;
+    *o = a.accumulate ? fmaf(a.alpha, *o, s) : s;
 }
 
 // The same with 4 columns a thread, a workgroup a row, and behind it, if asked for, the RMS or layer norm (`centred`) of
@@ -440,6 +453,18 @@ __global__ __launch_bounds__(256) void k_moe_combine_norm(CombineArgs a) {
     for (int i = 0; i < NV; ++i) v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
     for (int j = 0; j < a.top; ++j) {
         const float w = a.wts[t * a.top + j];
+        if (a.idx && a.idx[t * a.top + j] >= a.n_exp) {
+            const bf16_t* r = a.x + t * a.ld_x;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                const int c = threadIdx.x + i * 256;
+                if (c >= n4) continue;
+                const uint2 x = *reinterpret_cast<const uint2*>(r + 4 * c);
+                v[i].x += w * __uint_as_float(x.x << 16); v[i].y += w * __uint_as_float(x.x & 0xffff0000u);
+                v[i].z += w * __uint_as_float(x.y << 16); v[i].w += w * __uint_as_float(x.y & 0xffff0000u);
+            }
+            continue;
+        }
         const float4* r = reinterpret_cast<const float4*>(a.yz + (t * a.top + j) * a.E);
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
@@ -450,7 +475,7 @@ __global__ __launch_bounds__(256) void k_moe_combine_norm(CombineArgs a) {
         }
     }
     float4* y = reinterpret_cast<float4*>(a.y + t * a.ld_y);
-    const float gs = a.y_side ? a.g_side[t] : 0.f;
+    const float gs = a.g_side ? a.g_side[t] : 1.f;
     const float4* side = reinterpret_cast<const float4*>(a.y_side + (a.y_side ? t * a.E : 0));
     float s = 0.f;
 #pragma unroll
@@ -463,9 +488,10 @@ __global__ __launch_bounds__(256) void k_moe_combine_norm(CombineArgs a) {
         }
         if (a.accumulate) {
             const float4 x = y[c];
-            v[i].x += x.x; v[i].y += x.y; v[i].z += x.z; v[i].w += x.w;
+            v[i].x = fmaf(a.alpha, x.x, v[i].x); v[i].y = fmaf(a.alpha, x.y, v[i].y);
+            v[i].z = fmaf(a.alpha, x.z, v[i].z); v[i].w = fmaf(a.alpha, x.w, v[i].w);
         }
-        y[c] = v[i];
+        if (!a.replace) y[c] = v[i];
         s += a.centred ? v[i].x + v[i].y + v[i].z + v[i].w : v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
     }
     if (!a.h) return;
@@ -489,8 +515,9 @@ __global__ __launch_bounds__(256) void k_moe_combine_norm(CombineArgs a) {
         float w[4];
 #pragma unroll
         for (int e = 0; e < 4; ++e) w[e] = a.norm_w_bf16 ? bf16_to_f32(((const bf16_t*)a.norm_w)[4 * c + e]) : ((const float*)a.norm_w)[4 * c + e];
-        *reinterpret_cast<uint2*>(a.h + t * a.E + 4 * c) = make_uint2(pack_bf16x2(v[i].x * rinv * w[0], v[i].y * rinv * w[1]),
-                                                                     pack_bf16x2(v[i].z * rinv * w[2], v[i].w * rinv * w[3]));
+        const float4 o = make_float4(v[i].x * rinv * w[0], v[i].y * rinv * w[1], v[i].z * rinv * w[2], v[i].w * rinv * w[3]);
+        if (a.replace) y[c] = o;
+        *reinterpret_cast<uint2*>(a.h + t * a.E + 4 * c) = make_uint2(pack_bf16x2(o.x, o.y), pack_bf16x2(o.z, o.w));
     }
 }
 #define COMBINE_MAX_E (4 * 256 * 8)
@@ -507,22 +534,24 @@ struct XrRowNorm {
     int w_bf16, centred;
     float eps;
     void* h;
+    int replace;        // 1: the old rows count alpha times in the sum, and the norm takes the rows' place as well
+    float alpha;
 };
 extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch, const void* h, const void* w_up,
                                       const void* w_down, const int* idx, const float* wts, int T, int E, int F, int ld_h,
                                       int ld_y, int n, int top, int accumulate, int gated, int gate, float param, const float* y_side,
-                                      const float* g_side, const XrRowNorm* norm, hipStream_t stream) {
+                                      const float* g_side, const XrRowNorm* norm, int n_id, hipStream_t stream) {
     XR_REQUIRE(gate >= 0 && gate < XR_ACT_COUNT, "moe_experts_grouped: unknown gate %d", gate);
-    XR_REQUIRE(!y_side == !g_side, "moe_experts_grouped: rows beside the experts come with a weight a row");
+    XR_REQUIRE(y_side || !g_side, "moe_experts_grouped: weights of rows beside the experts without the rows");
     XR_REQUIRE(T >= 0 && E > 0 && F > 0 && ld_h >= E && ld_y >= E, "moe_experts_grouped: bad sizes T=%d E=%d F=%d", T, E, F);
-    XR_REQUIRE(n >= 1 && n <= SORT_MAX_EXPERTS && top >= 1 && top <= n, "moe_experts_grouped: %d experts (at most %d), %d chosen", n,
-               SORT_MAX_EXPERTS, top);
+    XR_REQUIRE(n >= 1 && n_id >= 0 && n <= SORT_MAX_EXPERTS && top >= 1 && top <= n + n_id, "moe_experts_grouped: %d experts (at most %d) and %d that are the identity, %d chosen",
+               n, SORT_MAX_EXPERTS, n_id, top);
     XR_REQUIRE((long long)T * top <= (1 << 24), "moe_experts_grouped: too many rows");
     const int Fu = gated ? 2 * F : F;          // rows of an expert's first matrix
     XR_REQUIRE(grouped_operands_ok(h, w_up, E, ld_h, 0, (long long)Fu * E) && grouped_operands_ok(z, w_down, F, F, 0, (long long)E * F),
                "moe_experts_grouped: widths and row strides must be multiples of 8 and the operands 16-byte aligned");
     const bool rows4 = E % 4 == 0 && ld_y % 4 == 0 && E <= COMBINE_MAX_E && ((uintptr_t)y % 16) == 0 && ((uintptr_t)yz % 16) == 0 &&
-                       ((uintptr_t)y_side % 16) == 0;
+                       ((uintptr_t)y_side % 16) == 0 && (n_id == 0 || ((uintptr_t)h % 8 == 0 && ld_h % 4 == 0));
     XR_REQUIRE(!norm || (rows4 && norm->w && norm->h), "moe_experts_grouped: the norm behind the sum takes widths that are multiples of 4 up to %d, got %d",
                COMBINE_MAX_E, E);
     if (T == 0) return XR_OK;
@@ -536,7 +565,7 @@ extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch
     int* tile_start = tile_group + max_tiles;
     int* tile_count = tile_start + max_tiles;
     int* n_tiles = tile_count + max_tiles;
-    k_moe_sort<<<1, 1024, 0, stream>>>(idx, A, n, bm, perm, tile_group, tile_start, tile_count, n_tiles);
+    k_moe_sort<<<1, 1024, 0, stream>>>(idx, A, n, n_id, bm, perm, tile_group, tile_start, tile_count, n_tiles);
     GroupedArgs g{};
     g.perm = perm; g.tile_group = tile_group; g.tile_start = tile_start; g.tile_count = tile_count; g.n_tiles = n_tiles;
     g.a_group_stride = 0; g.o_group_stride = 0;
@@ -549,7 +578,8 @@ extern "C" int xr_moe_experts_grouped(float* y, void* z, float* yz, int* scratch
     g.a = (const bf16_t*)z; g.lda = F; g.w = (const bf16_t*)w_down; g.w_group_stride = (long long)E * F; g.out = yz; g.ldo = E;
     g.N = E; g.K = F; g.out_bf16 = 0; g.act = GM_ACT_NONE; g.gather_div = 1;
     launch_grouped(g, max_tiles, bm, stream);
-    CombineArgs c{y, yz, wts, E, ld_y, top, accumulate, y_side, g_side, nullptr, 0, 0, 0.f, nullptr};
+    CombineArgs c{y, yz, wts, E, ld_y, top, accumulate, y_side, g_side, 1.f, n_id ? idx : nullptr, (const bf16_t*)h, n, ld_h, 0, nullptr, 0, 0, 0.f, nullptr};
+    if (norm && norm->replace) { c.replace = 1; c.alpha = norm->alpha; c.accumulate = 1; }
     if (norm) { c.norm_w = norm->w; c.norm_w_bf16 = norm->w_bf16; c.centred = norm->centred; c.eps = norm->eps; c.h = (bf16_t*)norm->h; }
     if (!rows4) {
         const size_t cnt = (size_t)T * E;

@@ -11,6 +11,8 @@
 //                    a weight (the norm that the next sublayer reads through) in the same pass.
 // k_add_rows:        x[t] += s y[t] + v, a vector added to every row (y absent: the vector alone).
 // k_softcap:         x <- cap tanh(x / cap) in place on 32-bit rows.
+// k_post_norm:       x <- norm(alpha x + y) of 32-bit rows (an RMS norm with a weight), and a copy of the new rows in the
+//                    type that products take: a residual stream that is normed behind every sum.
 // k_attn_extra_partial: for the matrix-core attention kernels, which take a window's (or a chunk's) keys: what else
 //                    enters the same softmax, as a partial result of its own that their merge adds: a sink (a score
 //                    without key or value, one a head) and the first `keep` keys of the request where the
@@ -296,5 +298,88 @@ extern "C" int xr_softcap(float* x, int R, int W, int ld, float cap, hipStream_t
     if (n == 0) return XR_OK;
     k_softcap<<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(x, W, ld, n, cap, 1.0f / cap);
     XR_CHECK_LAUNCH("softcap");
+    return XR_OK;
+}
+
+// A workgroup of NW waves a row.  VEC: a thread keeps its float4 pieces (NV of them) in registers from the sum to the
+// store; else the sum is stored into x on the first pass and read back, each thread what it wrote itself.
+template <typename TO, int NW, int NV, bool VEC>
+__global__ __launch_bounds__(64 * NW) void k_post_norm(float* __restrict__ x, const float* __restrict__ y,
+                                                      const float* __restrict__ w, TO* __restrict__ h, int E, int ld_x,
+                                                      float alpha, float eps) {
+    constexpr int NT = 64 * NW;
+    __shared__ float part[NW];
+    const int t = blockIdx.x;
+    float* xr = x + (size_t)t * ld_x;
+    const float* yr = y + (size_t)t * E;
+    float4 v[VEC ? NV : 1];
+    float ss = 0.f;
+    if (VEC) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int c = threadIdx.x + i * NT;
+            v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (4 * c < E) {
+                const float4 a = reinterpret_cast<const float4*>(xr)[c], b = reinterpret_cast<const float4*>(yr)[c];
+                v[i] = make_float4(fmaf(alpha, a.x, b.x), fmaf(alpha, a.y, b.y), fmaf(alpha, a.z, b.z), fmaf(alpha, a.w, b.w));
+            }
+            ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+        }
+    } else {
+        for (int c = threadIdx.x; c < E; c += NT) {
+            const float a = fmaf(alpha, xr[c], yr[c]);
+            xr[c] = a;
+            ss = fmaf(a, a, ss);
+        }
+    }
+    ss = wave_sum(ss);
+    if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = ss;
+    __syncthreads();
+    float tot = 0.f;
+#pragma unroll
+    for (int i = 0; i < NW; ++i) tot += part[i];
+    const float f = 1.0f / sqrtf(tot / (float)E + eps);
+    if (VEC) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int c = threadIdx.x + i * NT;
+            if (4 * c >= E) continue;
+            const float4 g = reinterpret_cast<const float4*>(w)[c];
+            const float4 o = make_float4(v[i].x * f * g.x, v[i].y * f * g.y, v[i].z * f * g.z, v[i].w * f * g.w);
+            reinterpret_cast<float4*>(xr)[c] = o;
+            if constexpr (sizeof(TO) == 4) reinterpret_cast<float4*>((float*)h + (size_t)t * E)[c] = o;
+            else *reinterpret_cast<uint2*>((bf16_t*)h + (size_t)t * E + 4 * c) = make_uint2(pack_bf16x2(o.x, o.y), pack_bf16x2(o.z, o.w));
+        }
+    } else {
+        for (int c = threadIdx.x; c < E; c += NT) {
+            const float o = xr[c] * f * w[c];
+            xr[c] = o;
+            st<TO>(h, (size_t)t * E + c, o);
+        }
+    }
+}
+
+extern "C" int xr_post_norm(float* x, const float* y, const float* w, void* h, int T, int E, int ld_x, float alpha, float eps,
+                            int h_dtype, hipStream_t stream) {
+    XR_REQUIRE(T >= 0 && E > 0 && ld_x >= E && eps >= 0.f, "post_norm: bad sizes T=%d E=%d ld=%d eps=%g", T, E, ld_x, (double)eps);
+    XR_REQUIRE(x && y && w && h && (h_dtype == XR_F32 || h_dtype == XR_BF16), "post_norm: an operand is missing, or output type %d", h_dtype);
+    if (T == 0) return XR_OK;
+    auto on16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };
+    const bool vec = E % 4 == 0 && ld_x % 4 == 0 && on16(x) && on16(y) && on16(w) && on16(h) && E <= 4 * 256 * 8;
+    const bool few = T <= 128 && E >= 1024;         // the few rows of a decode step: the latency of one workgroup's pass
+#define PN(TO)                                                                                                          \
+    do {                                                                                                                \
+        TO* o = (TO*)h;                                                                                                 \
+        if (!vec) k_post_norm<TO, 4, 1, false><<<T, 256, 0, stream>>>(x, y, w, o, E, ld_x, alpha, eps);                  \
+        else if (few && E <= 4096) k_post_norm<TO, 16, 1, true><<<T, 1024, 0, stream>>>(x, y, w, o, E, ld_x, alpha, eps); \
+        else if (few) k_post_norm<TO, 16, 2, true><<<T, 1024, 0, stream>>>(x, y, w, o, E, ld_x, alpha, eps);             \
+        else if (E <= 4 * 256 * 2) k_post_norm<TO, 4, 2, true><<<T, 256, 0, stream>>>(x, y, w, o, E, ld_x, alpha, eps);  \
+        else if (E <= 4 * 256 * 4) k_post_norm<TO, 4, 4, true><<<T, 256, 0, stream>>>(x, y, w, o, E, ld_x, alpha, eps);  \
+        else k_post_norm<TO, 4, 8, true><<<T, 256, 0, stream>>>(x, y, w, o, E, ld_x, alpha, eps);                        \
+    } while (0)
+    if (h_dtype == XR_BF16) PN(bf16_t);
+    else PN(float);
+#undef PN
+    XR_CHECK_LAUNCH("post_norm");
     return XR_OK;
 }

@@ -4,7 +4,7 @@
 // all experts, the `top` experts with the largest score + correction (ties: the lower index), and
 // their weights: the chosen scores (without the correction) over their sum + 1e-20.  Options: the scores are
 // sigmoid(logit), every expert for itself, instead of a softmax; the experts form `groups` equal groups of
-// neighbours, a group's score is the sum of its two largest score + correction, and only experts of the `keep`
+// neighbours, a group's score is the sum of its two largest score + correction (or the largest alone), and only experts of the `keep`
 // groups that score highest can be chosen (ties: the lower group); the weights are the chosen scores times a
 // given number instead of their share of their sum; or the choice is by logit + correction (the router's bias) and
 // the weights are the softmax of these over the chosen experts.  `side` given: column n of a token's logits is no
@@ -13,8 +13,9 @@
 // weights of the chosen experts streamed: what a few decoded tokens need.  Expert:
 // down(act(up h)), act = relu squared, or gated: down(value(gate h, up h)) with a gate of common.h (SiLU: silu(g) u)
 // and the gate's rows before the up rows in one matrix [2F, E].  The down product adds a token's experts up in the order
-// of its choice, then rows that come from elsewhere times the token's weight for them (a shared expert's), and writes
-// (or adds to) 32-bit rows.
+// of its choice, then rows that come from elsewhere times the token's weight for them (a shared expert's; without weights
+// they count as they are), and writes (or adds to) 32-bit rows.  Choices n .. n + n_id - 1 are identity experts: their output
+// is the token's row h itself.
 // k_moe_table_route: the choice without a router, a row of a table [vocab, top] by the token's id, every
 // chosen expert with the same weight.
 #include "common.h"
@@ -29,7 +30,7 @@
 __global__ __launch_bounds__(64) void k_moe_route(int* __restrict__ idx, float* __restrict__ wts, float* __restrict__ side,
                                                   const float* __restrict__ logits,
                                                   const float* __restrict__ correction, int ld, int n, int top, int scores,
-                                                  int groups, int keep, float weight_scale) {
+                                                  int groups, int keep, float weight_scale, int group_max) {
     __shared__ float z[MOE_MAX_EXPERTS];
     __shared__ float gsc[MOE_MAX_EXPERTS];          // a group's score; then 1 if its experts can be chosen, else 0
     const int t = blockIdx.x, lane = threadIdx.x;
@@ -97,7 +98,7 @@ __global__ __launch_bounds__(64) void k_moe_route(int* __restrict__ idx, float* 
                 if (!(c == c)) c = -INFINITY;
                 if (c > a) { b = a; a = c; } else if (c > b) b = c;
             }
-            gsc[g] = per > 1 ? a + b : a;
+            gsc[g] = per > 1 && !group_max ? a + b : a;
         }
         __syncthreads();
         float mine_g[MOE_MAX_EXPERTS / 64];
@@ -154,7 +155,7 @@ __global__ __launch_bounds__(64) void k_moe_route(int* __restrict__ idx, float* 
 }
 
 extern "C" int xr_moe_route(int* idx, float* wts, float* side, const float* logits, const float* correction, int T, int ld, int n,
-                            int top, int scores, int groups, int keep, float weight_scale, hipStream_t stream) {
+                            int top, int scores, int groups, int keep, float weight_scale, int group_max, hipStream_t stream) {
     XR_REQUIRE(T >= 0 && ld >= n + (side ? 1 : 0), "moe_route: bad sizes T=%d ld=%d", T, ld);
     XR_REQUIRE(scores >= MOE_SCORES_SOFTMAX && scores <= MOE_SCORES_LOGITS, "moe_route: unknown scores %d", scores);
     XR_REQUIRE(scores != MOE_SCORES_LOGITS || (groups == 1 && weight_scale == 0.f), "moe_route: a choice by the logits has no groups and no weight scale");
@@ -164,7 +165,7 @@ extern "C" int xr_moe_route(int* idx, float* wts, float* side, const float* logi
                "moe_route: %d experts in %d groups of which %d are kept cannot give %d choices", n, groups, keep, top);
     XR_REQUIRE(weight_scale >= 0.f, "moe_route: weight scale %g (0: the chosen scores' shares of their sum)", (double)weight_scale);
     if (T == 0) return XR_OK;
-    k_moe_route<<<T, 64, 0, stream>>>(idx, wts, side, logits, correction, ld, n, top, scores, groups, keep, weight_scale);
+    k_moe_route<<<T, 64, 0, stream>>>(idx, wts, side, logits, correction, ld, n, top, scores, groups, keep, weight_scale, group_max);
     XR_CHECK_LAUNCH("moe_route");
     return XR_OK;
 }
@@ -229,11 +230,12 @@ template <> __device__ inline float wave_dot<bf16_t>(const bf16_t* __restrict__ 
 #define MOE_ACT_GATED 1
 template <typename TW>
 __global__ __launch_bounds__(256) void k_moe_up(TW* __restrict__ z, const TW* __restrict__ h, const TW* __restrict__ w_up,
-                                                const int* __restrict__ idx, int E, int F, int ld_h, int top, int n, int vec,
+                                                const int* __restrict__ idx, int E, int F, int ld_h, int top, int n, int n_id, int vec,
                                                 int gated, int gate, float param) {
     const int a = blockIdx.x, f = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (f >= F) return;
-    const int t = a / top, e = min(max(idx[a], 0), n - 1);
+    const int t = a / top, e = min(max(idx[a], 0), n + n_id - 1);
+    if (e >= n) return;             // an identity expert: nothing to multiply
     const TW* row = h + (size_t)t * ld_h;
     const TW* w = w_up + ((size_t)e * (gated ? 2 * F : F) + f) * E;
     const float acc = wave_dot<TW>(w, row, E, lane, vec != 0);
@@ -252,19 +254,24 @@ __global__ __launch_bounds__(256) void k_moe_up(TW* __restrict__ z, const TW* __
 template <typename TW>
 __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const TW* __restrict__ z, const TW* __restrict__ w_down,
                                                   const int* __restrict__ idx, const float* __restrict__ wts, int E, int F,
-                                                  int ld_y, int top, int n, int accumulate, int vec,
-                                                  const float* __restrict__ y_side, const float* __restrict__ g_side) {
+                                                  int ld_y, int top, int n, int n_id, int accumulate, int vec,
+                                                  const float* __restrict__ y_side, const float* __restrict__ g_side,
+                                                  const TW* __restrict__ h, int ld_h) {
     const int t = blockIdx.x, c = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (c >= E) return;
     float sum = 0.f;
     for (int j = 0; j < top; ++j) {
-        const int e = min(max(idx[(size_t)t * top + j], 0), n - 1);
+        const int e = min(max(idx[(size_t)t * top + j], 0), n + n_id - 1);
+        if (e >= n) {
+            sum = fmaf(wts[(size_t)t * top + j], ld<TW>(h, (size_t)t * ld_h + c), sum);
+            continue;
+        }
         const TW* w = w_down + ((size_t)e * E + c) * F;
         const TW* zr = z + ((size_t)t * top + j) * F;
         sum += wts[(size_t)t * top + j] * wave_dot<TW>(w, zr, F, lane, vec != 0);
     }
     if (lane == 0) {
-        if (y_side) sum = fmaf(g_side[t], y_side[(size_t)t * E + c], sum);
+        if (y_side) sum = fmaf(g_side ? g_side[t] : 1.f, y_side[(size_t)t * E + c], sum);
         float* o = y + (size_t)t * ld_y + c;
         *o = accumulate ? *o + sum : sum;
     }
@@ -272,14 +279,14 @@ __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const T
 
 extern "C" int xr_moe_experts(float* y, void* z, const void* h, const void* w_up, const void* w_down, const int* idx,
                               const float* wts, int T, int E, int F, int ld_h, int ld_y, int n, int top, int accumulate,
-                              int dtype, int act, int gate, float param, const float* y_side, const float* g_side,
+                              int dtype, int act, int gate, float param, const float* y_side, const float* g_side, int n_id,
                               hipStream_t stream) {
     XR_REQUIRE(act == MOE_ACT_RELU2 || act == MOE_ACT_GATED, "moe_experts: activation %d (0 = relu squared, 1 = gated)", act);
     XR_REQUIRE(gate >= 0 && gate < XR_ACT_COUNT, "moe_experts: unknown gate %d", gate);
-    XR_REQUIRE(!y_side == !g_side, "moe_experts: rows beside the experts come with a weight a row");
+    XR_REQUIRE(y_side || !g_side, "moe_experts: weights of rows beside the experts without the rows");
     const int gated = act == MOE_ACT_GATED;
     XR_REQUIRE(T >= 0 && E > 0 && F > 0 && ld_h >= E && ld_y >= E, "moe_experts: bad sizes T=%d E=%d F=%d", T, E, F);
-    XR_REQUIRE(n >= 1 && top >= 1 && top <= n && top <= MOE_MAX_TOP, "moe_experts: %d experts, %d chosen", n, top);
+    XR_REQUIRE(n >= 1 && n_id >= 0 && top >= 1 && top <= n + n_id && top <= MOE_MAX_TOP, "moe_experts: %d experts (and %d that are the identity), %d chosen", n, n_id, top);
     XR_REQUIRE((long long)T * top <= 0x7fffffffLL, "moe_experts: too many rows");
     if (T == 0) return XR_OK;
     const dim3 gu(T * top, (F + 3) / 4), gd(T, (E + 3) / 4);
@@ -287,11 +294,11 @@ extern "C" int xr_moe_experts(float* y, void* z, const void* h, const void* w_up
     const bool al = ((uintptr_t)h % 16) == 0 && ((uintptr_t)w_up % 16) == 0 && ((uintptr_t)w_down % 16) == 0 && ((uintptr_t)z % 16) == 0;
     const int vu = al && E % per16 == 0 && ld_h % per16 == 0, vd = al && F % per16 == 0;
     if (dtype == XR_F32) {
-        k_moe_up<float><<<gu, 256, 0, stream>>>((float*)z, (const float*)h, (const float*)w_up, idx, E, F, ld_h, top, n, vu, gated, gate, param);
-        k_moe_down<float><<<gd, 256, 0, stream>>>(y, (const float*)z, (const float*)w_down, idx, wts, E, F, ld_y, top, n, accumulate, vd, y_side, g_side);
+        k_moe_up<float><<<gu, 256, 0, stream>>>((float*)z, (const float*)h, (const float*)w_up, idx, E, F, ld_h, top, n, n_id, vu, gated, gate, param);
+        k_moe_down<float><<<gd, 256, 0, stream>>>(y, (const float*)z, (const float*)w_down, idx, wts, E, F, ld_y, top, n, n_id, accumulate, vd, y_side, g_side, (const float*)h, ld_h);
     } else if (dtype == XR_BF16) {
-        k_moe_up<bf16_t><<<gu, 256, 0, stream>>>((bf16_t*)z, (const bf16_t*)h, (const bf16_t*)w_up, idx, E, F, ld_h, top, n, vu, gated, gate, param);
-        k_moe_down<bf16_t><<<gd, 256, 0, stream>>>(y, (const bf16_t*)z, (const bf16_t*)w_down, idx, wts, E, F, ld_y, top, n, accumulate, vd, y_side, g_side);
+        k_moe_up<bf16_t><<<gu, 256, 0, stream>>>((bf16_t*)z, (const bf16_t*)h, (const bf16_t*)w_up, idx, E, F, ld_h, top, n, n_id, vu, gated, gate, param);
+        k_moe_down<bf16_t><<<gd, 256, 0, stream>>>(y, (const bf16_t*)z, (const bf16_t*)w_down, idx, wts, E, F, ld_y, top, n, n_id, accumulate, vd, y_side, g_side, (const bf16_t*)h, ld_h);
     } else { xr_set_error("moe_experts: bad dtype %d", dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("moe_experts");
     return XR_OK;

@@ -68,7 +68,9 @@ _PROTOS = {
     "xr_gemm_bf16": [_p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p, _sz, _p, _p, _p],
     "xr_pack_weight": [_p, _p, _i, _i, _p],
     "xr_rope_table": [_p, _p, _p, _i, _i, _f, _p],
-    "xr_attention_ref": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p, _p, _f, _p],
+    "xr_attention_ref": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p, _p, _f, _p, _i, _f, _i, _p],
+    "xr_head_norm_rope_write": [_p, _p, _p, _i, _p, _p, _f, _i, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p],
+    "xr_post_norm": [_p, _p, _p, _p, _i, _i, _i, _f, _f, _i, _p],
     "xr_attn_extra_partial": [_p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p, _p, _f, _i, _p],
     "xr_softcap": [_p, _i, _i, _i, _f, _p],
     "xr_decay_prepare": [_p, _i, _i, _i, _i, _i, _f, _p, _p, _p],
@@ -82,20 +84,20 @@ _PROTOS = {
     "xr_sample": [_p, _p, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p, _p, _i, _p, _i, _p, _p],
     "xr_layernorm": [_p, _p, _p, _p, _i, _i, _i, _f, _i, _p],
     "xr_layernorm_conv": [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _f, _i, _p],
-    "xr_causal_conv": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p],
+    "xr_causal_conv": [_p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p],
     "xr_polynorm": [_p, _p, _p, _i, _i, _i, _f, _i, _i, _p],
     "xr_rotate_rows": [_p, _p, _p, _i, _i, _i, _i, _i, _f, _p],
-    "xr_gated_rmsnorm": [_p, _p, _p, _p, _i, _i, _i, _i, _f, _i, _i, _i, _p],
+    "xr_gated_rmsnorm": [_p, _p, _p, _p, _i, _i, _i, _i, _f, _i, _i, _i, _i, _f, _i, _p],
     "xr_act_rows": [_p, _i, _i, _i, _i, _p, _i, _p],
     "xr_embedding_pairs": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _p],
     "xr_streams_expand": [_p, _p, _i, _i, _i, _p],
     "xr_streams_sum": [_p, _p, _i, _i, _i, _p],
     "xr_streams_step": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _f, _i, _p],
-    "xr_latent_prepare": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p],
-    "xr_moe_route": [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _p],
-    "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p, _p],
+    "xr_latent_prepare": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p],
+    "xr_moe_route": [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p],
+    "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p, _i, _p],
     "xr_heads_gemm_bf16": [_p, _p, _p, _i, _i, _i, _i, _i, C.c_longlong, _i, C.c_longlong, _i, _p],
-    "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p],
+    "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _i, _p],
     "xr_delta_prepare": [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _p],
     "xr_linear_recurrence": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p, _p, _i, _f, _f, _p],
     "xr_qkv_store": [_p, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p],
@@ -105,8 +107,11 @@ _PROTOS = {
 }
 
 CONV_ACTIVATIONS = {None: 0, "none": 0, "silu": 1}      # XR_CONV_* of sequence_kernels.hip
-RECURRENCES = {"retention": 0, "delta": 1, "wkv": 2, "gla": 3, "delta_channel": 4}    # XR_REC_* of recurrent_kernels.hip
-ROW_ACTIVATIONS = {"silu": 1, "tanh": 2}                # what act_rows_ applies in place
+RECURRENCES = {"retention": 0, "delta": 1, "wkv": 2, "gla": 3, "delta_channel": 4, "ssd": 5}    # XR_REC_* of recurrent_kernels.hip
+ROW_ACTIVATIONS = {"silu": 1, "tanh": 2, "relu2": 3}    # what act_rows_ applies in place
+PRODUCT_ACTIVATIONS = {None: 0, "relu2": 1}             # what a plain product's results pass (XR_POST_* of gemm_mfma.hip)
+HEAD_NORMS = {None: 0, "before": 1, "after": 2}         # HEAD_NORM_* of basic_kernels.hip: before the rotation, behind it
+GROUP_SCORES = {"top2": 0, "max": 1}                    # what a group of experts scores
 ROUTE_SCORES = {"softmax": 0, "sigmoid": 1, "logits": 2}    # MOE_SCORES_* of moe_kernels.hip
 # what an expert applies between its products: (MOE_ACT_* of moe_kernels.hip, the gate's code)
 EXPERT_ACTIVATIONS = {"relu2": (0, 0), "swiglu": (1, GATE_ACTIVATIONS["silu"]),
@@ -172,12 +177,13 @@ class UnscaledRows:
 class _GemmNorm(C.Structure):
     """XrGemmNorm of the library."""
     _fields_ = [("ss_in", _p), ("n_ss", _i), ("ss_inv_width", _f), ("ss_eps", _f), ("norm_w", _p),
-                ("norm_w_bf16", _i), ("xg", _p), ("ss_out", _p), ("ss_out_rows", _i), ("centred", _i)]
+                ("norm_w_bf16", _i), ("xg", _p), ("ss_out", _p), ("ss_out_rows", _i), ("centred", _i),
+                ("post_x", _p), ("post_ld", _i), ("post_alpha", _f)]
 
 
 class _RowNorm(C.Structure):
     """XrRowNorm of the library."""
-    _fields_ = [("w", _p), ("w_bf16", _i), ("centred", _i), ("eps", _f), ("h", _p)]
+    _fields_ = [("w", _p), ("w_bf16", _i), ("centred", _i), ("eps", _f), ("h", _p), ("replace", _i), ("alpha", _f)]
 
 
 class _GemmRope(C.Structure):
@@ -223,7 +229,7 @@ class Ops:
 
     def __init__(self, lib: _Lib):
         self.lib = lib
-        self._attn_libs: Dict[int, object] = {}
+        self._attn_libs: Dict[tuple, object] = {}
         self.use_mfma = True
         self.fold_norms = True      # False: linear_add_rmsnorm always runs the norm's own kernel
         self.fuse_rope = True       # False: project_rope_kv_write always runs two kernels
@@ -388,8 +394,10 @@ class Ops:
 
     def linear(self, a: torch.Tensor, w, bias: Optional[torch.Tensor] = None,
                out_dtype: Optional[torch.dtype] = None, out: Optional[torch.Tensor] = None,
-               accumulate: bool = False, variant: int = 0, _then: Optional[_GemmNorm] = None) -> torch.Tensor:
-        """``a [M, K] @ w [N, K]^T (+ bias)``; with ``accumulate`` added into 32-bit ``out``.
+               accumulate: bool = False, variant: int = 0, _then: Optional[_GemmNorm] = None,
+               activation: Optional[str] = None) -> torch.Tensor:
+        """``a [M, K] @ w [N, K]^T (+ bias)``; with ``accumulate`` added into 32-bit ``out``; ``activation`` "relu2": the
+        square of what is positive of it (in the kernels' epilogues).
 
         bfloat16 operands run on the matrix cores (32-bit accumulation); float32 operands, and
         shapes the MFMA kernels do not take, run the plain 32-bit FMA kernel.  ``w`` is a matrix
@@ -416,10 +424,12 @@ class Ops:
             raise KernelError(f"linear: output is {tuple(out.shape)}, product is {(M, N)}")
         if bias is not None and (bias.dtype != torch.float32 or bias.numel() != N):
             raise KernelError("linear: bias must be float32 [N]")
+        if activation not in PRODUCT_ACTIVATIONS or (activation is not None and (accumulate or norm is not None)):
+            raise KernelError(f"linear: activation {activation!r} (known: {list(PRODUCT_ACTIVATIONS)}; on a product of its own only)")
         if self._mfma_ok(a, wt):
             self.lib.check(self.lib.xr_gemm_bf16(out.data_ptr(), a.data_ptr(), wt.data_ptr(), _ptr(bias), M, N, K,
                                                  a.stride(0), out.stride(0), dtype_code(out.dtype),
-                                                 1 if accumulate else 0, 0, 0.0, variant, 1 if packed else 0,
+                                                 1 if accumulate else 0, PRODUCT_ACTIVATIONS[activation], 0.0, variant, 1 if packed else 0,
                                                  *self._gemm_workspace(a.device),
                                                  C.addressof(norm) if norm is not None else None, None, _stream()))
             return out
@@ -427,9 +437,13 @@ class Ops:
             raise KernelError("linear: rows that still lack their norm's scale need the MFMA kernels")
         if packed:
             raise KernelError("linear: a packed weight needs bfloat16 rows that are 16-byte aligned")
+        if activation is not None and out.dtype != torch.float32:
+            return out.copy_(self.act_rows(self.linear(a, w, bias=bias, out_dtype=torch.float32), activation, out.dtype))
         self.lib.check(self.lib.xr_gemm_ref(out.data_ptr(), a.data_ptr(), w.data_ptr(), _ptr(bias), M, N, K,
                                             a.stride(0), out.stride(0), dtype_code(a.dtype),
                                             dtype_code(out.dtype), 1 if accumulate else 0, _stream()))
+        if activation is not None:
+            self.act_rows_(out, activation)
         return out
 
     @staticmethod
@@ -486,6 +500,44 @@ class Ops:
             return normed(residual, norm_weight, eps, out_dtype)            # the library declined
         self.linear(a, w, bias=bias, out=residual, accumulate=True)
         return normed(residual, norm_weight, eps, out_dtype)
+
+    def post_norm(self, x: torch.Tensor, y: torch.Tensor, alpha: float, norm_weight: torch.Tensor, eps: float,
+                  out_dtype: torch.dtype) -> torch.Tensor:
+        """``x <- norm(alpha x + y)`` in place on 32-bit rows ``x [T, E]``, the RMS norm (eps inside the root) with the
+        32-bit weight ``norm_weight [E]``; the new rows come back in ``out_dtype`` as well."""
+        self._dev(x, y, norm_weight)
+        T, E = y.shape
+        if x.dtype != torch.float32 or y.dtype != torch.float32 or tuple(x.shape) != (T, E) or x.stride(1) != 1 or not y.is_contiguous():
+            raise KernelError(f"post_norm: x and y must be float32 [{T}, {E}]")
+        if norm_weight.dtype != torch.float32 or norm_weight.numel() != E or not norm_weight.is_contiguous():
+            raise KernelError(f"post_norm: the norm's weight must be float32 [{E}]")
+        h = torch.empty((T, E), dtype=out_dtype, device=x.device)
+        self.lib.check(self.lib.xr_post_norm(x.data_ptr(), y.data_ptr(), norm_weight.data_ptr(), h.data_ptr(), T, E, x.stride(0),
+                                             float(alpha), float(eps), dtype_code(out_dtype), _stream()))
+        return h
+
+    def linear_post_norm(self, a: torch.Tensor, w, x: torch.Tensor, alpha: float, norm_weight: torch.Tensor, eps: float,
+                         out_dtype: torch.dtype, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """``x <- norm(alpha x + a @ w^T (+ bias))``, as ``post_norm``.  Where the product is split over K and has more than
+        16 rows, the kernel that adds the K ranges up takes whole rows and writes both the rows and their copy."""
+        wt = w.data if isinstance(w, PackedWeight) else w
+        M, N = a.shape[0], w.shape[0]
+        y = torch.empty((M, N), dtype=torch.float32, device=a.device)
+        if (self.fold_norms and M > UnscaledRows.MAX_ROWS and out_dtype == torch.bfloat16 and N % 4 == 0 and x.stride(0) % 4 == 0
+                and x.dtype == torch.float32 and tuple(x.shape) == (M, N) and x.data_ptr() % 16 == 0 and norm_weight.numel() == N
+                and norm_weight.is_contiguous() and self._mfma_ok(a, wt)):
+            self._dev(x, norm_weight)
+            then = _GemmNorm()
+            h = torch.empty((M, N), dtype=torch.bfloat16, device=a.device)
+            then.norm_w, then.norm_w_bf16, then.xg = norm_weight.data_ptr(), dtype_code(norm_weight.dtype), h.data_ptr()
+            then.ss_inv_width, then.ss_eps = 1.0 / N, float(eps)
+            then.post_x, then.post_ld, then.post_alpha = x.data_ptr(), x.stride(0), float(alpha)
+            self.linear(a, w, bias=bias, out=y, _then=then)
+            if then.ss_out_rows < 0:
+                return h
+        else:
+            self.linear(a, w, bias=bias, out=y)
+        return self.post_norm(x, y, alpha, norm_weight, eps, out_dtype)
 
     def linear_gated(self, a: torch.Tensor, w, bias: Optional[torch.Tensor] = None, activation: str = "silu",
                      variant: int = 0, param: float = 0.0) -> torch.Tensor:
@@ -584,6 +636,41 @@ class Ops:
             page_size, dtype_code(out_dtype), _stream()))
         return q
 
+    def head_norm_rope_write(self, q_in, k_in, v_in, w_q, w_k, eps: float, norm: Optional[str], k_cache, v_cache, ctx, group: int,
+                             inv_freq, H: int, Hk: int, D: int, Dv: int, rot: int, interleaved: bool, mscale: float,
+                             page_size: int, out_dtype) -> torch.Tensor:
+        """Queries and keys rotated, every head over its root mean square (eps inside the root) times the weights ``w_q``,
+        ``w_k [D]`` (or None) ``norm`` "before" or "after" the rotation (None: no norm); queries come back ``[T, H * D]`` in
+        ``out_dtype``, keys and the values ``v_in`` (``Dv`` channels a head) go to their pages.  Inputs are 32-bit views with
+        one row stride; ``k_in`` None: queries alone."""
+        self._dev(q_in, k_in, v_in, w_q, w_k, k_cache, v_cache, inv_freq)
+        views = [t for t in (q_in, k_in, v_in) if t is not None]
+        T = q_in.shape[0]
+        if any(t.dtype != torch.float32 or t.stride(1) != 1 for t in views) or (T > 1 and len({t.stride(0) for t in views}) != 1):
+            raise KernelError("head_norm_rope_write: q, k and v must be float32 views with one row stride")
+        Hk = Hk if k_in is not None else 0
+        if (tuple(q_in.shape) != (T, H * D) or (k_in is None) != (v_in is None)
+                or (Hk and (tuple(k_in.shape) != (T, Hk * D) or tuple(v_in.shape) != (T, Hk * Dv)))):
+            raise KernelError("head_norm_rope_write: view widths do not fit the heads")
+        if norm not in HEAD_NORMS:
+            raise KernelError(f"head_norm_rope_write: norm {norm!r} (known: {list(HEAD_NORMS)})")
+        for w in (w_q, w_k):
+            if w is not None and (w.dtype != torch.float32 or w.numel() != D or not w.is_contiguous()):
+                raise KernelError(f"head_norm_rope_write: a weight must be float32 [{D}]")
+        if Hk and (k_cache.dtype != out_dtype or v_cache.dtype != out_dtype or tuple(k_cache.shape[1:]) != (Hk, page_size, D)
+                   or tuple(v_cache.shape[1:]) != (Hk, Dv, page_size)):
+            raise KernelError("head_norm_rope_write: the cache does not fit the heads")
+        if rot and (inv_freq is None or inv_freq.dtype != torch.float32 or inv_freq.numel() != rot // 2):
+            raise KernelError(f"head_norm_rope_write: {rot // 2} 32-bit frequencies are needed")
+        table = ctx.block_table(group)
+        q = torch.empty((T, H * D), dtype=out_dtype, device=q_in.device)
+        self.lib.check(self.lib.xr_head_norm_rope_write(
+            q_in.data_ptr(), _ptr(k_in), _ptr(v_in), q_in.stride(0), _ptr(w_q), _ptr(w_k), float(eps), HEAD_NORMS[norm], q.data_ptr(),
+            _ptr(k_cache) if Hk else None, _ptr(v_cache) if Hk else None, ctx.positions.data_ptr(), ctx.req_of_token.data_ptr(),
+            table.data_ptr(), table.stride(0), _ptr(inv_freq), T, H, Hk, D, Dv, int(rot), 1 if interleaved else 0, float(mscale),
+            page_size, dtype_code(out_dtype), _stream()))
+        return q
+
     def rope_table(self, positions: torch.Tensor, inv_freq: torch.Tensor, mscale: float = 1.0) -> torch.Tensor:
         """``[T, rot/2, 2]`` float32: cosine and sine (times ``mscale``) of every row's angles, as
         ``project_rope_kv_write`` takes them for a product of many rows (``cs_table``); the same for
@@ -653,7 +740,8 @@ class Ops:
     def attention(self, q, k_cache, v_cache, ctx, group: int, H: int, Hk: int, D: int, page_size: int,
                   scale: float, window: Optional[int] = None, slopes: Optional[torch.Tensor] = None,
                   chunk: Optional[int] = None, keep_first: int = 0, sinks: Optional[torch.Tensor] = None,
-                  v_head_dim: Optional[int] = None, softcap: float = 0.0) -> torch.Tensor:
+                  v_head_dim: Optional[int] = None, softcap: float = 0.0, gate: Optional[torch.Tensor] = None,
+                  out_scale: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Causal attention of every token of the step over its request's cached keys and values.
         ``slopes`` (32-bit ``[H]``): ``slopes[h] * (i - j)`` is taken off the score of query i and key j.
         ``window``: a position reads the last ``window`` keys; ``chunk``: it reads the keys of its own chunk of
@@ -661,9 +749,11 @@ class Ops:
         ``sinks`` (32-bit ``[H]``): the softmax's denominator also holds ``exp(sinks[h])``, an entry without key
         or value.  ``v_head_dim``: the size of a value where it is not the keys' (``[T, H * v_head_dim]`` comes back).
         ``softcap`` c > 0: a scaled score s counts as ``c tanh(s / c)`` (a slope's bias is taken off that; the sink is not capped).
+        ``gate`` (a 32-bit view ``[T, H]``): a head's output times ``sigmoid(gate[t, h])``; ``out_scale``: every output times a
+        number, both before the one rounding.  ``out``: a view ``[T, H * Dv]`` of wider rows that takes the result.
 
-        bfloat16 runs on the matrix cores (head sizes in steps of 16 up to 256, pages of at least
-        16 positions, a cap or slopes); float32, and what the MFMA kernel does not take, runs the 32-bit kernel.
+        bfloat16 runs on the matrix cores (head and value sizes in steps of 16 up to 256, pages of at least
+        16 positions, a cap or slopes; kept first keys only where values have the keys' size); float32, and what the MFMA kernel does not take, runs the 32-bit kernel.
         """
         positions, req_of_token, block_table = ctx.positions, ctx.req_of_token, ctx.block_table(group)
         self._dev(q, k_cache, v_cache, positions, req_of_token, block_table)
@@ -674,7 +764,14 @@ class Ops:
         if H % Hk:
             raise KernelError(f"attention: {H} query heads are not a multiple of {Hk} key/value heads")
         Dv = int(v_head_dim) if v_head_dim is not None else D
-        out = torch.empty((T, H * Dv), dtype=q.dtype, device=q.device)
+        if out is None:
+            out = torch.empty((T, H * Dv), dtype=q.dtype, device=q.device)
+        elif out.dtype != q.dtype or tuple(out.shape) != (T, H * Dv) or out.stride(1) != 1:
+            raise KernelError(f"attention: the output must be a {q.dtype} view [{T}, {H * Dv}] with unit column stride")
+        self._dev(gate, out)
+        if gate is not None and (gate.dtype != torch.float32 or tuple(gate.shape) != (T, H) or gate.stride(1) != 1):
+            raise KernelError(f"attention: the gate must be a float32 view [{T}, {H}]")
+        gating = (_ptr(gate), gate.stride(0) if gate is not None else 0, float(out_scale), out.stride(0))
         for name, t in (("slopes", slopes), ("sinks", sinks)):
             if t is not None:
                 self._dev(t)
@@ -682,19 +779,19 @@ class Ops:
                     raise KernelError(f"attention: the {name} must be float32 [{H}]")
         if chunk and window:
             raise KernelError("attention: a layer reads a window or its chunk, not both")
-        if (self.use_mfma and q.dtype == torch.bfloat16 and D == Dv and D % 16 == 0 and 16 <= D <= 256 and page_size >= 16
-                and not (softcap and slopes is not None)):
+        if (self.attention_on_matrix_cores(q.dtype, D, Dv, page_size) and not (softcap and slopes is not None)
+                and (D == Dv or not keep_first) and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0):
             # The first keys that a window has passed enter the same softmax as a partial result of its own, which
             # the kernels' merge adds to the key ranges' (with the sink, if there is one); a sink alone is added by
             # the kernels themselves where they finish a row.
             extra = keep_first > 0
-            lib = self.attention_lib(D)
+            lib = self.attention_lib(D, Dv)
             mask = Chunked(int(chunk)) if chunk else window
             plan = (ctx.attention_plan(group, H // Hk, mask, Hk, page_size, extra_slot=True) if extra
                     else ctx.attention_plan(group, H // Hk, mask, Hk, page_size))
             part_o = part_ml = None
             if plan.n_slots:
-                part_o = torch.empty((plan.n_slots, Hk, 32, D), dtype=torch.float32, device=q.device)
+                part_o = torch.empty((plan.n_slots, Hk, 32, Dv), dtype=torch.float32, device=q.device)
                 part_ml = torch.empty((plan.n_slots, Hk, 32, 2), dtype=torch.float32, device=q.device)
             if extra:
                 self.lib.check(self.lib.xr_attn_extra_partial(
@@ -705,16 +802,21 @@ class Ops:
             lib.check(lib.xr_attention_mfma(
                 out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), plan.items.data_ptr(),
                 plan.n_items, plan.n_cta_items, _ptr(plan.jobs), plan.n_jobs, ctx.cu_q.data_ptr(),
-                ctx.starts_dev.data_ptr(), block_table.data_ptr(), block_table.stride(0), _ptr(part_o), _ptr(part_ml), H, Hk, D, page_size,
+                ctx.starts_dev.data_ptr(), block_table.data_ptr(), block_table.stride(0), _ptr(part_o), _ptr(part_ml), H, Hk, D, Dv, page_size,
                 float(scale), int(window or 0), int(chunk or 0), _ptr(slopes), None if extra else _ptr(sinks),
-                float(softcap), _stream()))
+                float(softcap), *gating, _stream()))
             return out
         self.lib.check(self.lib.xr_attention_ref(
             out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), positions.data_ptr(),
             req_of_token.data_ptr(), block_table.data_ptr(), block_table.stride(0), T, H, Hk, D, Dv, page_size,
             float(scale), int(window or 0), int(chunk or 0), int(keep_first), dtype_code(q.dtype), _ptr(slopes),
-            _ptr(sinks), float(softcap), _stream()))
+            _ptr(sinks), float(softcap), *gating, _stream()))
         return out
+
+    def attention_on_matrix_cores(self, dtype: torch.dtype, D: int, Dv: int, page_size: int = 64) -> bool:
+        """Whether keys of ``D`` and values of ``Dv`` channels have matrix-core attention kernels."""
+        return (self.use_mfma and dtype == torch.bfloat16 and D % 16 == 0 and 16 <= D <= 256 and Dv % 16 == 0 and 16 <= Dv <= 256
+                and page_size >= 16)
 
     def softcap_(self, x: torch.Tensor, cap: float) -> None:
         """``x <- cap tanh(x / cap)`` in place on a 32-bit view ``[rows, width]`` with unit column stride."""
@@ -788,15 +890,16 @@ class Ops:
             raise KernelError(f"add_rows_: y must be contiguous float32 [{T}, {E}]")
         self.lib.check(self.lib.xr_add_rows(x.data_ptr(), _ptr(y), v.data_ptr(), float(scale), T, E, _stream()))
 
-    def attention_lib(self, D: int) -> "_Lib":
-        """The MFMA attention library for head size ``D`` (compiled at first use)."""
-        lib = self._attn_libs.get(D)
+    def attention_lib(self, D: int, Dv: Optional[int] = None) -> "_Lib":
+        """The MFMA attention library for head size ``D`` and values of ``Dv`` channels (compiled at first use)."""
+        Dv = D if Dv is None else Dv
+        lib = self._attn_libs.get((D, Dv))
         if lib is None:
-            unit = f"attn_d{D}"
+            unit = f"attn_d{D}" if D == Dv else f"attn_d{D}v{Dv}"
             path = _build.find_built(unit) or _build.build_unit(unit)
             lib = _Lib(path, {"xr_attention_mfma": [_p, _p, _p, _p, _p, _i, _i, _p, _i, _p, _p, _p, _i, _p, _p,
-                                                    _i, _i, _i, _i, _f, _i, _i, _p, _p, _f, _p]})
-            self._attn_libs[D] = lib
+                                                    _i, _i, _i, _i, _i, _f, _i, _i, _p, _p, _f, _p, _i, _f, _i, _p]})
+            self._attn_libs[(D, Dv)] = lib
         return lib
 
     # -- row-wise and time-wise operations around the sequence mixers ----------
@@ -895,12 +998,14 @@ class Ops:
                                                 int(temp_every), _stream()))
 
     def causal_conv(self, u: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], ctx, out_dtype: torch.dtype,
-                    residual: bool = False, activation: Optional[str] = None) -> torch.Tensor:
+                    residual: bool = False, activation: Optional[str] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
         """A convolution over time on every channel of ``u [T, C]``: ``y_t = sum_j w[:, j] u_(t-taps+1+j)``
-        (plus ``u_t`` with ``residual``), then the activation.  ``state [slots + 1, taps - 1, C]`` (the
+        (plus a 32-bit ``bias [C]``, plus ``u_t`` with ``residual``), then the activation.  ``state [slots + 1, taps - 1, C]`` (the
         dtype of ``u``) holds every request's last ``taps - 1`` inputs and is brought up to date;
         ``ctx`` gives the step's rows (``cu_q``, ``slots``, ``req_of_token``)."""
-        self._dev(u, w, state)
+        self._dev(u, w, state, bias)
+        if bias is not None and (bias.dtype != torch.float32 or bias.numel() != w.shape[0] or not bias.is_contiguous()):
+            raise KernelError(f"causal_conv: the bias must be float32 [{w.shape[0]}]")
         if u.dim() != 2 or u.stride(1) != 1:
             raise KernelError("causal_conv input must be [rows, channels] with unit column stride")
         T, Cn = u.shape
@@ -913,7 +1018,7 @@ class Ops:
         if activation not in CONV_ACTIVATIONS:
             raise KernelError(f"causal_conv: activation {activation!r} is not built (known: none, silu)")
         out = torch.empty((T, Cn), dtype=out_dtype, device=u.device)
-        self.lib.check(self.lib.xr_causal_conv(out.data_ptr(), u.data_ptr(), w.data_ptr(), _ptr(state), ctx.cu_q.data_ptr(),
+        self.lib.check(self.lib.xr_causal_conv(out.data_ptr(), u.data_ptr(), w.data_ptr(), _ptr(bias), _ptr(state), ctx.cu_q.data_ptr(),
                                                ctx.slots.data_ptr(), ctx.req_of_token.data_ptr(), T, ctx.B, Cn, taps,
                                                u.stride(0), Cn, dtype_code(u.dtype), dtype_code(out_dtype),
                                                1 if residual else 0, CONV_ACTIVATIONS[activation],
@@ -972,11 +1077,14 @@ class Ops:
                                                rot, x.stride(0), float(scale), _stream()))
 
     def gated_rmsnorm(self, o: torch.Tensor, gate: torch.Tensor, w: Optional[torch.Tensor], H: int, Dv: int, eps: float,
-                      out_dtype: torch.dtype, gate_activation: str = "silu") -> torch.Tensor:
+                      out_dtype: torch.dtype, gate_activation: str = "silu", gate_first: bool = False, out_scale: float = 1.0,
+                      out: Optional[torch.Tensor] = None) -> torch.Tensor:
         """``o / rms(o) * w * act(gate)`` per head: ``o [T, H * Dv]`` 32-bit and contiguous, ``gate`` a
         32-bit view of the same shape; ``w`` 32-bit: ``[Dv]`` (the heads share it), ``[H * Dv]`` (one a
         channel of the row) or absent; ``act`` "silu" or "sigmoid".  A norm over all heads together is
-        ``H = 1`` with ``Dv`` the whole row."""
+        ``H = 1`` with ``Dv`` the whole row.  ``gate_first``: the gate comes before the norm, ``u / rms(u) * w`` with
+        ``u = o * act(gate)``.  ``out_scale``: the result times a number; ``out``: a view ``[T, H * Dv]`` of wider rows that
+        takes it."""
         self._dev(o, gate, w)
         T = o.shape[0]
         if o.dtype != torch.float32 or not o.is_contiguous() or o.shape[1] != H * Dv:
@@ -987,11 +1095,15 @@ class Ops:
             raise KernelError(f"gated_rmsnorm: the weight must be float32 [{Dv}] or [{H * Dv}]")
         if gate_activation not in NORM_GATES:
             raise KernelError(f"gated_rmsnorm: gate activation {gate_activation!r} (known: {sorted(NORM_GATES)})")
-        out = torch.empty((T, H * Dv), dtype=out_dtype, device=o.device)
+        if out is None:
+            out = torch.empty((T, H * Dv), dtype=out_dtype, device=o.device)
+        elif out.dtype != out_dtype or tuple(out.shape) != (T, H * Dv) or out.stride(1) != 1:
+            raise KernelError(f"gated_rmsnorm: the output must be a {out_dtype} view [{T}, {H * Dv}] with unit column stride")
         self.lib.check(self.lib.xr_gated_rmsnorm(out.data_ptr(), o.data_ptr(), gate.data_ptr(), _ptr(w), T, H, Dv,
                                                  gate.stride(0), float(eps), dtype_code(out_dtype),
                                                  1 if (w is not None and H > 1 and w.numel() == H * Dv) else 0,
-                                                 NORM_GATES[gate_activation], _stream()))
+                                                 NORM_GATES[gate_activation], 1 if gate_first else 0, float(out_scale), out.stride(0),
+                                                 _stream()))
         return out
 
     def act_rows_(self, x: torch.Tensor, activation: str = "silu") -> None:
@@ -1096,7 +1208,7 @@ class Ops:
     # -- latent attention ------------------------------------------------------------
     def latent_prepare(self, q_in: torch.Tensor, kv_in: torch.Tensor, c_w: torch.Tensor, eps: float, q_out: torch.Tensor,
                        k_cache: torch.Tensor, v_cache: torch.Tensor, ctx, group: int, inv_freq: Optional[torch.Tensor],
-                       H: int, D: int, R: int, C: int, dims: int, page_size: int) -> torch.Tensor:
+                       H: int, D: int, R: int, C: int, dims: int, page_size: int, halves: bool = False) -> torch.Tensor:
         """Between a latent attention's down projections and its attention.  ``q_in [T, H * (D + R)]`` and
         ``kv_in [T, C + R]`` are 32-bit views.  The first ``C`` channels of ``kv_in`` are normed (RMS, weight
         ``c_w``) into the latent; the last ``R`` are the shared key part, whose first ``dims`` channels are
@@ -1104,14 +1216,15 @@ class Ops:
         query head.  The row ``[latent | key part]`` goes to the key pages ``[pages, 1, page, C + R]`` and,
         transposed, to the value pages ``[pages, 1, C or C + R, page]``; the rotated query channels go to
         ``q_out[:, h, C:]`` (``q_out [T, H * (C + R)]``); the unrotated ones come back ``[T, H * D]`` in
-        ``q_out``'s dtype."""
+        ``q_out``'s dtype.  ``halves``: the rotation's pairs are ``(i, i + dims / 2)``.  ``kv_in`` None: a layer that stores
+        nothing (it reads another layer's rows); its queries alone."""
         self._dev(q_in, kv_in, c_w, q_out, k_cache, v_cache, inv_freq)
         T = q_in.shape[0]
-        if any(t.dtype != torch.float32 or t.stride(1) != 1 for t in (q_in, kv_in)):
+        if any(t is not None and (t.dtype != torch.float32 or t.stride(1) != 1) for t in (q_in, kv_in)):
             raise KernelError("latent_prepare: q and kv inputs must be float32 views with unit column stride")
-        if tuple(q_in.shape) != (T, H * (D + R)) or tuple(kv_in.shape) != (T, C + R):
+        if tuple(q_in.shape) != (T, H * (D + R)) or (kv_in is not None and tuple(kv_in.shape) != (T, C + R)):
             raise KernelError("latent_prepare: input widths do not fit the heads")
-        if c_w.dtype != torch.float32 or c_w.numel() != C or not c_w.is_contiguous():
+        if kv_in is not None and (c_w.dtype != torch.float32 or c_w.numel() != C or not c_w.is_contiguous()):
             raise KernelError(f"latent_prepare: the latent norm's weight must be float32 [{C}]")
         dt = q_out.dtype
         if tuple(q_out.shape) != (T, H * (C + R)) or not q_out.is_contiguous():
@@ -1125,9 +1238,10 @@ class Ops:
         table = ctx.block_table(group)
         qn = torch.empty((T, H * D), dtype=dt, device=q_in.device)
         self.lib.check(self.lib.xr_latent_prepare(qn.data_ptr(), q_out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
-                                                  q_in.data_ptr(), kv_in.data_ptr(), c_w.data_ptr(), ctx.positions.data_ptr(),
+                                                  q_in.data_ptr(), _ptr(kv_in), _ptr(c_w), ctx.positions.data_ptr(),
                                                   ctx.req_of_token.data_ptr(), table.data_ptr(), table.stride(0), _ptr(inv_freq),
-                                                  T, H, D, R, C, Dvc, int(dims), q_in.stride(0), kv_in.stride(0), page_size,
+                                                  T, H, D, R, C, Dvc, int(dims), 1 if halves else 0, q_in.stride(0),
+                                                  kv_in.stride(0) if kv_in is not None else 0, page_size,
                                                   float(eps), dtype_code(dt), _stream()))
         return qn
 
@@ -1162,10 +1276,12 @@ class Ops:
         return self.route_logits(logits, correction, top, **how)
 
     def route_logits(self, logits: torch.Tensor, correction: torch.Tensor, top: int, scores: str = "softmax",
-                     groups: int = 1, keep_groups: int = 1, weight_scale: Optional[float] = None, side_gate: bool = False):
+                     groups: int = 1, keep_groups: int = 1, weight_scale: Optional[float] = None, side_gate: bool = False,
+                     group_score: str = "top2"):
         """``moe_route`` from the 32-bit logits ``[T, n]``.  ``scores`` "sigmoid": every expert's score is the sigmoid
         of its logit.  ``groups`` > 1: the experts form that many equal groups of neighbours, a group scores the
-        sum of its two largest score + correction, and only the ``keep_groups`` best groups' experts can be chosen.
+        sum of its two largest score + correction (``group_score`` "max": the largest), and only the ``keep_groups`` best
+        groups' experts can be chosen.
         ``weight_scale``: the weights are the chosen scores times it instead of their shares of their sum.  ``scores``
         "logits": the choice is by logit + ``correction`` (the router's bias), the weights are the softmax of these over
         the chosen experts.  ``side_gate``: the logits have one column more, ``[T, n + 1]``, which is no expert's; its
@@ -1174,6 +1290,8 @@ class Ops:
             raise KernelError(f"route_logits: scores {scores!r} ({', '.join(ROUTE_SCORES)})")
         if scores == "logits" and (groups != 1 or weight_scale is not None):
             raise KernelError("route_logits: a choice by the logits has no groups and no weight scale")
+        if group_score not in GROUP_SCORES:
+            raise KernelError(f"route_logits: group score {group_score!r} ({', '.join(GROUP_SCORES)})")
         if weight_scale is not None and not weight_scale > 0:
             raise KernelError(f"route_logits: weight scale {weight_scale} must be positive")
         self._dev(logits, correction)
@@ -1188,7 +1306,7 @@ class Ops:
         side = torch.empty((T,), dtype=torch.float32, device=logits.device) if side_gate else None
         self.lib.check(self.lib.xr_moe_route(idx.data_ptr(), wts.data_ptr(), _ptr(side), logits.data_ptr(), correction.data_ptr(), T,
                                              logits.stride(0), n, int(top), ROUTE_SCORES[scores], int(groups),
-                                             int(keep_groups), float(weight_scale or 0.0), _stream()))
+                                             int(keep_groups), float(weight_scale or 0.0), GROUP_SCORES[group_score], _stream()))
         return (idx, wts, side) if side_gate else (idx, wts)
 
     def table_route(self, table: torch.Tensor, ids: torch.Tensor, n_experts: int):
@@ -1209,14 +1327,16 @@ class Ops:
 
     def moe_experts(self, h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor,
                     out: Optional[torch.Tensor] = None, accumulate: bool = False, activation: str = "relu2", param: float = 0.0,
-                    beside=None, norm=None):
+                    beside=None, norm=None, identity: int = 0, post_alpha: Optional[float] = None):
         """``out[t] (+)= sum_j wts[t, j] * w_down[e] @ relu(w_up[e] @ h[t])^2`` with ``e = idx[t, j]``, as 32-bit
         rows; ``w_up [n, F, E]`` and ``w_down [n, E, F]`` in ``h``'s dtype.  ``activation`` "swiglu": gated experts,
         ``w_down[e] @ (silu(g) * u)`` with ``[g; u] = w_up[e] @ h[t]`` for ``w_up [n, 2F, E]`` (an expert's gate rows
         before its up rows); "clamped_swish" and "gelu_tanh" likewise with that gate (its number ``param``).  ``beside`` =
-        (32-bit rows ``[T, E]``, one weight a row ``[T]``): these rows enter the sum too.  ``norm`` = (weight, eps,
-        centred), the norm of the updated rows (an RMS norm, or with ``centred`` the layer norm with a 32-bit weight): its
-        result in ``h``'s dtype comes back instead of the rows.  A few choices stream the chosen
+        (32-bit rows ``[T, E]``, one weight a row ``[T]`` or None for the rows as they are): these rows enter the sum too.
+        ``norm`` = (weight, eps, centred), the norm of the updated rows (an RMS norm, or with ``centred`` the layer norm with a
+        32-bit weight): its result in ``h``'s dtype comes back instead of the rows.  With ``post_alpha`` the rows ``out``
+        become ``norm(post_alpha * out + the sum)`` themselves (an RMS norm with a 32-bit weight).  ``identity``: choices
+        ``n .. n + identity - 1`` stand for experts whose output is ``h[t]`` itself.  A few choices stream the chosen
         experts' weights, a wave an output column; from ``GROUPED_EXPERTS_FROM`` choices on (bfloat16, widths
         that are multiples of 8) the rows are sorted by expert on the device, both products run on the matrix
         cores and a last kernel adds a token's experts up in the order of its choice (and writes the norm)."""
@@ -1230,7 +1350,7 @@ class Ops:
         if beside is not None:
             self._dev(y_beside, g_beside)
             if (y_beside.dtype != torch.float32 or tuple(y_beside.shape) != tuple(h.shape) or not y_beside.is_contiguous()
-                    or g_beside.dtype != torch.float32 or g_beside.numel() != h.shape[0] or not g_beside.is_contiguous()):
+                    or (g_beside is not None and (g_beside.dtype != torch.float32 or g_beside.numel() != h.shape[0] or not g_beside.is_contiguous()))):
                 raise KernelError(f"moe_experts: the rows beside must be contiguous float32 {tuple(h.shape)} with a float32 weight a row")
         n, Fu, _ = w_up.shape
         F = Fu // 2 if gated else Fu
@@ -1247,6 +1367,9 @@ class Ops:
             out = torch.empty((T, E), dtype=torch.float32, device=h.device)
         elif out.dtype != torch.float32 or tuple(out.shape) != (T, E) or out.stride(1) != 1:
             raise KernelError(f"moe_experts: the output must be float32 [{T}, {E}]")
+        post = post_alpha is not None
+        if post and (norm is None or norm[2] or norm[0].dtype != torch.float32 or accumulate):
+            raise KernelError("moe_experts: rows that become a norm need an RMS norm with a 32-bit weight")
         z = torch.empty((T * top, F), dtype=h.dtype, device=h.device)
         if (self.use_mfma and h.dtype == torch.bfloat16 and T * top >= self.GROUPED_EXPERTS_FROM and E % 8 == 0 and F % 8 == 0
                 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0 and n <= 1024 and T * top <= (1 << 24)):
@@ -1258,17 +1381,25 @@ class Ops:
             if norm is not None and E % 4 == 0 and E <= 8192 and out.stride(0) % 4 == 0 and out.data_ptr() % 16 == 0:
                 self._dev(norm[0])
                 normed = torch.empty((T, E), dtype=h.dtype, device=h.device)
-                rn = _RowNorm(norm[0].data_ptr(), dtype_code(norm[0].dtype), 1 if norm[2] else 0, float(norm[1]), normed.data_ptr())
-            self.lib.check(self.lib.xr_moe_experts_grouped(out.data_ptr(), z.data_ptr(), yz.data_ptr(), scratch.data_ptr(),
+                rn = _RowNorm(norm[0].data_ptr(), dtype_code(norm[0].dtype), 1 if norm[2] else 0, float(norm[1]), normed.data_ptr(),
+                              1 if post else 0, float(post_alpha) if post else 1.0)
+            target = out if not post or rn is not None else torch.empty((T, E), dtype=torch.float32, device=h.device)
+            self.lib.check(self.lib.xr_moe_experts_grouped(target.data_ptr(), z.data_ptr(), yz.data_ptr(), scratch.data_ptr(),
                                                            h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(), idx.data_ptr(),
-                                                           wts.data_ptr(), T, E, F, h.stride(0), out.stride(0), n, top,
+                                                           wts.data_ptr(), T, E, F, h.stride(0), target.stride(0), n, top,
                                                            1 if accumulate else 0, form, gate, float(param), _ptr(y_beside),
-                                                           _ptr(g_beside), C.addressof(rn) if rn is not None else None, _stream()))
-            return normed if normed is not None else self._then_norm(out, norm, h.dtype)
-        self.lib.check(self.lib.xr_moe_experts(out.data_ptr(), z.data_ptr(), h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(),
-                                               idx.data_ptr(), wts.data_ptr(), T, E, F, h.stride(0), out.stride(0), n, top,
+                                                           _ptr(g_beside), C.addressof(rn) if rn is not None else None,
+                                                           int(identity), _stream()))
+            if normed is not None:
+                return normed
+            return self.post_norm(out, target, post_alpha, norm[0], norm[1], h.dtype) if post else self._then_norm(out, norm, h.dtype)
+        target = torch.empty((T, E), dtype=torch.float32, device=h.device) if post else out
+        self.lib.check(self.lib.xr_moe_experts(target.data_ptr(), z.data_ptr(), h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(),
+                                               idx.data_ptr(), wts.data_ptr(), T, E, F, h.stride(0), target.stride(0), n, top,
                                                1 if accumulate else 0, dtype_code(h.dtype), form, gate, float(param),
-                                               _ptr(y_beside), _ptr(g_beside), _stream()))
+                                               _ptr(y_beside), _ptr(g_beside), int(identity), _stream()))
+        if post:
+            return self.post_norm(out, target, post_alpha, norm[0], norm[1], h.dtype)
         return self._then_norm(out, norm, h.dtype)
 
     def _then_norm(self, rows: torch.Tensor, norm, dtype: torch.dtype):
@@ -1314,6 +1445,8 @@ class Ops:
         a token, head and key channel from ``gate`` = x ``[T, H * D]`` and the bonus ``decay`` = u ``[H, D]``.
         "gla": ``S <- diag(w) S + k v^T`` with the decays ``gate`` = w ``[T, H * D]`` as they are, read out after the
         update; "delta_channel": the delta rule with a decay a key channel, ``gate`` = w ``[T, H * D]``, ``beta [T, H]``.
+        "ssd": a state space: with the step size ``dt = softplus(z + bias)`` from ``gate`` = z ``[T, H]`` and ``decay`` =
+        (a, bias, D) as 32-bit ``[3, H]``: ``S <- exp(-a dt) S + dt k v^T``, ``o = S^T q + D v``.
         ``q, k [T, G * D]``, ``v [T, H * Dv]``: 32-bit views that share a row stride.  ``activation`` "silu":
         q, k and v pass SiLU on their way into the kernel (the views themselves stay as they are).  ``q_scale`` / ``k_scale``:
         factors on the queries and on the keys, applied on the way in as well (behind the activation)."""
@@ -1348,6 +1481,10 @@ class Ops:
             if (G != H or beta is not None or activation is not None or gate is None or tuple(gate.shape) != (T, H * D)
                     or decay is None or decay.dtype != torch.float32 or decay.numel() != H * D or not decay.is_contiguous()):
                 raise KernelError(f"linear_recurrence: wkv needs a key head a head, decays [T, {H * D}] and float32 bonus [{H}, {D}]")
+        elif kind == "ssd":
+            if (beta is not None or activation is not None or gate is None or tuple(gate.shape) != (T, H) or decay is None
+                    or decay.dtype != torch.float32 or tuple(decay.shape) != (3, H) or not decay.is_contiguous()):
+                raise KernelError(f"linear_recurrence: ssd needs step sizes [T, {H}] and float32 constants [3, {H}]")
         elif decay is None or decay.dtype != torch.float32 or decay.numel() != H:
             raise KernelError(f"linear_recurrence: retention needs float32 decay [{H}]")
         out = torch.empty((T, H * Dv), dtype=torch.float32, device=q.device)
@@ -1355,13 +1492,15 @@ class Ops:
         # chunk's last state through the chunk's decays alone: one number a head, or their product channel by
         # channel; a chunk's sum from zero and that add up); the delta rule's chain cannot be cut.
         chunk_len, n_chunks, scratch, prod = 0, 0, None, None
-        if kind in ("retention", "wkv", "gla") and ctx.max_q_len >= self.RETENTION_CHUNKED_FROM:
+        if kind in ("retention", "wkv", "gla", "ssd") and ctx.max_q_len >= self.RETENTION_CHUNKED_FROM:
             n = -(-ctx.max_q_len // self.RETENTION_CHUNK)
             if ctx.B * n <= 4096:
                 chunk_len, n_chunks = self.RETENTION_CHUNK, n
                 scratch = torch.empty((ctx.B * n,) + tuple(state.shape[1:]), dtype=torch.float32, device=q.device)
                 if kind in ("wkv", "gla"):
                     prod = torch.empty((ctx.B * n, H, rows.value * lanes.value), dtype=torch.float32, device=q.device)
+                elif kind == "ssd":
+                    prod = torch.empty((ctx.B * n, H), dtype=torch.float32, device=q.device)
         self.lib.check(self.lib.xr_linear_recurrence(out.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(), _ptr(beta),
                                                      _ptr(gate), _ptr(decay), state.data_ptr(), ctx.cu_q.data_ptr(),
                                                      ctx.slots.data_ptr(), ctx.B, H, G, D, Dv, q.stride(0),
@@ -1440,8 +1579,8 @@ class Ops:
             lib.check(lib.xr_attention_mfma(
                 out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), plan.items.data_ptr(),
                 plan.n_items, plan.n_cta_items, _ptr(plan.jobs), plan.n_jobs, ctx.cu_q.data_ptr(),
-                ctx.starts_dev.data_ptr(), table.data_ptr(), table.stride(0), _ptr(part_o), _ptr(part_ml), H, Hk, D, page_size,
-                float(scale), int(size), 0, None, None, 0.0, _stream()))
+                ctx.starts_dev.data_ptr(), table.data_ptr(), table.stride(0), _ptr(part_o), _ptr(part_ml), H, Hk, D, D, page_size,
+                float(scale), int(size), 0, None, None, 0.0, None, 0, 1.0, out.stride(0), _stream()))
             return out
         self.lib.check(self.lib.xr_attention_pooled(
             out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), _ptr(pk) if P else None,

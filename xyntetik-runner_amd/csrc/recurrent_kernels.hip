@@ -8,6 +8,8 @@
 //   gla:         S <- diag(w) S + k v^T;                            o = S^T q    (w a decay a token, head and key
 //                channel, given as it is: "gated linear attention")
 //   delta rule with a decay a key channel:  S <- diag(w) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//   ssd:         S <- exp(-a_h dt) S + dt k v^T;                    o = S^T q + D_h v    (a state space with one decay
+//                a token and head, made here from the step size dt = softplus(z + bias_h) as the rows are fetched)
 //
 // S is [D, Dv] and its columns never meet: column c only needs v[c].  A group of R adjacent lanes
 // owns one column (lane r the rows r, r+R, r+2R, ...), keeps it in registers over the whole
@@ -29,6 +31,7 @@
 #define XR_REC_WKV 2
 #define XR_REC_GLA 3
 #define XR_REC_DELTA_CH 4
+#define XR_REC_SSD 5
 
 static inline int rec_lanes(int D) { return D > 32 ? 16 : 4; }
 
@@ -39,8 +42,8 @@ struct RecArgs {
     const float* v;          // H heads of Dv
     const float* beta;       // [T, ld_g] at head 0 (delta rule)
     const float* gate;       // [T, ld_g] at head 0: the decay of every token and head (delta rule); wkv: x of the decay, H heads of D;
-                             // gla and the delta rule with channel decays: the decays themselves, H heads of D
-    const float* decay;      // [H] (retention); wkv: the bonus u [H, D]
+                             // gla and the delta rule with channel decays: the decays themselves, H heads of D; ssd: z of the step size
+    const float* decay;      // [H] (retention); wkv: the bonus u [H, D]; ssd: [3][H]: a, the step size's bias, D
     float* state;
     const int* cu_q;
     const int* slots;
@@ -61,7 +64,8 @@ struct RecArgs {
     // wkv in chunks: its decay is a number a token and key channel, so the state before a chunk enters the
     // chunk's last state through the product of the chunk's decays, channel by channel: pass 1 leaves that
     // product in prod [request x chunk][head][J][R] (row R j + r at j R + r) beside the chunk's last state;
-    // pass 2 runs with v = 0, so that the state only decays and the bonus term is nothing.
+    // pass 2 runs with v = 0, so that the state only decays and the bonus term is nothing.  (ssd: one product a
+    // request, chunk and head, prod [request x chunk][head].)
     float* prod;
     float q_scale, k_scale;  // factors on the queries and on the keys as they are fetched (behind the activation, if there is one)
 };
@@ -113,6 +117,9 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
 #pragma unroll
     for (int j = 0; j < DPER; ++j) S[j] = (live && j < J && from) ? from[((size_t)j * a.Dv + col) * R + r] : 0.f;
     const float dec = MODE == XR_REC_RETENTION ? a.decay[h] : 1.f;
+    constexpr bool SSD = MODE == XR_REC_SSD;
+    const float ssd_a = SSD ? a.decay[h] : 0.f, ssd_b = SSD ? a.decay[a.H + h] : 0.f, ssd_d = SSD ? a.decay[2 * a.H + h] : 0.f;
+    float gp = 1.f;                 // (ssd, pass 1) the product of the chunk's decays
     float* qf = reinterpret_cast<float*>(&qs[0][0]);
     float* kf = reinterpret_cast<float*>(&ks[0][0]);
     float* wf = reinterpret_cast<float*>(&ws[0][0]);
@@ -162,6 +169,11 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
             rb = a.beta[(size_t)(row0 + c0 + tid) * a.ld_b + h];
             if (MODE == XR_REC_DELTA) rg = a.gate[(size_t)(row0 + c0 + tid) * a.ld_g + h];
         }
+        if (SSD && tid < nt) {
+            const float z = a.gate[(size_t)(row0 + c0 + tid) * a.ld_g + h] + ssd_b;
+            rb = z > 20.0f ? z : log1pf(expf(z));       // the step size
+            rg = expf(-ssd_a * rb);                     // the decay
+        }
     };
     fetch(0);
     float4 qp[DPER / 4];            // (delta rule) the query of the token before, whose read-out is still owed
@@ -180,7 +192,7 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
 #pragma unroll
         for (int i = 0; i < NV; ++i)
             if (tid + i * 256 < REC_TOKENS * COLS) (&vs[0][0])[tid + i * 256] = rv[i];
-        if (CHAIN && tid < REC_TOKENS) { bs[tid] = rb; gs[tid] = rg; }
+        if ((CHAIN || SSD) && tid < REC_TOKENS) { bs[tid] = rb; gs[tid] = rg; }
         __syncthreads();
         if (c0 + REC_TOKENS < n) fetch(c0 + REC_TOKENS);
         if (MODE == XR_REC_DELTA_CH) {
@@ -292,7 +304,8 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
                 }
             }
         } else {
-            // Retention's chain is one multiply-add a token; four tokens' read-outs run side by side.
+            // Retention's chain (and ssd's, whose decay is the token's own) is one multiply-add a token; four tokens'
+            // read-outs run side by side.
             int tt = 0;
             for (; tt + 4 <= nt; tt += 4) {
                 float oo[4];
@@ -300,20 +313,24 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
                 for (int x = 0; x < 4; ++x) {
                     const float4* kq = &ks[tt + x][r * (DPER / 4)];
                     const float4* qq = &qs[tt + x][r * (DPER / 4)];
-                    const float vv = vs[tt + x][cl];
+                    const float g = SSD ? gs[tt + x] : dec, vv = SSD ? vs[tt + x][cl] * bs[tt + x] : vs[tt + x][cl];
                     float o0 = 0.f, o1 = 0.f;
+                    if (SSD) gp *= g;
 #pragma unroll
                     for (int j = 0; j < DPER; j += 4) {
                         const float4 kk = kq[j >> 2], q4 = qq[j >> 2];
-                        S[j] = fmaf(dec, S[j], kk.x * vv); S[j + 1] = fmaf(dec, S[j + 1], kk.y * vv);
-                        S[j + 2] = fmaf(dec, S[j + 2], kk.z * vv); S[j + 3] = fmaf(dec, S[j + 3], kk.w * vv);
+                        S[j] = fmaf(g, S[j], kk.x * vv); S[j + 1] = fmaf(g, S[j + 1], kk.y * vv);
+                        S[j + 2] = fmaf(g, S[j + 2], kk.z * vv); S[j + 3] = fmaf(g, S[j + 3], kk.w * vv);
                         o0 = fmaf(S[j], q4.x, o0); o1 = fmaf(S[j + 1], q4.y, o1);
                         o0 = fmaf(S[j + 2], q4.z, o0); o1 = fmaf(S[j + 3], q4.w, o1);
                     }
                     oo[x] = o0 + o1;
                 }
 #pragma unroll
-                for (int x = 0; x < 4; ++x) oo[x] = group_sum<R>(oo[x]);
+                for (int x = 0; x < 4; ++x) {
+                    oo[x] = group_sum<R>(oo[x]);
+                    if (SSD) oo[x] = fmaf(ssd_d, vs[tt + x][cl], oo[x]);       // (values are zeros in pass 2)
+                }
                 if (live && r == 0) {
 #pragma unroll
                     for (int x = 0; x < 4; ++x) {
@@ -325,17 +342,19 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
             for (; tt < nt; ++tt) {
                 const float4* kq = &ks[tt][r * (DPER / 4)];
                 const float4* qq = &qs[tt][r * (DPER / 4)];
-                const float vv = vs[tt][cl];
+                const float g = SSD ? gs[tt] : dec, vv = SSD ? vs[tt][cl] * bs[tt] : vs[tt][cl];
                 float o0 = 0.f, o1 = 0.f;
+                if (SSD) gp *= g;
 #pragma unroll
                 for (int j = 0; j < DPER; j += 4) {
                     const float4 kk = kq[j >> 2], q4 = qq[j >> 2];
-                    S[j] = fmaf(dec, S[j], kk.x * vv); S[j + 1] = fmaf(dec, S[j + 1], kk.y * vv);
-                    S[j + 2] = fmaf(dec, S[j + 2], kk.z * vv); S[j + 3] = fmaf(dec, S[j + 3], kk.w * vv);
+                    S[j] = fmaf(g, S[j], kk.x * vv); S[j + 1] = fmaf(g, S[j + 1], kk.y * vv);
+                    S[j + 2] = fmaf(g, S[j + 2], kk.z * vv); S[j + 3] = fmaf(g, S[j + 3], kk.w * vv);
                     o0 = fmaf(S[j], q4.x, o0); o1 = fmaf(S[j + 1], q4.y, o1);
                     o0 = fmaf(S[j + 2], q4.z, o0); o1 = fmaf(S[j + 3], q4.w, o1);
                 }
-                const float o = group_sum<R>(o0 + o1);
+                float o = group_sum<R>(o0 + o1);
+                if (SSD) o = fmaf(ssd_d, vs[tt][cl], o);
                 if (live && r == 0) {
                     float* dst = a.out + ((size_t)(row0 + c0 + tt) * a.H + h) * a.Dv + col;
                     *dst = pass == 2 ? *dst + o : o;
@@ -359,6 +378,7 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
         for (int j = 0; j < DPER; ++j)
             if (j < J) to[((size_t)j * a.Dv + col) * R + r] = S[j];
     }
+    if (SSD && pass == 1 && blockIdx.x == 0 && tid == 0) a.prod[((size_t)b * a.n_chunks + chunk) * a.H + h] = gp;
     if ((MODE == XR_REC_WKV || MODE == XR_REC_GLA) && pass == 1 && col == 0) {      // every column holds the same products: the first writes them
         float* pp = a.prod + (((size_t)b * a.n_chunks + chunk) * a.H + h) * J * R;
 #pragma unroll
@@ -370,7 +390,7 @@ __global__ __launch_bounds__(256) void k_recurrence(RecArgs a) {
 // Between the two passes over the chunks: scratch[b][c] holds chunk c's last state as if it had begun at
 // zero (chunk 0's is true).  In place, chunk by chunk: the true first state of chunk c (for pass 2), and
 // at the end the request's new state.  One thread an element of a head's state.
-template <bool WKV>
+template <int PROD>         // 0: decay^length; 1: a product a key channel; 2: a product a head
 __global__ __launch_bounds__(256) void k_retention_carry(RecArgs a, int per_head, int R) {
     const int b = blockIdx.z, h = blockIdx.y;
     const int e = blockIdx.x * 256 + threadIdx.x;
@@ -378,18 +398,19 @@ __global__ __launch_bounds__(256) void k_retention_carry(RecArgs a, int per_head
     const int n = a.cu_q[b + 1] - a.cu_q[b];
     if (n <= 0) return;
     const int nc = (n + a.chunk_len - 1) / a.chunk_len;
-    const float dec = WKV ? 1.f : a.decay[h];
+    const float dec = PROD ? 1.f : a.decay[h];
     const size_t step = (size_t)a.H * per_head;
     float* cp = a.scratch + ((size_t)b * a.n_chunks * a.H + h) * per_head + e;
     // (wkv) element e = (j Dv + c) R + r of the state is row R j + r, whose product lies at j R + r
     const int JR = per_head / a.Dv;
-    const float* pp = WKV ? a.prod + ((size_t)b * a.n_chunks * a.H + h) * JR + (e / (a.Dv * R)) * R + e % R : nullptr;
+    const float* pp = PROD == 1 ? a.prod + ((size_t)b * a.n_chunks * a.H + h) * JR + (e / (a.Dv * R)) * R + e % R
+                    : PROD == 2 ? a.prod + (size_t)b * a.n_chunks * a.H + h : nullptr;
     float t = cp[0];
     for (int c = 1; c < nc; ++c) {
         const int len = n - c * a.chunk_len < a.chunk_len ? n - c * a.chunk_len : a.chunk_len;
         const float own = cp[c * step];
         cp[c * step] = t;
-        t = fmaf(WKV ? pp[(size_t)c * a.H * JR] : powf(dec, (float)len), t, own);
+        t = fmaf(PROD == 1 ? pp[(size_t)c * a.H * JR] : PROD == 2 ? pp[(size_t)c * a.H] : powf(dec, (float)len), t, own);
     }
     a.state[((size_t)a.slots[b] * a.H + h) * per_head + e] = t;
 }
@@ -408,13 +429,14 @@ extern "C" int xr_linear_recurrence(float* out, const float* q, const float* k, 
                                     hipStream_t stream) {
     XR_REQUIRE(B >= 0 && H > 0 && G > 0 && H % G == 0, "recurrence: %d heads over %d key heads", H, G);
     XR_REQUIRE(D > 0 && D <= 256 && Dv > 0, "recurrence: key size %d (1 to 256), value size %d", D, Dv);
-    XR_REQUIRE(mode >= XR_REC_RETENTION && mode <= XR_REC_DELTA_CH, "recurrence: mode %d", mode);
+    XR_REQUIRE(mode >= XR_REC_RETENTION && mode <= XR_REC_SSD, "recurrence: mode %d", mode);
     const bool chain = mode == XR_REC_DELTA || mode == XR_REC_DELTA_CH;
     XR_REQUIRE(mode == XR_REC_RETENTION ? decay != nullptr : chain ? (beta != nullptr && gate != nullptr)
                : mode == XR_REC_GLA ? gate != nullptr : (gate != nullptr && decay != nullptr),
                "recurrence: the mode's gates are missing");
     XR_REQUIRE(mode != XR_REC_WKV || (G == H && ld_g >= H * D && act == 0), "recurrence: wkv has a key head a head and decays of %d x %d a row", H, D);
     XR_REQUIRE(mode != XR_REC_GLA || (G == H && ld_g >= H * D), "recurrence: gla has a key head a head and decays of %d x %d a row", H, D);
+    XR_REQUIRE(mode != XR_REC_SSD || (ld_g >= H && act == 0), "recurrence: ssd needs a step size of %d heads a row", H);
     XR_REQUIRE(mode != XR_REC_DELTA_CH || (ld_g >= H * D && ld_b >= H), "recurrence: the delta rule with channel decays needs decays of %d x %d a row", H, D);
     XR_REQUIRE(mode != XR_REC_DELTA || ld_b >= H, "recurrence: beta of %d heads a row", H);
     XR_REQUIRE(out && q && k && v && state && cu_q && slots, "recurrence: a pointer is missing");
@@ -423,7 +445,7 @@ extern "C" int xr_linear_recurrence(float* out, const float* q, const float* k, 
     const bool chunks = chunk_len > 0;
     XR_REQUIRE(!chunks || (!chain && n_chunks > 1 && scratch && chunk_len % REC_TOKENS == 0),
                "recurrence: chunks are for retention and wkv, with room for their states");
-    XR_REQUIRE(!chunks || (mode != XR_REC_WKV && mode != XR_REC_GLA) || prod, "recurrence: channel decays in chunks need room for the chunks' decay products");
+    XR_REQUIRE(!chunks || mode == XR_REC_RETENTION || prod, "recurrence: channel decays in chunks need room for the chunks' decay products");
     XR_REQUIRE(!chunks || (long long)B * n_chunks <= 65535, "recurrence: %d requests of %d chunks", B, n_chunks);
     RecArgs a{out, q, k, v, beta, gate, decay, state, cu_q, slots, H, G, D, Dv, ld, ld_g, ld_b, chunks ? 1 : 0, chunk_len, n_chunks, scratch, act, prod,
               q_scale, k_scale};
@@ -440,15 +462,18 @@ extern "C" int xr_linear_recurrence(float* out, const float* q, const float* k, 
     else if (mode == XR_REC_DELTA_CH) REC(XR_REC_DELTA_CH);
     else if (mode == XR_REC_WKV) REC(XR_REC_WKV);
     else if (mode == XR_REC_GLA) REC(XR_REC_GLA);
+    else if (mode == XR_REC_SSD) REC(XR_REC_SSD);
     else REC(XR_REC_RETENTION);
     if (chunks) {
         const int per_head = per * Dv * R;
         const dim3 cgrid((per_head + 255) / 256, H, B);
-        if (mode == XR_REC_WKV || mode == XR_REC_GLA) k_retention_carry<true><<<cgrid, 256, 0, stream>>>(a, per_head, R);
-        else k_retention_carry<false><<<cgrid, 256, 0, stream>>>(a, per_head, R);
+        if (mode == XR_REC_WKV || mode == XR_REC_GLA) k_retention_carry<1><<<cgrid, 256, 0, stream>>>(a, per_head, R);
+        else if (mode == XR_REC_SSD) k_retention_carry<2><<<cgrid, 256, 0, stream>>>(a, per_head, R);
+        else k_retention_carry<0><<<cgrid, 256, 0, stream>>>(a, per_head, R);
         a.pass = 2;
         if (mode == XR_REC_WKV) REC(XR_REC_WKV);
         else if (mode == XR_REC_GLA) REC(XR_REC_GLA);
+        else if (mode == XR_REC_SSD) REC(XR_REC_SSD);
         else REC(XR_REC_RETENTION);
     }
 #undef REC

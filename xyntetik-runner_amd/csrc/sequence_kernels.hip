@@ -114,7 +114,7 @@ extern "C" int xr_layernorm(void* out, const float* x, const float* w, const int
 }
 
 // ---------------------------------------------------------------- short causal convolution over time
-// y_t[c] = sum_j w[c][j] * u_(t - taps + 1 + j)[c]  (+ u_t[c] with `residual`), then the activation.
+// y_t[c] = sum_j w[c][j] * u_(t - taps + 1 + j)[c]  (+ bias[c]) (+ u_t[c] with `residual`), then the activation.
 // Inputs before a portion's first row come from the request's state row, which holds its last
 // taps - 1 inputs, oldest first, and is zero for a request that begins.  The state is rewritten by
 // a second kernel once every row has been read; in a step where every request brings one row
@@ -125,7 +125,7 @@ extern "C" int xr_layernorm(void* out, const float* x, const float* w, const int
 
 template <typename TU, typename TO>
 __global__ __launch_bounds__(256) void k_causal_conv(TO* __restrict__ out, const TU* __restrict__ u,
-                                                     const float* __restrict__ w, TU* state,
+                                                     const float* __restrict__ w, const float* __restrict__ bias, TU* state,
                                                      const int* __restrict__ cu_q, const int* __restrict__ slots,
                                                      const int* __restrict__ req_of_token, int C, int taps, int ld_u,
                                                      int ld_out, int residual, int act, int fuse) {
@@ -144,6 +144,7 @@ __global__ __launch_bounds__(256) void k_causal_conv(TO* __restrict__ out, const
         // one row a request: input j of this row is state entry j, which moves one place down
         if (fuse && j > 0) st<TU>(srow, (size_t)(j - 1) * C + c, val);
     }
+    if (bias) acc += bias[c];
     if (residual) acc += ld<TU>(u, (size_t)t * ld_u + c);
     if (act == XR_CONV_SILU) acc = acc / (1.0f + expf(-acc));
     st<TO>(out, (size_t)t * ld_out + c, acc);
@@ -157,7 +158,8 @@ __global__ __launch_bounds__(256) void k_causal_conv(TO* __restrict__ out, const
 #define CONV_ROWS 8
 template <typename TU, typename TO>
 __global__ __launch_bounds__(256) void k_causal_conv_rows(TO* __restrict__ out, const TU* __restrict__ u,
-                                                          const float* __restrict__ w, const TU* __restrict__ state,
+                                                          const float* __restrict__ w, const float* __restrict__ bias,
+                                                          const TU* __restrict__ state,
                                                           const int* __restrict__ cu_q, const int* __restrict__ slots,
                                                           const int* __restrict__ req_of_token, int T, int C, int taps,
                                                           int ld_u, int ld_out, int residual, int act) {
@@ -174,6 +176,7 @@ __global__ __launch_bounds__(256) void k_causal_conv_rows(TO* __restrict__ out, 
     float wt[CONV_MAX_TAPS];
 #pragma unroll
     for (int j = 0; j < CONV_MAX_TAPS; ++j) wt[j] = j < taps ? w[(size_t)c * taps + j] : 0.f;
+    const float bc = bias ? bias[c] : 0.f;
 #pragma unroll
     for (int r = 0; r < CONV_ROWS; ++r) {
         const int t = t0 + r;
@@ -188,6 +191,7 @@ __global__ __launch_bounds__(256) void k_causal_conv_rows(TO* __restrict__ out, 
             const float val = s >= 0 ? ld<TU>(u, (size_t)(row0[r] + s) * ld_u + c) : ld<TU>(srow, (size_t)(taps - 1 + s) * C + c);
             acc = fmaf(wt[j], val, acc);
         }
+        acc += bc;
         if (residual) acc += ld<TU>(u, (size_t)t * ld_u + c);
         if (act == XR_CONV_SILU) acc = acc / (1.0f + expf(-acc));
         st<TO>(out, (size_t)t * ld_out + c, acc);
@@ -218,7 +222,7 @@ __global__ __launch_bounds__(256) void k_conv_state(TU* __restrict__ state, cons
     }
 }
 
-extern "C" int xr_causal_conv(void* out, const void* u, const float* w, void* state, const int* cu_q, const int* slots,
+extern "C" int xr_causal_conv(void* out, const void* u, const float* w, const float* bias, void* state, const int* cu_q, const int* slots,
                               const int* req_of_token, int T, int B, int C, int taps, int ld_u, int ld_out,
                               int u_dtype, int out_dtype, int residual, int act, int one_row_each, hipStream_t stream) {
     XR_REQUIRE(T >= 0 && B >= 0 && C > 0 && ld_u >= C && ld_out >= C, "causal_conv: bad sizes T=%d B=%d C=%d ld_u=%d ld_out=%d",
@@ -235,11 +239,11 @@ extern "C" int xr_causal_conv(void* out, const void* u, const float* w, void* st
 #define CC(TU, TO)                                                                                                   \
     do {                                                                                                             \
         if (T >= 8 * CONV_ROWS && !fuse)                                                                             \
-            k_causal_conv_rows<TU, TO><<<rgrid, 256, 0, stream>>>((TO*)out, (const TU*)u, w, (const TU*)state, cu_q,  \
+            k_causal_conv_rows<TU, TO><<<rgrid, 256, 0, stream>>>((TO*)out, (const TU*)u, w, bias, (const TU*)state, cu_q,  \
                                                                   slots, req_of_token, T, C, taps, ld_u, ld_out,     \
                                                                   residual, act);                                    \
         else                                                                                                         \
-        k_causal_conv<TU, TO><<<grid, 256, 0, stream>>>((TO*)out, (const TU*)u, w, (TU*)state, cu_q, slots,           \
+        k_causal_conv<TU, TO><<<grid, 256, 0, stream>>>((TO*)out, (const TU*)u, w, bias, (TU*)state, cu_q, slots,           \
                                                         req_of_token, C, taps, ld_u, ld_out, residual, act, fuse);    \
         if (taps > 1 && !fuse) k_conv_state<TU><<<sgrid, 256, 0, stream>>>((TU*)state, (const TU*)u, cu_q, slots, C, taps, ld_u); \
     } while (0)
@@ -440,62 +444,72 @@ extern "C" int xr_rotate_rows(float* x, const int* positions, const float* inv_f
 // out[t][h][d] = o[t][h][d] / sqrt(mean_d(o^2) + eps) * w * act(gate[t][h][d]); w may be absent, is one
 // weight a channel of a head that the heads share (w [Dv]) or, with w_full, one a channel of the row
 // (w [H * Dv]); act is SiLU (gate_act 0) or the sigmoid (1).  A norm over all heads together is
-// H = 1 with Dv the whole row.  One wave per (token, head).
+// H = 1 with Dv the whole row.  One wave per (token, head).  With gate_first the gate comes before the norm:
+// u = o * act(gate), out = u / sqrt(mean_d(u^2) + eps) * w.  Everything is multiplied by `scale` at last; output rows are
+// ld_out apart.
 #define XR_GATE_SILU 0
 #define XR_GATE_SIGMOID 1
+__device__ inline float norm_gate(float g, int gate_act) {
+    const float sg = 1.0f / (1.0f + expf(-g));
+    return gate_act == XR_GATE_SIGMOID ? sg : g * sg;
+}
 template <typename TO>
 __global__ __launch_bounds__(64) void k_gated_rmsnorm(TO* __restrict__ out, const float* __restrict__ o,
                                                       const float* __restrict__ gate, const float* __restrict__ w,
-                                                      int H, int Dv, int ld_g, float eps, int w_full, int gate_act) {
+                                                      int H, int Dv, int ld_g, float eps, int w_full, int gate_act,
+                                                      int gate_first, float scale, int ld_out) {
     const int t = blockIdx.x, h = blockIdx.y;
     const float* orow = o + ((size_t)t * H + h) * Dv;
     const float* grow = gate + (size_t)t * ld_g + (size_t)h * Dv;
     const float* wrow = w ? (w_full ? w + (size_t)h * Dv : w) : nullptr;
     float ss = 0.f;
-    for (int d = threadIdx.x; d < Dv; d += 64) ss += orow[d] * orow[d];
-    const float rinv = 1.0f / sqrtf(wave_sum(ss) / (float)Dv + eps);
-    TO* dst = out + ((size_t)t * H + h) * Dv;
     for (int d = threadIdx.x; d < Dv; d += 64) {
-        const float g = grow[d];
-        const float sg = 1.0f / (1.0f + expf(-g));
-        st<TO>(dst, d, orow[d] * rinv * (wrow ? wrow[d] : 1.f) * (gate_act == XR_GATE_SIGMOID ? sg : g * sg));
+        const float u = gate_first ? orow[d] * norm_gate(grow[d], gate_act) : orow[d];
+        ss += u * u;
     }
+    const float rinv = scale / sqrtf(wave_sum(ss) / (float)Dv + eps);
+    TO* dst = out + (size_t)t * ld_out + (size_t)h * Dv;
+    for (int d = threadIdx.x; d < Dv; d += 64)
+        st<TO>(dst, d, orow[d] * rinv * (wrow ? wrow[d] : 1.f) * norm_gate(grow[d], gate_act));
 }
 
 // The same with a workgroup of 256 a (token, head), for long rows (all heads normed together).
 template <typename TO>
 __global__ __launch_bounds__(256) void k_gated_rmsnorm_wide(TO* __restrict__ out, const float* __restrict__ o,
                                                            const float* __restrict__ gate, const float* __restrict__ w,
-                                                           int H, int Dv, int ld_g, float eps, int w_full, int gate_act) {
+                                                           int H, int Dv, int ld_g, float eps, int w_full, int gate_act,
+                                                           int gate_first, float scale, int ld_out) {
     __shared__ float part[4];
     const int t = blockIdx.x, h = blockIdx.y;
     const float* orow = o + ((size_t)t * H + h) * Dv;
     const float* grow = gate + (size_t)t * ld_g + (size_t)h * Dv;
     const float* wrow = w ? (w_full ? w + (size_t)h * Dv : w) : nullptr;
     float ss = 0.f;
-    for (int d = threadIdx.x; d < Dv; d += 256) ss += orow[d] * orow[d];
+    for (int d = threadIdx.x; d < Dv; d += 256) {
+        const float u = gate_first ? orow[d] * norm_gate(grow[d], gate_act) : orow[d];
+        ss += u * u;
+    }
     ss = wave_sum(ss);
     if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = ss;
     __syncthreads();
-    const float rinv = 1.0f / sqrtf(((part[0] + part[1]) + (part[2] + part[3])) / (float)Dv + eps);
-    TO* dst = out + ((size_t)t * H + h) * Dv;
-    for (int d = threadIdx.x; d < Dv; d += 256) {
-        const float g = grow[d];
-        const float sg = 1.0f / (1.0f + expf(-g));
-        st<TO>(dst, d, orow[d] * rinv * (wrow ? wrow[d] : 1.f) * (gate_act == XR_GATE_SIGMOID ? sg : g * sg));
-    }
+    const float rinv = scale / sqrtf(((part[0] + part[1]) + (part[2] + part[3])) / (float)Dv + eps);
+    TO* dst = out + (size_t)t * ld_out + (size_t)h * Dv;
+    for (int d = threadIdx.x; d < Dv; d += 256)
+        st<TO>(dst, d, orow[d] * rinv * (wrow ? wrow[d] : 1.f) * norm_gate(grow[d], gate_act));
 }
 
 extern "C" int xr_gated_rmsnorm(void* out, const float* o, const float* gate, const float* w, int T, int H, int Dv,
-                                int ld_g, float eps, int out_dtype, int w_full, int gate_act, hipStream_t stream) {
+                                int ld_g, float eps, int out_dtype, int w_full, int gate_act, int gate_first, float scale,
+                                int ld_out, hipStream_t stream) {
+    XR_REQUIRE(ld_out >= H * Dv, "gated_rmsnorm: output rows of %d are %d apart", H * Dv, ld_out);
     XR_REQUIRE(T >= 0 && H > 0 && Dv > 0 && ld_g >= H * Dv, "gated_rmsnorm: bad sizes T=%d H=%d Dv=%d ld=%d", T, H, Dv, ld_g);
     XR_REQUIRE(gate_act == XR_GATE_SILU || gate_act == XR_GATE_SIGMOID, "gated_rmsnorm: unknown gate activation %d", gate_act);
     if (T == 0) return XR_OK;
     const bool wide = Dv > 256;       // (the sums' order differs between the two kernels, not between calls of one size)
-    if (out_dtype == XR_F32 && wide) k_gated_rmsnorm_wide<float><<<dim3(T, H), 256, 0, stream>>>((float*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act);
-    else if (out_dtype == XR_BF16 && wide) k_gated_rmsnorm_wide<bf16_t><<<dim3(T, H), 256, 0, stream>>>((bf16_t*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act);
-    else if (out_dtype == XR_F32) k_gated_rmsnorm<float><<<dim3(T, H), 64, 0, stream>>>((float*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act);
-    else if (out_dtype == XR_BF16) k_gated_rmsnorm<bf16_t><<<dim3(T, H), 64, 0, stream>>>((bf16_t*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act);
+    if (out_dtype == XR_F32 && wide) k_gated_rmsnorm_wide<float><<<dim3(T, H), 256, 0, stream>>>((float*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
+    else if (out_dtype == XR_BF16 && wide) k_gated_rmsnorm_wide<bf16_t><<<dim3(T, H), 256, 0, stream>>>((bf16_t*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
+    else if (out_dtype == XR_F32) k_gated_rmsnorm<float><<<dim3(T, H), 64, 0, stream>>>((float*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
+    else if (out_dtype == XR_BF16) k_gated_rmsnorm<bf16_t><<<dim3(T, H), 64, 0, stream>>>((bf16_t*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
     else { xr_set_error("gated_rmsnorm: bad dtype %d", out_dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("gated_rmsnorm");
     return XR_OK;
@@ -505,6 +519,7 @@ extern "C" int xr_gated_rmsnorm(void* out, const float* o, const float* gate, co
 // x[t][c] <- act(x[t][c]) for the first W columns of rows of stride ld, in place; or, with `out`, into
 // contiguous rows [T, W] of the type the next product reads.  act 1 = SiLU, 2 = tanh.
 #define XR_ACT_ROWS_TANH 2
+#define XR_ACT_ROWS_RELU2 3
 template <typename TO>
 __global__ void k_act_rows(float* __restrict__ x, TO* __restrict__ out, int W, int ld, size_t n, int act) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -512,14 +527,15 @@ __global__ void k_act_rows(float* __restrict__ x, TO* __restrict__ out, int W, i
     const size_t t = i / W;
     float* p = x + t * ld + (i - t * W);
     const float v = *p;
-    const float y = act == XR_ACT_ROWS_TANH ? tanhf(v) : v / (1.0f + expf(-v));
+    const float r = fmaxf(v, 0.f);
+    const float y = act == XR_ACT_ROWS_TANH ? tanhf(v) : act == XR_ACT_ROWS_RELU2 ? r * r : v / (1.0f + expf(-v));
     if (out) st<TO>(out, i, y);
     else *p = y;
 }
 
 extern "C" int xr_act_rows(float* x, int T, int W, int ld, int act, void* out, int out_dtype, hipStream_t stream) {
     XR_REQUIRE(T >= 0 && W > 0 && ld >= W, "act_rows: bad sizes T=%d W=%d ld=%d", T, W, ld);
-    XR_REQUIRE(act == XR_CONV_SILU || act == XR_ACT_ROWS_TANH, "act_rows: activation %d is not built (1 = SiLU, 2 = tanh)", act);
+    XR_REQUIRE(act == XR_CONV_SILU || act == XR_ACT_ROWS_TANH || act == XR_ACT_ROWS_RELU2, "act_rows: activation %d is not built (1 = SiLU, 2 = tanh, 3 = relu squared)", act);
     XR_REQUIRE(!out || out_dtype == XR_F32 || out_dtype == XR_BF16, "act_rows: output type %d", out_dtype);
     const size_t n = (size_t)T * W;
     if (n == 0) return XR_OK;

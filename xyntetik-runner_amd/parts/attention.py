@@ -23,11 +23,16 @@ run in); ``keep_first``: with a window, the first so many keys stay readable, at
 tensor ``sink_name``, unscaled) or "zero" (the score 0: one is added to the denominator); ``gate_name``: a
 projection ``[H, E]`` of the mixer's input whose sigmoid multiplies every head's output before the output
 projection; ``softcap`` c > 0: every scaled score s becomes ``c tanh(s / c)`` (before a slope's bias and not the sink).
+
+Where values have another size than keys, or a head norm comes behind the rotation, one kernel takes the input product's
+32-bit rows through norm and rotation to the queries and the cache, and the gate's rows are part of that product.  Such an
+attention may also be a side of a joint pair of mixers (``parts/parallel.py``): its input rows and output columns are then
+part of the pair's two products (``joint_*``).
 """
 from __future__ import annotations
 
 import math
-from typing import Dict, Optional
+from typing import Dict, Optional, Tuple
 
 import torch
 
@@ -96,6 +101,13 @@ class PagedAttention(Mixer):
         # any rows, so keys that are the values stand once in the input matrix
         self.row_normed = (self.qk_transform is not None and hasattr(self.qk_transform, "row_norm") and self.v_head_dim == self.head_dim
                            and (self.position is None or type(self.position).rotary is not PositionEncoding.rotary))
+        # one kernel from the product's rows through a norm a head and the rotation to the queries and the cache
+        self.head_kernel = ((self.position is None or type(self.position).rotary is not PositionEncoding.rotary)
+                            and (self.qk_transform is None or (hasattr(self.qk_transform, "head_norm") and self.qk_transform.can_head_norm)))
+        late = bool(getattr(self.qk_transform, "after_rotation", False))
+        if late and not self.head_kernel:
+            raise ValueError("attention: a norm behind the rotation needs a rotation by a table and both sides normed, without a temperature")
+        self.by_head = self.head_kernel and (late or self.v_head_dim != self.head_dim)
         self.q_size = self.num_heads * self.head_dim
         self.kv_size = self.num_kv_heads * self.head_dim
         self.v_size = self.num_kv_heads * self.v_head_dim
@@ -141,15 +153,67 @@ class PagedAttention(Mixer):
         return ((self.position is None or self.position.capturable)
                 and (self.qk_transform is None or self.qk_transform.capturable))
 
-    def bind(self, tensors, rt) -> None:
+    def _input_names(self):
+        """The projections of the input product, in its rows' order."""
+        q, k, v, _ = self.names
+        if self.kv_shared:
+            return [q]
+        return [q, k] if self.values_are_keys else [q, k, v]
+
+    def _bind_constants(self, tensors, rt) -> None:
         self.rt = rt
         if self.position is not None:
             self.position.bind({}, rt)
         if self.qk_transform is not None:
             self.qk_transform.bind({n: tensors[n] for n in self.qk_transform.param_specs()}, rt)
+        if self.slope_values is not None:
+            self.slopes = torch.tensor(self.slope_values, dtype=torch.float32, device=rt.device)
+        if self.sink == "learned":
+            self.sinks = tensors[self.sink_name].float().contiguous()
+        elif self.sink == "zero":
+            self.sinks = torch.zeros((self.num_heads,), dtype=torch.float32, device=rt.device)
+
+    # ------------------------------------------------------------------ as a side of a joint pair of mixers
+    @property
+    def joint(self) -> bool:
+        return self.head_kernel
+
+    def joint_inputs(self, tensors) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+        """(rows of the input product: queries, keys, values, the gate; their 32-bit biases or None)."""
+        names = self._input_names()
+        mats = [tensors[f"{n}{self.w_sfx}"] for n in names]
+        bias = [tensors[f"{n}{self.b_sfx}"].float() for n in names] if self.bias else []
+        if self.gate_name is not None:
+            mats.append(tensors[f"{self.gate_name}{self.w_sfx}"])
+            if bias:
+                bias.append(torch.zeros((self.num_heads,), dtype=torch.float32, device=bias[0].device))
+        return torch.cat(mats, dim=0).contiguous(), torch.cat(bias).contiguous() if bias else None
+
+    def joint_outputs(self, tensors) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+        """(the output projection ``[E, H * Dv]``, its bias or None)."""
+        o = self.names[3]
+        return tensors[f"{o}{self.w_sfx}"], tensors[f"{o}{self.b_sfx}"].float() if self.out_bias else None
+
+    def joint_bind(self, tensors, rt) -> None:
+        self._bind_constants(tensors, rt)
+
+    def joint_read_out(self, ctx, cache, proj, out, scale: float) -> None:
+        """What the output projection reads, times ``scale``, into the view ``out [T, H * Dv]``, from the input product's
+        32-bit rows ``proj`` (in the order of ``joint_inputs``)."""
+        self._attend_rows(ctx, cache, proj, out=out, scale=scale)
+
+    def bind(self, tensors, rt) -> None:
+        self._bind_constants(tensors, rt)
         q, k, v, o = self.names
         H, Hk, D = self.num_heads, self.num_kv_heads, self.head_dim
         ws, bsf = self.w_sfx, self.b_sfx
+        self.paired = False
+        if self.by_head:
+            w_in, self.b_in = self.joint_inputs(tensors)
+            self.w_in = rt.ops.pack_weight(w_in)
+            w_out, self.b_out = self.joint_outputs(tensors)
+            self.w_out = rt.ops.pack_weight(w_out)
+            return
         # the value projection is the key projection: its rows stand twice in the one matrix, or once where the kernel
         # behind the product takes both from the same columns
         inputs = [q] if self.kv_shared else [q, k, k if self.values_are_keys else v]
@@ -160,12 +224,6 @@ class PagedAttention(Mixer):
         b_in = None
         if self.bias:
             b_in = torch.cat([tensors[f"{n}{bsf}"].float() for n in inputs]).contiguous()
-        if self.slope_values is not None:
-            self.slopes = torch.tensor(self.slope_values, dtype=torch.float32, device=rt.device)
-        if self.sink == "learned":
-            self.sinks = tensors[self.sink_name].float().contiguous()
-        elif self.sink == "zero":
-            self.sinks = torch.zeros((H,), dtype=torch.float32, device=rt.device)
         if self.gate_name is not None:
             self.w_gate = rt.ops.pack_weight(tensors[f"{self.gate_name}{ws}"].contiguous())
         # A rotation that pairs channel j with j + rot/2: the rows of every query and key head go
@@ -189,8 +247,27 @@ class PagedAttention(Mixer):
         if self.out_bias:
             self.b_out = tensors[f"{o}{bsf}"].float().contiguous()
 
+    def _attend_rows(self, ctx, cache, proj, out=None, scale: float = 1.0):
+        """Attention from the input product's rows: ``[queries | keys | values | gate]``, channels in the checkpoint's order."""
+        ops, rt = self.rt.ops, self.rt
+        Q, K, V, H, Hk, D, Dv = self.q_size, self.kv_size, self.v_size, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim
+        writes = not self.kv_shared and cache.owns
+        rot = self.position.rotary() if self.position is not None else None
+        gate = proj[:, proj.shape[1] - H:] if self.gate_name is not None else None
+        k_in = proj[:, Q:Q + K] if writes else None
+        v_in = k_in if self.values_are_keys or not writes else proj[:, Q + K:Q + K + V]
+        w_q, w_k, eps, order = self.qk_transform.head_norm() if self.qk_transform is not None else (None, None, 0.0, None)
+        q = ops.head_norm_rope_write(proj[:, :Q], k_in, v_in, w_q, w_k, eps, order, cache.k, cache.v, ctx, cache.group,
+                                     rot.inv_freq if rot else None, H, Hk, D, Dv, rot.rotary_dim if rot else 0,
+                                     rot.interleaved if rot else False, rot.mscale if rot else 1.0, cache.page_size, rt.dtype)
+        return ops.attention(q, cache.k, cache.v, ctx, cache.group, H, Hk, D, cache.page_size, self.scale, self.window,
+                             slopes=self.slopes, chunk=self.chunk, keep_first=self.keep_first, sinks=self.sinks, v_head_dim=Dv,
+                             softcap=self.softcap, gate=gate, out_scale=scale, out=out)
+
     def _attend(self, ctx, cache, h):
         ops, rt = self.rt.ops, self.rt
+        if self.by_head:
+            return self._attend_rows(ctx, cache, ops.linear(h, self.w_in, bias=self.b_in, out_dtype=torch.float32))
         Q, K, H, Hk, D = self.q_size, self.kv_size, self.num_heads, self.num_kv_heads, self.head_dim
         Dv, V = self.v_head_dim, self.v_size
         T = h.shape[0]
@@ -282,6 +359,13 @@ class PagedAttention(Mixer):
             return super().forward_add_norm(ctx, cache, h, residual, norm, defer)
         return self.rt.ops.linear_add_rmsnorm(self._attend(ctx, cache, h), self.w_out, residual, fold[0], fold[1],
                                               self.rt.dtype, bias=self.b_out, defer=defer, centred=fold[2])
+
+
+    def forward_post(self, ctx, cache, h, x, alpha, norm):
+        w, eps = norm.fold()
+        if w.dtype != torch.float32:
+            return super().forward_post(ctx, cache, h, x, alpha, norm)
+        return self.rt.ops.linear_post_norm(self._attend(ctx, cache, h), self.w_out, x, alpha, w, eps, self.rt.dtype, bias=self.b_out)
 
 
 register_mixer("paged_attention", PagedAttention)

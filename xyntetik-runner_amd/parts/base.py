@@ -32,6 +32,9 @@ Families and what each must offer:
 * ``Block``: the arrangement; it names its norms (``norm_names``), may do without a mixer or a
   feed-forward, and ``forward(ctx, cache, x)`` updates ``x`` in place.
 
+``forward_post(..., x, alpha, norm)`` of a mixer or feed-forward is for an arrangement whose residual stream is normed
+behind every sum: ``x <- norm(alpha x + result)`` in place, the new rows in the compute dtype come back.
+
 Optional, for fewer kernels when a few tokens are decoded: a mixer or feed-forward
 may override ``forward_add_norm(..., residual, norm, defer)``, which adds into the
 residual stream and returns ``norm`` of the result, so that its last product can do
@@ -215,6 +218,21 @@ class Mixer(Part):
         self.forward_add(ctx, cache, h, residual)
         return norm.forward(ctx, residual)
 
+    def forward_post(self, ctx, cache, h, x: torch.Tensor, alpha: float, norm: Norm) -> torch.Tensor:
+        """``x <- norm(alpha x + forward(h))``; a part whose last kernel can do that overrides it."""
+        return post_sum(ctx, self.rt.dtype, x, self.forward_f32(ctx, cache, h), alpha, norm)
+
+
+def post_sum(ctx, dtype, x: torch.Tensor, y: torch.Tensor, alpha: float, norm: Norm) -> torch.Tensor:
+    """``x <- norm(alpha x + y)`` by a kernel of its own; the new rows in ``dtype``."""
+    w, eps = norm.fold()
+    if w.dtype != torch.float32:                # (a weight kept in bfloat16; once, the norm keeps the copy)
+        kept = getattr(norm, "_f32_weight", None)
+        if kept is None or kept[0] is not w:
+            kept = norm._f32_weight = (w, w.float().contiguous())
+        w = kept[1]
+    return ctx.ops.post_norm(x, y.contiguous(), alpha, w, eps, dtype)
+
 
 class SequenceFilter(Part):
     """What a sublayer's input passes through on its way from the norm, with the inputs it carries
@@ -265,6 +283,10 @@ class FeedForward(Part):
         """``forward_add``, then ``norm`` of the updated residual stream."""
         self.forward_add(ctx, h, residual)
         return norm.forward(ctx, residual)
+
+    def forward_post(self, ctx, h, x: torch.Tensor, alpha: float, norm: Norm) -> torch.Tensor:
+        """As ``Mixer.forward_post``."""
+        return post_sum(ctx, self.rt.dtype, x, self.forward_f32(ctx, h), alpha, norm)
 
 
 class Block:

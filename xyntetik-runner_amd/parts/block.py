@@ -15,6 +15,10 @@ without a feed-forward.
 ``[S, T, E]``; the model makes the copies after the embedding and adds them up before the final norm.
 The write of one sublayer and the read and norm of the next run in one kernel.
 
+"postnorm": the residual stream itself is normed behind every sum: ``x <- norm_m(alpha x + mixer(x)); x <-
+norm_f(alpha x + feed_forward(x))`` with one number ``alpha``; the sublayers read the stream as it is (in the
+compute dtype), and a layer without a feed-forward ends behind the first norm.
+
 "sandwich": every sublayer is normed before and after, and what it adds is scaled:
 ``x += m post_m(mixer(pre_m(x))); x += m post_f(feed_forward(pre_f(x)))`` with one number ``m`` for the
 layer.  A layer of it may come without a feed-forward.  Where all four norms are dynamic tanh, which
@@ -27,7 +31,7 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import Block, Connection, ParamSpec, register_block, register_connection
+from .base import Block, Connection, Norm, ParamSpec, register_block, register_connection
 
 
 def _takes_unscaled(part) -> bool:
@@ -63,6 +67,9 @@ class PreNormBlock(Block):
             h = self.feed_forward_norm.forward(ctx, x)
         add_norm = getattr(self.feed_forward, "forward_add_norm", None)
         if after is None or add_norm is None:
+            self.feed_forward.forward_add(ctx, h, x)
+            return None
+        if not isinstance(after, tuple):        # (a block of another arrangement makes its first input itself)
             self.feed_forward.forward_add(ctx, h, x)
             return None
         next_norm, defer = after
@@ -248,7 +255,37 @@ class SandwichBlock(Block):
         return self._add(ctx, x, y, self.norms["feed_forward_post_norm"], nxt)
 
 
+class PostNormEntry:
+    """What the block before needs to make this block's first input: the stream itself, in the compute dtype."""
+
+
+class PostNormBlock(Block):
+    chained = True
+    norm_names = ("mixer_norm", "feed_forward_norm")
+    needs_feed_forward = None       # with or without; the second norm then does nothing
+
+    def __init__(self, mixer, feed_forward, norms, filters=None, connections=None, alpha: float = 1.0):
+        super().__init__(mixer, feed_forward, norms, filters, connections)
+        self.alpha = float(alpha)
+        for name, norm in self.norms.items():
+            if type(norm).fold is Norm.fold:
+                raise ValueError(f"PostNormBlock: {name} must be an RMS norm (its kernels write the norm themselves)")
+
+    def entry_norm(self):
+        return PostNormEntry()
+
+    def forward(self, ctx, cache, x, h=None, after=None):
+        """``h``: the stream in the compute dtype, if the block before left it."""
+        if h is None:
+            h = ctx.ops.convert(x.contiguous(), self.mixer.rt.dtype)
+        h = self.mixer.forward_post(ctx, cache, h, x, self.alpha, self.norms["mixer_norm"])
+        if self.feed_forward is not None:
+            h = self.feed_forward.forward_post(ctx, h, x, self.alpha, self.norms["feed_forward_norm"])
+        return h if isinstance(after, PostNormEntry) else None
+
+
 register_connection("stream_connection", StreamConnection)
+register_block("postnorm", PostNormBlock)
 register_block("sandwich", SandwichBlock)
 register_block("prenorm_streams", StreamsPreNormBlock)
 register_block("prenorm", PreNormBlock)

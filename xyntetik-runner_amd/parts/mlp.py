@@ -21,11 +21,15 @@ the chosen scores times a number (``weight_scale``) instead of their shares of t
 themselves, the correction being the router's bias (``scores="logits"``: the weights are the softmax over the chosen
 logits, bias included); experts and a shared expert gated by any gate of ``GATE_ACTIVATIONS`` with a number of its own
 (``activation``, ``activation_param``; ``shared_activation``, ``shared_param``); a number a token on the shared expert,
-``sigmoid(w . h)`` (``shared_gate_name``: the ``[1, E]`` tensor ``w``).
+``sigmoid(w . h)`` (``shared_gate_name``: the ``[1, E]`` tensor ``w``); a shared expert without a gate, ``down(relu(up h)^2)``
+(``shared_activation="relu2"``); a group's score that is its largest choice score alone (``group_score="max"``); identity
+experts (``identity`` of them behind the others in the router's rows, in the choice and in the groups: their output is the
+input itself, and they have no tensors).
 
 Dense feed-forward: ``down(act(up(h)))`` with an activation over the whole row.  "polynorm":
 ``a N(z) + b N(z^2) + c N(z^3) + e`` with four learned numbers, powers element by element and
-``N(v) = v / sqrt(mean(v^2) + eps)`` over the row, in 32-bit.
+``N(v) = v / sqrt(mean(v^2) + eps)`` over the row, in 32-bit.  "relu2": the square of what is positive, in the product's
+epilogue.
 """
 from __future__ import annotations
 
@@ -99,7 +103,7 @@ class GatedMLP(FeedForward):
 
 
 class DenseMLP(FeedForward):
-    ACTIVATIONS = ("polynorm",)
+    ACTIVATIONS = ("polynorm", "relu2")
 
     def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "polynorm", eps: float = 1e-5,
                  up_name: str = "up", down_name: str = "down", act_name: str = "act"):
@@ -113,22 +117,30 @@ class DenseMLP(FeedForward):
     def param_specs(self) -> Dict[str, ParamSpec]:
         E, F = self.hidden_size, self.intermediate_size
         u, d, a = self.names
-        return {u: ParamSpec((F, E)), d: ParamSpec((E, F)), a: ParamSpec((4,), role="vector", init="normal:0.5")}
+        specs = {u: ParamSpec((F, E)), d: ParamSpec((E, F))}
+        if self.activation == "polynorm":
+            specs[a] = ParamSpec((4,), role="vector", init="normal:0.5")
+        return specs
 
     def bind(self, tensors, rt) -> None:
         self.rt = rt
         u, d, a = self.names
         self.w_up = rt.ops.pack_weight(tensors[u])
         self.w_down = rt.ops.pack_weight(tensors[d])
-        self.coef = tensors[a].float().contiguous()
+        self.coef = tensors[a].float().contiguous() if self.activation == "polynorm" else None
 
     def _hidden(self, ctx, h):
+        if self.activation == "relu2":
+            return self.rt.ops.linear(h, self.w_up, activation="relu2")
         # the row's statistics are of the unrounded products
         z = self.rt.ops.linear(h, self.w_up, out_dtype=torch.float32)
         return self.rt.ops.polynorm(z, self.coef, self.eps, self.rt.dtype)
 
     def forward(self, ctx, h):
         return self.rt.ops.linear(self._hidden(ctx, h), self.w_down)
+
+    def forward_f32(self, ctx, h):
+        return self.rt.ops.linear(self._hidden(ctx, h), self.w_down, out_dtype=torch.float32)
 
     def forward_add(self, ctx, h, residual) -> None:
         self.rt.ops.linear(self._hidden(ctx, h), self.w_down, out=residual, accumulate=True)
@@ -151,7 +163,7 @@ class RoutedExperts(FeedForward):
                  vocab_size: int = 0, table_name: str = "table", shared_size: int = 0, shared_prefix: str = "shared.",
                  scores: str = "softmax", groups: int = 1, keep_groups: int = 1, weight_scale=None,
                  activation_param: float = 0.0, shared_activation: str = "silu", shared_param: float = 0.0,
-                 shared_gate_name: Optional[str] = None):
+                 shared_gate_name: Optional[str] = None, identity: int = 0, group_score: str = "top2"):
         if activation not in self.ACTIVATIONS:
             raise ValueError(f"routed experts: activation {activation!r} is not built (known: {list(self.ACTIVATIONS)})")
         if routing not in self.ROUTINGS:
@@ -161,32 +173,43 @@ class RoutedExperts(FeedForward):
         self.activation, self.routing, self.vocab_size = activation, routing, int(vocab_size)
         self.gate_name, self.table_name = gate_name, table_name
         self.activation_param = float(activation_param)
-        self.shared = (GatedMLP(hidden_size, int(shared_size), activation=shared_activation, activation_param=shared_param, gate_name=shared_prefix + "gate",
-                                up_name=shared_prefix + "up", down_name=shared_prefix + "down", weight_suffix="")
-                       if int(shared_size) > 0 else None)
+        self.shared = None
+        if int(shared_size) > 0 and shared_activation in DenseMLP.ACTIVATIONS:
+            self.shared = DenseMLP(hidden_size, int(shared_size), activation=shared_activation, up_name=shared_prefix + "up",
+                                   down_name=shared_prefix + "down", act_name=shared_prefix + "act")
+        elif int(shared_size) > 0:
+            self.shared = GatedMLP(hidden_size, int(shared_size), activation=shared_activation, activation_param=shared_param,
+                                   gate_name=shared_prefix + "gate", up_name=shared_prefix + "up", down_name=shared_prefix + "down",
+                                   weight_suffix="")
+        self.identity = int(identity)
+        if self.identity < 0 or (self.identity and routing != "router"):
+            raise ValueError(f"routed experts: {identity} identity experts need a router that can choose them")
+        choices = int(num_experts) + self.identity          # what the router scores
         self.shared_gate_name = shared_gate_name
         if shared_gate_name is not None and (self.shared is None or routing != "router"):
             raise ValueError("routed experts: a gate on the shared expert needs one, and a router whose product makes its logit")
-        if not (1 <= int(top) <= int(num_experts)):
-            raise ValueError(f"routed experts: {top} of {num_experts} experts a token")
-        if int(num_experts) > self.MAX_EXPERTS or int(top) > self.MAX_TOP:       # refused when the model is built, not at its first step
+        if int(num_experts) < 1 or not (1 <= int(top) <= choices):
+            raise ValueError(f"routed experts: {top} of {choices} experts a token")
+        if choices > self.MAX_EXPERTS or int(top) > self.MAX_TOP:       # refused when the model is built, not at its first step
             raise ValueError(f"routed experts: the kernels take up to {self.MAX_EXPERTS} experts and {self.MAX_TOP} a token, "
-                             f"not {num_experts} and {top}")
+                             f"not {choices} and {top}")
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
-        self.num_experts, self.top = int(num_experts), int(top)
+        self.num_experts, self.top, self.choices = int(num_experts), int(top), choices
         groups, keep_groups = int(groups), int(keep_groups)
         if scores not in ("softmax", "sigmoid", "logits"):
             raise ValueError(f"routed experts: scores {scores!r} (softmax, sigmoid or logits)")
+        if group_score not in ("top2", "max"):
+            raise ValueError(f"routed experts: a group scores its 'top2' added up or its 'max', not {group_score!r}")
         if scores == "logits" and (groups != 1 or weight_scale is not None):
             raise ValueError("routed experts: a choice by the logits has no groups, and its weights are the softmax over the chosen")
-        if (groups < 1 or self.num_experts % groups or not (1 <= keep_groups <= groups)
-                or self.top > keep_groups * (self.num_experts // groups)):
-            raise ValueError(f"routed experts: {num_experts} experts in {groups} groups of which {keep_groups} are kept "
+        if (groups < 1 or choices % groups or not (1 <= keep_groups <= groups)
+                or self.top > keep_groups * (choices // groups)):
+            raise ValueError(f"routed experts: {choices} experts in {groups} groups of which {keep_groups} are kept "
                              f"cannot give {top} choices a token")
         if weight_scale is not None and not float(weight_scale) > 0.0:
             raise ValueError(f"routed experts: weight scale {weight_scale} must be positive")
         self.how = dict(scores=scores, groups=groups, keep_groups=keep_groups,
-                        weight_scale=float(weight_scale) if weight_scale is not None else None)
+                        weight_scale=float(weight_scale) if weight_scale is not None else None, group_score=group_score)
         self.names = (router_name, correction_name, expert_prefix, up_name, down_name)
 
     @property
@@ -200,8 +223,8 @@ class RoutedExperts(FeedForward):
             specs = {self.table_name: ParamSpec((self.vocab_size, self.top), role="int", init=f"choice:{self.num_experts}")}
         else:
             # a router of N(0, 0.02) would score all experts alike; a correction that matters is as large as the scores differ
-            specs = {r: ParamSpec((self.num_experts, E), init="normal:0.5"),
-                     c: ParamSpec((self.num_experts,), role="vector", init="normal:0.1")}
+            specs = {r: ParamSpec((self.choices, E), init="normal:0.5"),
+                     c: ParamSpec((self.choices,), role="vector", init="normal:0.1")}
         for e in range(self.num_experts):
             if self.gated:
                 specs[f"{p}{e}.{self.gate_name}"] = ParamSpec((F, E))
@@ -234,7 +257,7 @@ class RoutedExperts(FeedForward):
         if self.shared is not None:
             self.shared.bind({name: tensors[name] for name in self.shared.param_specs()}, rt)
 
-    def _run(self, ctx, h, out=None, accumulate=False, norm=None):
+    def _run(self, ctx, h, out=None, accumulate=False, norm=None, post_alpha=None):
         ops = self.rt.ops
         beside = None
         if self.routing == "table":
@@ -244,8 +267,10 @@ class RoutedExperts(FeedForward):
         else:       # the shared expert's rows enter the sum of the chosen ones with the token's gate
             idx, wts, gate = ops.moe_route(h, self.router, self.correction, self.top, side_gate=True, **self.how)
             beside = (self.shared.forward_f32(ctx, h), gate)
+        if post_alpha is not None and self.shared is not None and beside is None:      # all of it before the norm
+            beside = (self.shared.forward_f32(ctx, h), None)
         out = ops.moe_experts(h, self.w_up, self.w_down, idx, wts, out=out, accumulate=accumulate, activation=self.activation,
-                              param=self.activation_param, beside=beside, norm=norm)
+                              param=self.activation_param, beside=beside, norm=norm, identity=self.identity, post_alpha=post_alpha)
         if self.shared is not None and beside is None:
             self.shared.forward_add(ctx, h, out)
         return out
@@ -264,6 +289,13 @@ class RoutedExperts(FeedForward):
         if fold is None or (self.shared is not None and self.shared_gate_name is None):      # (a shared expert without a gate adds to the rows afterwards)
             return super().forward_add_norm(ctx, h, residual, norm, defer)
         return self._run(ctx, h, out=residual, accumulate=True, norm=fold)
+
+
+    def forward_post(self, ctx, h, x, alpha, norm):
+        w, eps = norm.fold()
+        if w.dtype != torch.float32:
+            return super().forward_post(ctx, h, x, alpha, norm)
+        return self._run(ctx, h, out=x, norm=(w, eps, False), post_alpha=alpha)
 
 
 register_feed_forward("gated_mlp", GatedMLP)

@@ -1,7 +1,8 @@
 """Norms of the residual stream, in 32-bit.
 
 RMSNorm: ``y = x / sqrt(mean(x^2) + eps) * w``
-(src/model.c:3386-3392; kernel src/kernels.cu:32-48).
+(src/model.c:3386-3392; kernel src/kernels.cu:32-48); with ``weight_offset`` c the stored weight counts as ``c + w``
+(c = 1: a weight stored around zero), summed once in 32 bits.
 LayerNorm: ``y = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * w``, a weight and no bias.
 DynamicTanh: ``y = tanh(alpha x) * w + b`` with one learned number ``alpha``: no mean and no variance,
 so every element stands alone and a block may fold it into whatever pass touches the rows anyway.
@@ -16,19 +17,23 @@ from .base import Norm, ParamSpec, register_norm
 
 
 class RMSNorm(Norm):
-    def __init__(self, size: int, eps: float, weight_name: str = "weight", has_weight: bool = True, optional: bool = False):
-        self.size, self.eps = int(size), float(eps)
+    def __init__(self, size: int, eps: float, weight_name: str = "weight", has_weight: bool = True, optional: bool = False,
+                 weight_offset: float = 0.0):
+        self.size, self.eps, self.weight_offset = int(size), float(eps), float(weight_offset)
         self.weight_name, self.has_weight, self.optional = weight_name, has_weight, bool(optional)
         self.weight: Optional[torch.Tensor] = None
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         if not self.has_weight:
             return {}
-        return {self.weight_name: ParamSpec((self.size,), role="vector", init="ones_jitter", optional=self.optional)}
+        init = "ones_jitter" if self.weight_offset == 0.0 else f"around:{1.0 - self.weight_offset}:0.1"
+        return {self.weight_name: ParamSpec((self.size,), role="vector", init=init, optional=self.optional)}
 
     def bind(self, tensors, rt) -> None:
         self.rt = rt
         self.weight = tensors.get(self.weight_name)
+        if self.weight is not None and self.weight_offset != 0.0:
+            self.weight = (self.weight.float() + self.weight_offset).contiguous()
 
     def forward(self, ctx, x, rows=None):
         return self.rt.ops.rmsnorm(x, self.weight, self.eps, self.rt.dtype, rows=rows)

@@ -36,6 +36,12 @@ Every head's read-out is divided by its root mean square, times a weight a chann
 ``silu(Wg h_g)``, then ``Wo``.  The width of ``W1``/``W2``'s inner side is no constant of a configuration:
 the stored tensors decide it.
 
+``StateSpace``: a selective state space with one decay a head ("Mamba-2", state-space duality).  ``W_in h`` is ``[z | x | B | C |
+dt]``: a gate and the inputs (H heads of Dv), what writes the state and what reads it (G groups of N, head h uses group
+``h // (H / G)``), and a step size a head.  x, B and C together pass a short causal convolution with a bias and SiLU;
+``dt = softplus(dt + dt_bias)``; per head ``S <- exp(-exp(A_log) dt) S + dt B x^T`` (S is N x Dv), ``y = S^T C + D x``.
+``y silu(z)`` over its root mean square, in ``norm_groups`` equal parts of the row, times a weight a channel, then ``Wo``.
+
 All keep their projections in 32 bits from the product to the recurrence: what enters a
 recurrence is not rounded on the way.
 """
@@ -430,7 +436,90 @@ class TimeMixWKV(Mixer):
         self.rt.ops.linear(self._read_out(ctx, cache, h), self.w_out, out=residual, accumulate=True)
 
 
+class StateSpace(Mixer):
+    joint = True
+
+    def __init__(self, hidden_size: int, num_heads: int, v_head_dim: int, state_size: int, groups: int, conv_taps: int, eps: float,
+                 norm_groups: int = 1, in_name: str = "in", conv_name: str = "conv", conv_bias_name: str = "conv.b",
+                 dt_bias_name: str = "dt_bias", a_log_name: str = "A_log", d_name: str = "D", norm_name: str = "norm",
+                 o_name: str = "o"):
+        _check_sizes("state space", num_heads, groups, state_size, v_head_dim)
+        if not (1 <= int(conv_taps) <= 16):
+            raise ValueError(f"state space: {conv_taps} convolution taps (1 to 16)")
+        self.hidden_size, self.num_heads, self.v_head_dim = int(hidden_size), int(num_heads), int(v_head_dim)
+        self.state_size, self.groups, self.conv_taps = int(state_size), int(groups), int(conv_taps)
+        self.norm_groups, self.eps = int(norm_groups), float(eps)
+        self.inner, self.bc = self.num_heads * self.v_head_dim, self.groups * self.state_size
+        self.conv_size = self.inner + 2 * self.bc
+        if self.norm_groups < 1 or self.inner % self.norm_groups:
+            raise ValueError(f"state space: {self.inner} channels do not form {norm_groups} equal parts")
+        self.names = dict(w_in=in_name, conv=conv_name, conv_b=conv_bias_name, dt_bias=dt_bias_name, a_log=a_log_name, d=d_name,
+                          norm=norm_name, o=o_name)
+
+    def state_spec(self):
+        from ..csrc.ops import Ops
+        out = {"S": StateSpec(Ops.recurrence_state_shape(self.num_heads, self.state_size, self.v_head_dim), torch.float32)}
+        if self.conv_taps > 1:
+            out["conv"] = StateSpec((self.conv_taps - 1, self.conv_size), torch.float32)
+        return out
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        E, H, n = self.hidden_size, self.num_heads, self.names
+        return {n["w_in"]: ParamSpec((self.inner + self.conv_size + H, E)),
+                n["conv"]: ParamSpec((self.conv_size, self.conv_taps), role="vector", init="normal:0.6"),
+                n["conv_b"]: ParamSpec((self.conv_size,), role="vector", init="normal:0.2"),
+                # step sizes around a tenth and rates around one: a state that lasts some tens of tokens
+                n["dt_bias"]: ParamSpec((H,), role="vector", init="around:-2.0:0.7"),
+                n["a_log"]: ParamSpec((H,), role="vector", init="normal:0.7"),
+                n["d"]: ParamSpec((H,), role="vector", init="around:0.8:0.4"),
+                n["norm"]: ParamSpec((self.inner,), role="vector", init="ones_jitter"), n["o"]: ParamSpec((E, self.inner))}
+
+    def joint_inputs(self, tensors):
+        return tensors[self.names["w_in"]].contiguous(), None
+
+    def joint_outputs(self, tensors):
+        return tensors[self.names["o"]], None
+
+    def joint_bind(self, tensors, rt) -> None:
+        self.rt = rt
+        n = self.names
+        self.w_conv, self.b_conv = tensors[n["conv"]].float().contiguous(), tensors[n["conv_b"]].float().contiguous()
+        self.constants = torch.stack([torch.exp(tensors[n["a_log"]].float()), tensors[n["dt_bias"]].float(),
+                                      tensors[n["d"]].float()]).contiguous()
+        self.w_norm = tensors[n["norm"]].float().contiguous()
+
+    def bind(self, tensors, rt) -> None:
+        self.joint_bind(tensors, rt)
+        self.w_in = rt.ops.pack_weight(self.joint_inputs(tensors)[0])
+        self.w_out = rt.ops.pack_weight(self.joint_outputs(tensors)[0])
+
+    def joint_read_out(self, ctx, cache, proj, out, scale: float):
+        """What ``Wo`` reads, times ``scale``, from the rows ``[z | x | B | C | dt]`` of the input product (into ``out``,
+        if it is given)."""
+        ops = self.rt.ops
+        H, G, N, Dv, I, BC = self.num_heads, self.groups, self.state_size, self.v_head_dim, self.inner, self.bc
+        y = ops.causal_conv(proj[:, I:I + self.conv_size], self.w_conv, cache.states.get("mixer.conv"), ctx, torch.float32,
+                            activation="silu", bias=self.b_conv)
+        o = ops.linear_recurrence("ssd", y[:, I + BC:], y[:, I:I + BC], y[:, :I], cache.states["mixer.S"], ctx, H, G, N, Dv,
+                                  gate=proj[:, I + self.conv_size:], decay=self.constants)
+        return ops.gated_rmsnorm(o, proj[:, :I], self.w_norm, self.norm_groups, I // self.norm_groups, self.eps, self.rt.dtype,
+                                 gate_first=True, out_scale=scale, out=out)
+
+    def _read_out(self, ctx, cache, h):
+        return self.joint_read_out(ctx, cache, self.rt.ops.linear(h, self.w_in, out_dtype=torch.float32), None, 1.0)
+
+    def forward(self, ctx, cache, h):
+        return self.rt.ops.linear(self._read_out(ctx, cache, h), self.w_out)
+
+    def forward_f32(self, ctx, cache, h):
+        return self.rt.ops.linear(self._read_out(ctx, cache, h), self.w_out, out_dtype=torch.float32)
+
+    def forward_add(self, ctx, cache, h, residual) -> None:
+        self.rt.ops.linear(self._read_out(ctx, cache, h), self.w_out, out=residual, accumulate=True)
+
+
 register_mixer("retention", Retention)
+register_mixer("state_space", StateSpace)
 register_mixer("wkv_time_mix", TimeMixWKV)
 register_mixer("gated_delta", GatedDelta)
 register_mixer("gated_linear_attention", GatedLinearAttention)
