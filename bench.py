@@ -393,8 +393,31 @@ def girolorn_config(width, layers, vocab=32000):
             "layers": [dict(layer) for _ in range(layers - again)] + [dict(layer, weights_of=i) for i in range(again)]}
 
 
+def pevolorn_config(width, layers, vocab=32000):
+    """A Pevolorn model of real layer sizes: of every four layers latent attention with a cached row of 192 + 64 channels
+    (128 unrotated and 64 rotated query channels a head, values of 128), such a layer that reads the rows of the one before,
+    and two of soft-capped attention (heads of 128, four query heads a key/value head, half the head rotated) beside a state
+    space of twice the width (heads of 64, states of 128, 8 groups, four taps); every layer with 14 experts of width / 2 and
+    2 identity experts (2 a token, from 2 of 4 groups) and a shared expert of the model's width."""
+    H = width // 128
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "router": {"experts": 14, "identity": 2, "top": 2, "groups": {"count": 4, "keep": 2}},
+           "shared": {"ff": width}}
+    latent = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "scale": 192 ** -0.5, "rot": {"base": 1e4, "dims": 64}}
+    both = {"left": {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 50.0,
+                     "rot": {"base": 1e5, "dims": 64}},
+            "right": {"heads": width // 32, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8},
+            "left_scale": 0.7, "right_scale": 0.7}
+    out = []
+    for i in range(layers):
+        k = i % 4
+        mixer = latent if k == 0 else dict(latent, kv_from=i - 1) if k == 1 else both
+        out.append({"type": "latent_attention" if k < 2 else "parallel", "mixer": mixer, "mlp": moe})
+    return {"architecture": "Pevolorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "postln_alpha": 2.0, "layers": out}
+
+
 DESIGNS = {"suripel": ("Suripel", suripel_config), "sugosun": ("Sugosun", sugosun_config), "dinasun": ("Dinasun", dinasun_config),
-           "kegorax": ("Kegorax", kegorax_config), "girolorn": ("Girolorn", girolorn_config)}
+           "kegorax": ("Kegorax", kegorax_config), "girolorn": ("Girolorn", girolorn_config),
+           "pevolorn": ("Pevolorn", pevolorn_config)}
 
 
 def llama_like(width, layers, vocab=32000):
@@ -497,7 +520,7 @@ def main():
                     help="also write the command and the JSON line into FILE (markdown)")
     ap.add_argument("--mixed", type=int, default=0, metavar="N",
                     help="also run N requests with prompts of 128..2048 tokens and 128 decoded tokens each through the scheduler")
-    ap.add_argument("--design", default="", choices=["", "suripel", "sugosun", "dinasun", "kegorax", "girolorn"],
+    ap.add_argument("--design", default="", choices=["", *DESIGNS],
                     help="instead of the serving benchmark: this design at real layer sizes beside the Llama decoder of equal size")
     ap.add_argument("--design-sizes", default="2048,4096", metavar="LIST", help="widths of the --design models")
     ap.add_argument("--design-layers", type=int, default=12, help="layers of the --design models")

@@ -1077,10 +1077,14 @@ __global__ __launch_bounds__(256) void k_attn_merge(MergeArgs a) {
     const int G = a.H / a.Hk;
     const int q0 = job[5], q_len = job[6];          // (with the job: one dependent read less before the partial results)
     const int n_rows = (q_len * G - row0) < ROWS ? (q_len * G - row0) : ROWS;      // rows of this block that exist
-    for (int idx = threadIdx.x; idx < n_rows * (HV / 4); idx += 256) {
+    // (the third axis deals the block's outputs to workgroups: one workgroup that took the 16 heads of a lone latent row one
+    // after another waited out three rounds of loads)
+    const int idx = (int)blockIdx.z * 256 + threadIdx.x;
+    if (idx < n_rows * (HV / 4)) {
         const int r = idx / (HV / 4), d4 = (idx % (HV / 4)) * 4;
         const int rho = row0 + r;
         const int tok = rho / G, hg = rho - tok * G;
+        const float factor = row_factor(a.gate, a.ld_gate, a.out_scale, q0 + tok, kvh * G + hg);
         const float* ml = a.part_ml + (((size_t)s0 * a.Hk + kvh) * ROWS + r) * 2;
         const float* po = a.part_o + (((size_t)s0 * a.Hk + kvh) * ROWS + r) * HV + d4;
         const size_t ml_step = (size_t)stride * a.Hk * ROWS * 2, po_step = (size_t)stride * a.Hk * ROWS * HV;
@@ -1116,7 +1120,7 @@ __global__ __launch_bounds__(256) void k_attn_merge(MergeArgs a) {
             }
         }
         wsum = with_sink(a.sinks, kvh * G + hg, mx, wsum);
-        const float inv = (wsum > 0.f ? 1.0f / wsum : 0.f) * row_factor(a.gate, a.ld_gate, a.out_scale, q0 + tok, kvh * G + hg);
+        const float inv = (wsum > 0.f ? 1.0f / wsum : 0.f) * factor;
         bf16_t* op = a.out + (size_t)(q0 + tok) * a.ld_out + (kvh * G + hg) * HV + d4;
         *reinterpret_cast<uint2*>(op) = make_uint2(pack2(acc.x * inv, acc.y * inv), pack2(acc.z * inv, acc.w * inv));
     }
@@ -1151,7 +1155,7 @@ static int launch_mode(const AttnArgs& a, const int* jobs, int n_jobs, const int
         mg.jobs = jobs; mg.cu_q = cu_q; mg.part_o = a.part_o; mg.part_ml = a.part_ml; mg.out = a.out;
         mg.H = a.H; mg.Hk = a.Hk; mg.sinks = a.sinks;
         mg.gate = a.gate; mg.ld_gate = a.ld_gate; mg.out_scale = a.out_scale; mg.ld_out = a.ld_out;
-        k_attn_merge<<<dim3(n_jobs, a.Hk), 256, 0, stream>>>(mg);
+        k_attn_merge<<<dim3(n_jobs, a.Hk, (ROWS * (HV / 4) + 255) / 256), 256, 0, stream>>>(mg);
         XR_CHECK_LAUNCH("attention_merge");
     }
     return XR_OK;

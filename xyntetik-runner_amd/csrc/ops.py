@@ -70,6 +70,7 @@ _PROTOS = {
     "xr_rope_table": [_p, _p, _p, _i, _i, _f, _p],
     "xr_attention_ref": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p, _p, _f, _p, _i, _f, _i, _p],
     "xr_head_norm_rope_write": [_p, _p, _p, _i, _p, _p, _f, _i, _p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p],
+    "xr_ssd_chunks": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p],
     "xr_post_norm": [_p, _p, _p, _p, _i, _i, _i, _f, _f, _i, _p],
     "xr_attn_extra_partial": [_p, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _i, _f, _i, _i, _i, _p, _p, _f, _i, _p],
     "xr_softcap": [_p, _i, _i, _i, _f, _p],
@@ -1509,6 +1510,59 @@ class Ops:
                                                      chunk_len, n_chunks, _ptr(scratch), _ptr(prod), 1 if activation else 0,
                                                      float(q_scale), float(k_scale), _stream()))
         return out
+
+    SSD_CHUNKED_FROM = 64            # the longest portion of a step from which a state space runs in chunks on the matrix cores
+
+    def ssd_in_chunks(self, dtype: torch.dtype, ctx, N: int, Dv: int) -> bool:
+        """Whether ``ssd_chunks`` takes a step: bfloat16, sizes in eights, and a portion that is worth it."""
+        return (self.use_mfma and dtype == torch.bfloat16 and ctx.max_q_len >= self.SSD_CHUNKED_FROM and N % 8 == 0 and N <= 256
+                and Dv % 8 == 0)
+
+    def ssd_chunks(self, xbc: torch.Tensor, z: torch.Tensor, constants: torch.Tensor, state: torch.Tensor, ctx, H: int, G: int,
+                   N: int, Dv: int) -> torch.Tensor:
+        """``linear_recurrence("ssd")`` over long portions, in chunks on the matrix cores: the read-outs ``[T, H * Dv]`` (32-bit)
+        from and into the same ``state``.  ``xbc [T, H * Dv + 2 G * N]`` (bfloat16, contiguous): every row's values, what writes
+        the state and what reads it; ``z [T, H]`` and ``constants [3, H]`` as there."""
+        self._dev(xbc, z, constants, state)
+        T, W = xbc.shape
+        I, BC = H * Dv, G * N
+        if xbc.dtype != torch.bfloat16 or not xbc.is_contiguous() or W != I + 2 * BC or W % 8:
+            raise KernelError(f"ssd_chunks: the rows must be contiguous bfloat16 [T, {I + 2 * BC}] in multiples of 8")
+        if z.dtype != torch.float32 or tuple(z.shape) != (T, H) or z.stride(1) != 1:
+            raise KernelError(f"ssd_chunks: the step sizes must be a float32 view [T, {H}]")
+        if constants.dtype != torch.float32 or tuple(constants.shape) != (3, H) or not constants.is_contiguous():
+            raise KernelError(f"ssd_chunks: the constants must be float32 [3, {H}]")
+        shape = self.recurrence_state_shape(H, N, Dv)
+        if state.dtype != torch.float32 or tuple(state.shape[1:]) != shape or not state.is_contiguous():
+            raise KernelError(f"ssd_chunks: state must be float32 [slots, {shape}]")
+        items, requests, n_items = self._ssd_plan(ctx)
+        out = torch.empty((T, I), dtype=torch.float32, device=xbc.device)
+        scratch = torch.empty((n_items,) + shape, dtype=torch.float32, device=xbc.device)
+        prod = torch.empty((n_items, H), dtype=torch.float32, device=xbc.device)
+        self.lib.check(self.lib.xr_ssd_chunks(out.data_ptr(), xbc.data_ptr(), xbc[:, I:].data_ptr(), xbc[:, I + BC:].data_ptr(),
+                                              z.data_ptr(), constants.data_ptr(), state.data_ptr(), scratch.data_ptr(),
+                                              prod.data_ptr(), items.data_ptr(), n_items, requests.data_ptr(), ctx.slots.data_ptr(),
+                                              ctx.B, H, G, N, Dv, shape[3], xbc.stride(0), z.stride(0), _stream()))
+        return out
+
+    def _ssd_plan(self, ctx):
+        """(chunks ``[n, 4]``: request, first row, rows; requests ``[B, 2]``: first chunk, chunks; n), once a step."""
+        shared = getattr(ctx, "shared", None)
+        plan = shared.get("ssd_plan") if shared is not None else None
+        if plan is None:
+            L = int(self.lib.dll.xr_ssd_chunk_rows())
+            items, requests, row0 = [], [], 0
+            for b, n in enumerate(ctx.q_lens):
+                requests += [len(items), -(-n // L)]
+                items += [(b, row0 + i, min(L, n - i), 0) for i in range(0, n, L)]
+                row0 += n
+            flat = [v for it in items for v in it] + requests
+            host = torch.tensor(flat, dtype=torch.int32).pin_memory()
+            dev = host.to(ctx.device, non_blocking=True)
+            plan = (dev[:4 * len(items)], dev[4 * len(items):], len(items), host)      # (the pinned copy lives as long as the plan)
+            if shared is not None:
+                shared["ssd_plan"] = plan
+        return plan[:3]
 
     RETENTION_CHUNK = 256            # rows a chunk; a multiple of the kernel's 16 staged tokens
     RETENTION_CHUNKED_FROM = 1024    # the longest portion of a step from which chunks pay

@@ -177,6 +177,30 @@ __global__ __launch_bounds__(256) void k_causal_conv_rows(TO* __restrict__ out, 
 #pragma unroll
     for (int j = 0; j < CONV_MAX_TAPS; ++j) wt[j] = j < taps ? w[(size_t)c * taps + j] : 0.f;
     const float bc = bias ? bias[c] : 0.f;
+    if (taps <= 4 && t0 + CONV_ROWS <= T && row0[0] == row0[CONV_ROWS - 1]) {
+        // all rows of one request (the usual case): every input is read once, the rows share them in registers
+        const int i0 = t0 - row0[0];
+        const TU* srow = state + (size_t)slot[0] * (taps - 1) * C;
+        float v[CONV_ROWS + 3];
+#pragma unroll
+        for (int k = 0; k < CONV_ROWS + 3; ++k) {
+            const int s = i0 + k - 3;               // (taps below 4 leave the first of them unread)
+            v[k] = k < 4 - taps ? 0.f : s >= 0 ? ld<TU>(u, (size_t)(row0[0] + s) * ld_u + c) : ld<TU>(srow, (size_t)(taps - 1 + s) * C + c);
+        }
+#pragma unroll
+        for (int r = 0; r < CONV_ROWS; ++r) {
+            float acc = 0.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                if (j < taps) acc = fmaf(wt[j], taps == 4 ? v[r + j] : taps == 3 ? v[r + j + 1 < CONV_ROWS + 3 ? r + j + 1 : 0]
+                                                : taps == 2 ? v[r + j + 2 < CONV_ROWS + 3 ? r + j + 2 : 0] : v[r + 3], acc);
+            acc += bc;
+            if (residual) acc += v[r + 3];
+            if (act == XR_CONV_SILU) acc = acc / (1.0f + expf(-acc));
+            st<TO>(out, (size_t)(t0 + r) * ld_out + c, acc);
+        }
+        return;
+    }
 #pragma unroll
     for (int r = 0; r < CONV_ROWS; ++r) {
         const int t = t0 + r;
@@ -498,6 +522,44 @@ __global__ __launch_bounds__(256) void k_gated_rmsnorm_wide(TO* __restrict__ out
         st<TO>(dst, d, orow[d] * rinv * (wrow ? wrow[d] : 1.f) * norm_gate(grow[d], gate_act));
 }
 
+// Rows of up to 64 * 4 * NV channels that come in fours: a wave a (token, head) keeps its float4 pieces in registers from the
+// sum to the store, and every gate is made once.
+template <typename TO, int NV>
+__global__ __launch_bounds__(256) void k_gated_rmsnorm_v4(TO* __restrict__ out, const float* __restrict__ o,
+                                                         const float* __restrict__ gate, const float* __restrict__ w,
+                                                         int TH, int H, int Dv, int ld_g, float eps, int w_full, int gate_act,
+                                                         int gate_first, float scale, int ld_out) {
+    const int th = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (th >= TH) return;
+    const int t = th / H, h = th - t * H, n4 = Dv >> 2;
+    const float4* o4 = reinterpret_cast<const float4*>(o + (size_t)th * Dv);
+    const float4* g4 = reinterpret_cast<const float4*>(gate + (size_t)t * ld_g + (size_t)h * Dv);
+    const float4* w4 = reinterpret_cast<const float4*>(w ? (w_full ? w + (size_t)h * Dv : w) : nullptr);
+    float4 u[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = lane + 64 * i;
+        u[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (c >= n4) continue;
+        const float4 x = o4[c], g = g4[c];
+        u[i] = make_float4(x.x * norm_gate(g.x, gate_act), x.y * norm_gate(g.y, gate_act), x.z * norm_gate(g.z, gate_act), x.w * norm_gate(g.w, gate_act));
+        const float4 y = gate_first ? u[i] : x;
+        ss += y.x * y.x + y.y * y.y + y.z * y.z + y.w * y.w;
+    }
+    const float f = scale / sqrtf(wave_sum(ss) / (float)Dv + eps);
+    TO* dst = out + (size_t)t * ld_out + (size_t)h * Dv;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = lane + 64 * i;
+        if (c >= n4) continue;
+        const float4 g = w ? w4[c] : make_float4(1.f, 1.f, 1.f, 1.f);
+        const float4 y = make_float4(u[i].x * f * g.x, u[i].y * f * g.y, u[i].z * f * g.z, u[i].w * f * g.w);
+        if constexpr (sizeof(TO) == 4) *reinterpret_cast<float4*>((float*)dst + 4 * c) = y;
+        else *reinterpret_cast<uint2*>((bf16_t*)dst + 4 * c) = make_uint2(pack_bf16x2(y.x, y.y), pack_bf16x2(y.z, y.w));
+    }
+}
+
 extern "C" int xr_gated_rmsnorm(void* out, const float* o, const float* gate, const float* w, int T, int H, int Dv,
                                 int ld_g, float eps, int out_dtype, int w_full, int gate_act, int gate_first, float scale,
                                 int ld_out, hipStream_t stream) {
@@ -505,6 +567,18 @@ extern "C" int xr_gated_rmsnorm(void* out, const float* o, const float* gate, co
     XR_REQUIRE(T >= 0 && H > 0 && Dv > 0 && ld_g >= H * Dv, "gated_rmsnorm: bad sizes T=%d H=%d Dv=%d ld=%d", T, H, Dv, ld_g);
     XR_REQUIRE(gate_act == XR_GATE_SILU || gate_act == XR_GATE_SIGMOID, "gated_rmsnorm: unknown gate activation %d", gate_act);
     if (T == 0) return XR_OK;
+    // (bfloat16 only: results in 32 bits keep the order of sums they had)
+    const bool v4 = out_dtype == XR_BF16 && Dv % 4 == 0 && Dv >= 128 && Dv <= 1024 && ld_g % 4 == 0 && ld_out % 4 == 0 && ((uintptr_t)out % 8) == 0 &&
+                    ((uintptr_t)o % 16) == 0 && ((uintptr_t)gate % 16) == 0 && ((uintptr_t)w % 16) == 0;
+    if (v4) {
+        const int TH = T * H, blocks = (TH + 3) / 4;
+        bf16_t* ob = (bf16_t*)out;
+        if (Dv <= 256) k_gated_rmsnorm_v4<bf16_t, 1><<<blocks, 256, 0, stream>>>(ob, o, gate, w, TH, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
+        else if (Dv <= 512) k_gated_rmsnorm_v4<bf16_t, 2><<<blocks, 256, 0, stream>>>(ob, o, gate, w, TH, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
+        else k_gated_rmsnorm_v4<bf16_t, 4><<<blocks, 256, 0, stream>>>(ob, o, gate, w, TH, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
+        XR_CHECK_LAUNCH("gated_rmsnorm");
+        return XR_OK;
+    }
     const bool wide = Dv > 256;       // (the sums' order differs between the two kernels, not between calls of one size)
     if (out_dtype == XR_F32 && wide) k_gated_rmsnorm_wide<float><<<dim3(T, H), 256, 0, stream>>>((float*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);
     else if (out_dtype == XR_BF16 && wide) k_gated_rmsnorm_wide<bf16_t><<<dim3(T, H), 256, 0, stream>>>((bf16_t*)out, o, gate, w, H, Dv, ld_g, eps, w_full, gate_act, gate_first, scale, ld_out);

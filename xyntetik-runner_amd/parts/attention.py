@@ -24,9 +24,9 @@ tensor ``sink_name``, unscaled) or "zero" (the score 0: one is added to the deno
 projection ``[H, E]`` of the mixer's input whose sigmoid multiplies every head's output before the output
 projection; ``softcap`` c > 0: every scaled score s becomes ``c tanh(s / c)`` (before a slope's bias and not the sink).
 
-Where values have another size than keys, or a head norm comes behind the rotation, one kernel takes the input product's
-32-bit rows through norm and rotation to the queries and the cache, and the gate's rows are part of that product.  Such an
-attention may also be a side of a joint pair of mixers (``parts/parallel.py``): its input rows and output columns are then
+Where a head norm comes behind the rotation, one kernel takes the input product's 32-bit rows through rotation and norm to
+the queries and the cache, and the gate's rows are part of that product.  An attention that this kernel serves (any size of
+values, a norm a head on either side of the rotation or none) may also be a side of a joint pair of mixers (``parts/parallel.py``): its input rows and output columns are then
 part of the pair's two products (``joint_*``).
 """
 from __future__ import annotations
@@ -107,7 +107,7 @@ class PagedAttention(Mixer):
         late = bool(getattr(self.qk_transform, "after_rotation", False))
         if late and not self.head_kernel:
             raise ValueError("attention: a norm behind the rotation needs a rotation by a table and both sides normed, without a temperature")
-        self.by_head = self.head_kernel and (late or self.v_head_dim != self.head_dim)
+        self.by_head = late
         self.q_size = self.num_heads * self.head_dim
         self.kv_size = self.num_kv_heads * self.head_dim
         self.v_size = self.num_kv_heads * self.v_head_dim

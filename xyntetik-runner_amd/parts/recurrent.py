@@ -498,10 +498,15 @@ class StateSpace(Mixer):
         if it is given)."""
         ops = self.rt.ops
         H, G, N, Dv, I, BC = self.num_heads, self.groups, self.state_size, self.v_head_dim, self.inner, self.bc
-        y = ops.causal_conv(proj[:, I:I + self.conv_size], self.w_conv, cache.states.get("mixer.conv"), ctx, torch.float32,
-                            activation="silu", bias=self.b_conv)
-        o = ops.linear_recurrence("ssd", y[:, I + BC:], y[:, I:I + BC], y[:, :I], cache.states["mixer.S"], ctx, H, G, N, Dv,
-                                  gate=proj[:, I + self.conv_size:], decay=self.constants)
+        # a long portion runs in chunks on the matrix cores, which take what the convolution leaves in bfloat16
+        chunks = ops.ssd_in_chunks(self.rt.dtype, ctx, N, Dv)
+        y = ops.causal_conv(proj[:, I:I + self.conv_size], self.w_conv, cache.states.get("mixer.conv"), ctx,
+                            torch.bfloat16 if chunks else torch.float32, activation="silu", bias=self.b_conv)
+        if chunks:
+            o = ops.ssd_chunks(y, proj[:, I + self.conv_size:], self.constants, cache.states["mixer.S"], ctx, H, G, N, Dv)
+        else:
+            o = ops.linear_recurrence("ssd", y[:, I + BC:], y[:, I:I + BC], y[:, :I], cache.states["mixer.S"], ctx, H, G, N, Dv,
+                                      gate=proj[:, I + self.conv_size:], decay=self.constants)
         return ops.gated_rmsnorm(o, proj[:, :I], self.w_norm, self.norm_groups, I // self.norm_groups, self.eps, self.rt.dtype,
                                  gate_first=True, out_scale=scale, out=out)
 
