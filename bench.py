@@ -403,7 +403,7 @@ def pevolorn_config(width, layers, vocab=32000):
     moe = {"kind": "moe", "expert": {"ff": width // 2}, "router": {"experts": 14, "identity": 2, "top": 2, "groups": {"count": 4, "keep": 2}},
            "shared": {"ff": width}}
     latent = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "scale": 192 ** -0.5, "rot": {"base": 1e4, "dims": 64}}
-    both = {"left": {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 50.0,
+    both = {"left": {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 40.0,
                      "rot": {"base": 1e5, "dims": 64}},
             "right": {"heads": width // 32, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8},
             "left_scale": 0.7, "right_scale": 0.7}

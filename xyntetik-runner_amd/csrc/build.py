@@ -187,8 +187,8 @@ def build_unit(unit: str, force: bool = False, jobs: int = 8) -> str:
     return lib
 
 
-def default_units(head_dims: Sequence[int] = (16, 32, 64, 128)) -> List[str]:
-    return ["kernels"] + [f"attn_d{d}" for d in head_dims]
+def default_units(head_dims: Sequence[int] = (16, 32, 64, 128), key_value_dims: Sequence[tuple] = ()) -> List[str]:
+    return ["kernels"] + [f"attn_d{d}" for d in head_dims] + [f"attn_d{d}v{v}" for d, v in key_value_dims]
 
 
 if __name__ == "__main__":
