@@ -471,6 +471,27 @@ def test_experts_of_which_some_are_the_identity(ops, dt, T, n, ident, top, E, F)
     close(out.float().cpu().numpy(), normed, ntol, "and its copy")
 
 
+@pytest.mark.parametrize("dt", ["float32", "bfloat16"])
+@pytest.mark.parametrize("T", [1, 2])
+@pytest.mark.parametrize("n,ident,top,E,F,Fs", [(6, 2, 2, 64, 24, 40), (3, 1, 4, 256, 512, 136), (2, 1, 1, 48, 10, 21), (2, 0, 2, 30, 9, 6), (4, 0, 1, 72, 16, 8)])
+def test_a_shared_expert_in_the_chosen_experts_launches(ops, dt, T, n, ident, top, E, F, Fs):
+    """A shared expert wider and narrower than the others, from packed matrices and from plain ones."""
+    rng = np.random.default_rng(T + E + Fs)
+    h = dev(rng.normal(size=(T, E)), DT[dt])
+    mats = [dev(rng.normal(size=s) / math.sqrt(s[-1]), DT[dt]) for s in ((n, F, E), (n, E, F), (Fs, E), (E, Fs))]
+    idx = np.stack([rng.permutation(n + ident)[:top] for _ in range(T)])
+    wts = rng.uniform(0.1, 1.0, size=(T, top))
+    hd, ud, dd, su, sd = (t.double().cpu().numpy() for t in [h] + mats)
+    want = P.relu2(hd @ su.T) @ sd.T
+    for t in range(T):
+        for e, a in zip(idx[t], wts[t]):
+            want[t] += a * (hd[t] if e >= n else P.relu2(ud[e] @ hd[t]) @ dd[e].T)
+    packed = [ops.pack_weight(m) for m in mats[2:]]
+    for shared in (mats[2:], packed) if type(packed[0]) is type(packed[1]) else (mats[2:],):
+        got = ops.moe_experts(h, mats[0], mats[1], dev(idx, torch.int32), dev(wts), identity=ident, shared=tuple(shared))
+        close(got.cpu().numpy(), want, 1e-5 if dt == "float32" else 1e-2, "sum")
+
+
 # ----------------------------------------------------------------------------- a model with made weights
 def needle_model():
     """Three layers without feed-forwards: latent attention, latent attention over the first layer's rows, and the pair whose

@@ -15,14 +15,15 @@
 // follows.  Without kv_in (a layer that reads another layer's rows) only the queries are made.  A workgroup a token.
 #include "common.h"
 
-template <typename TO>
-__global__ __launch_bounds__(256) void k_latent_prepare(
+template <typename TO, int NW>
+__global__ __launch_bounds__(64 * NW) void k_latent_prepare(
     TO* __restrict__ qn_out, TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __restrict__ v_cache,
     const float* __restrict__ q_in, const float* __restrict__ kv_in, const float* __restrict__ c_w,
     const int* __restrict__ positions, const int* __restrict__ req_of_token, const int* __restrict__ block_table,
     const float* __restrict__ inv_freq, int table_stride, int H, int D, int R, int C, int Dvc, int dims, int halves, int ld_q, int ld_kv,
     int page_shift, int page_size, float eps) {
-    __shared__ float part[4];
+    constexpr int NT = 64 * NW;
+    __shared__ float part[NW];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int pos = positions[t];
     const float* kv = kv_in + (kv_in ? (size_t)t * ld_kv : 0);
@@ -31,15 +32,18 @@ __global__ __launch_bounds__(256) void k_latent_prepare(
     if (kv_in) {
         // the latent's norm
         float ss = 0.f;
-        for (int i = tid; i < C; i += 256) ss += kv[i] * kv[i];
+        for (int i = tid; i < C; i += NT) ss += kv[i] * kv[i];
         ss = wave_sum(ss);
         if ((tid & 63) == 0) part[tid >> 6] = ss;
         __syncthreads();
-        const float rinv = 1.0f / sqrtf(((part[0] + part[1]) + (part[2] + part[3])) / (float)C + eps);
+        float tot = 0.f;
+#pragma unroll
+        for (int i = 0; i < NW; ++i) tot += part[i];
+        const float rinv = 1.0f / sqrtf(tot / (float)C + eps);
         const PageRef pr = page_of(block_table, table_stride, req_of_token[t], pos, page_shift, page_size - 1);
         krow = k_cache + ((size_t)pr.page * page_size + pr.off) * DK;
         vpage = v_cache + (size_t)pr.page * Dvc * page_size + pr.off;
-        for (int i = tid; i < C; i += 256) {
+        for (int i = tid; i < C; i += NT) {
             const float c = kv[i] * rinv * c_w[i];
             st<TO>(krow, i, c);
             st<TO>(vpage, (size_t)i * page_size, c);
@@ -47,7 +51,7 @@ __global__ __launch_bounds__(256) void k_latent_prepare(
     }
     // the shared key part and every head's rotated query channels: unit u = 0 is the key, u = 1 + h head h
     const int half = dims >> 1, pairs_r = (R + 1) >> 1;       // a "pair" past `dims` is two channels that pass unchanged
-    for (int w = tid + (kv_in ? 0 : pairs_r); w < (H + 1) * pairs_r; w += 256) {
+    for (int w = tid + (kv_in ? 0 : pairs_r); w < (H + 1) * pairs_r; w += NT) {
         const int u = w / pairs_r, i = w - u * pairs_r;
         const float* src = u == 0 ? kv + C : q_in + (size_t)t * ld_q + (size_t)(u - 1) * (D + R) + D;
         const int c0 = halves && i < half ? i : 2 * i, c1 = halves && i < half ? i + half : 2 * i + 1;
@@ -73,7 +77,7 @@ __global__ __launch_bounds__(256) void k_latent_prepare(
         }
     }
     // the unrotated query channels, head by head, for the product into the latent's space
-    for (int w = tid; w < H * D; w += 256) {
+    for (int w = tid; w < H * D; w += NT) {
         const int h = w / D, d = w - h * D;
         st<TO>(qn_out, (size_t)t * H * D + w, q_in[(size_t)t * ld_q + (size_t)h * (D + R) + d]);
     }
@@ -90,15 +94,16 @@ extern "C" int xr_latent_prepare(void* qn_out, void* q_out, void* k_cache, void*
     const int shift = ilog2_exact(page_size);
     XR_REQUIRE(shift >= 0, "latent_prepare: page size %d is no power of two", page_size);
     if (T == 0) return XR_OK;
-    if (dtype == XR_F32)
-        k_latent_prepare<float><<<T, 256, 0, stream>>>((float*)qn_out, (float*)q_out, (float*)k_cache, (float*)v_cache, q_in, kv_in, c_w,
-                                                       positions, req_of_token, block_table, inv_freq, table_stride, H, D, R, C, Dvc,
-                                                       dims, halves, ld_q, ld_kv, shift, page_size, eps);
-    else if (dtype == XR_BF16)
-        k_latent_prepare<bf16_t><<<T, 256, 0, stream>>>((bf16_t*)qn_out, (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, q_in, kv_in,
-                                                        c_w, positions, req_of_token, block_table, inv_freq, table_stride, H, D, R, C,
-                                                        Dvc, dims, halves, ld_q, ld_kv, shift, page_size, eps);
+#define LP(TO, NW)                                                                                                            \
+    k_latent_prepare<TO, NW><<<T, 64 * NW, 0, stream>>>((TO*)qn_out, (TO*)q_out, (TO*)k_cache, (TO*)v_cache, q_in, kv_in, c_w,  \
+                                                        positions, req_of_token, block_table, inv_freq, table_stride, H, D, R, \
+                                                        C, Dvc, dims, halves, ld_q, ld_kv, shift, page_size, eps)
+    // (a decode step's few rows: their time is the latency of one workgroup's passes)
+    const bool few = T <= 128 && H * (D + R) >= 1024;
+    if (dtype == XR_F32) { if (few) LP(float, 16); else LP(float, 4); }
+    else if (dtype == XR_BF16) { if (few) LP(bf16_t, 16); else LP(bf16_t, 4); }
     else { xr_set_error("latent_prepare: bad dtype %d", dtype); return XR_BAD_ARG; }
+#undef LP
     XR_CHECK_LAUNCH("latent_prepare");
     return XR_OK;
 }

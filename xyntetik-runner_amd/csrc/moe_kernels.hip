@@ -224,6 +224,37 @@ template <> __device__ inline float wave_dot<bf16_t>(const bf16_t* __restrict__ 
     return wave_sum(acc);
 }
 
+// A wave's dot product of row `row` of a packed bfloat16 matrix (blocks of 16 rows x 32 columns, see k_pack_weight) with x:
+// the four waves of a workgroup take neighbouring rows, which lie side by side in a block.
+__device__ inline float wave_dot_packed(const bf16_t* __restrict__ w, int row, const bf16_t* __restrict__ x, int n, int lane) {
+    const bf16_t* wr = w + (size_t)(row >> 4) * ((n + 31) / 32) * 512 + (row & 15) * 32;
+    float acc = 0.f;
+    for (int i = lane * 8; i < n; i += 512) {       // (n is a multiple of 8)
+        const uint4 a = *reinterpret_cast<const uint4*>(wr + (size_t)(i >> 5) * 512 + (i & 31)), b = *reinterpret_cast<const uint4*>(x + i);
+        acc = fmaf(bf_lo(a.x), bf_lo(b.x), acc); acc = fmaf(bf_hi(a.x), bf_hi(b.x), acc);
+        acc = fmaf(bf_lo(a.y), bf_lo(b.y), acc); acc = fmaf(bf_hi(a.y), bf_hi(b.y), acc);
+        acc = fmaf(bf_lo(a.z), bf_lo(b.z), acc); acc = fmaf(bf_hi(a.z), bf_hi(b.z), acc);
+        acc = fmaf(bf_lo(a.w), bf_lo(b.w), acc); acc = fmaf(bf_hi(a.w), bf_hi(b.w), acc);
+    }
+    return wave_sum(acc);
+}
+template <typename TW> __device__ inline float shared_dot(const void* w, int row, const TW* x, int n, int lane, int packed, bool vec);
+template <> __device__ inline float shared_dot<float>(const void* w, int row, const float* x, int n, int lane, int, bool vec) {
+    return wave_dot<float>((const float*)w + (size_t)row * n, x, n, lane, vec);
+}
+template <> __device__ inline float shared_dot<bf16_t>(const void* w, int row, const bf16_t* x, int n, int lane, int packed, bool vec) {
+    return packed ? wave_dot_packed((const bf16_t*)w, row, x, n, lane) : wave_dot<bf16_t>((const bf16_t*)w + (size_t)row * n, x, n, lane, vec);
+}
+
+// A shared expert down(relu(up h)^2) that runs beside the chosen ones in the same two launches: for one or two tokens, each of
+// which streams its weights anew.
+struct MoeShared {
+    const void* up;         // [F, E], or packed; null: none
+    const void* down;       // [E, F], or packed
+    void* z;                // [T, F] between the products
+    int F, packed, vec_up, vec_down;
+};
+
 // z[t * top + j][f] = relu(W_up[e][f] . h[t])^2 for e = idx[t][j]; `gated`: the gate's value of W_up[e][f] . h[t] and W_up[e][F + f] . h[t].
 // Grid (T * top, ceil(F / 4)); a wave a column.
 #define MOE_ACT_RELU2 0
@@ -231,8 +262,14 @@ template <> __device__ inline float wave_dot<bf16_t>(const bf16_t* __restrict__ 
 template <typename TW>
 __global__ __launch_bounds__(256) void k_moe_up(TW* __restrict__ z, const TW* __restrict__ h, const TW* __restrict__ w_up,
                                                 const int* __restrict__ idx, int E, int F, int ld_h, int top, int n, int n_id, int vec,
-                                                int gated, int gate, float param) {
+                                                int gated, int gate, float param, int A, MoeShared sh) {
     const int a = blockIdx.x, f = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (a >= A) {                   // the shared expert of token a - A
+        if (f >= sh.F) return;
+        const float r = fmaxf(shared_dot<TW>(sh.up, f, h + (size_t)(a - A) * ld_h, E, lane, sh.packed, sh.vec_up != 0), 0.f);
+        if (lane == 0) st<TW>((TW*)sh.z, (size_t)(a - A) * sh.F + f, r * r);
+        return;
+    }
     if (f >= F) return;
     const int t = a / top, e = min(max(idx[a], 0), n + n_id - 1);
     if (e >= n) return;             // an identity expert: nothing to multiply
@@ -256,7 +293,7 @@ __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const T
                                                   const int* __restrict__ idx, const float* __restrict__ wts, int E, int F,
                                                   int ld_y, int top, int n, int n_id, int accumulate, int vec,
                                                   const float* __restrict__ y_side, const float* __restrict__ g_side,
-                                                  const TW* __restrict__ h, int ld_h) {
+                                                  const TW* __restrict__ h, int ld_h, MoeShared sh) {
     const int t = blockIdx.x, c = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (c >= E) return;
     float sum = 0.f;
@@ -270,6 +307,7 @@ __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const T
         const TW* zr = z + ((size_t)t * top + j) * F;
         sum += wts[(size_t)t * top + j] * wave_dot<TW>(w, zr, F, lane, vec != 0);
     }
+    if (sh.up) sum += shared_dot<TW>(sh.down, c, (const TW*)sh.z + (size_t)t * sh.F, sh.F, lane, sh.packed, sh.vec_down != 0);
     if (lane == 0) {
         if (y_side) sum = fmaf(g_side ? g_side[t] : 1.f, y_side[(size_t)t * E + c], sum);
         float* o = y + (size_t)t * ld_y + c;
@@ -280,6 +318,7 @@ __global__ __launch_bounds__(256) void k_moe_down(float* __restrict__ y, const T
 extern "C" int xr_moe_experts(float* y, void* z, const void* h, const void* w_up, const void* w_down, const int* idx,
                               const float* wts, int T, int E, int F, int ld_h, int ld_y, int n, int top, int accumulate,
                               int dtype, int act, int gate, float param, const float* y_side, const float* g_side, int n_id,
+                              const void* shared_up, const void* shared_down, void* shared_z, int shared_F, int shared_packed,
                               hipStream_t stream) {
     XR_REQUIRE(act == MOE_ACT_RELU2 || act == MOE_ACT_GATED, "moe_experts: activation %d (0 = relu squared, 1 = gated)", act);
     XR_REQUIRE(gate >= 0 && gate < XR_ACT_COUNT, "moe_experts: unknown gate %d", gate);
@@ -289,16 +328,23 @@ extern "C" int xr_moe_experts(float* y, void* z, const void* h, const void* w_up
     XR_REQUIRE(n >= 1 && n_id >= 0 && top >= 1 && top <= n + n_id && top <= MOE_MAX_TOP, "moe_experts: %d experts (and %d that are the identity), %d chosen", n, n_id, top);
     XR_REQUIRE((long long)T * top <= 0x7fffffffLL, "moe_experts: too many rows");
     if (T == 0) return XR_OK;
-    const dim3 gu(T * top, (F + 3) / 4), gd(T, (E + 3) / 4);
+    XR_REQUIRE(!shared_up || (shared_down && shared_z && shared_F > 0), "moe_experts: a shared expert of %d without its operands", shared_F);
+    XR_REQUIRE(!shared_up || !shared_packed || (dtype == XR_BF16 && E % 8 == 0 && shared_F % 8 == 0 && ld_h % 8 == 0 && ((uintptr_t)h % 16) == 0 &&
+               ((uintptr_t)shared_up % 16) == 0 && ((uintptr_t)shared_down % 16) == 0 && ((uintptr_t)shared_z % 16) == 0),
+               "moe_experts: packed shared weights take bfloat16 rows in eights (E %d, F %d)", E, shared_F);
+    const int A = T * top;
+    const dim3 gu(shared_up ? A + T : A, ((shared_up && shared_F > F ? shared_F : F) + 3) / 4), gd(T, (E + 3) / 4);
     const int per16 = dtype == XR_BF16 ? 8 : 4;             // elements in 16 bytes
     const bool al = ((uintptr_t)h % 16) == 0 && ((uintptr_t)w_up % 16) == 0 && ((uintptr_t)w_down % 16) == 0 && ((uintptr_t)z % 16) == 0;
+    const bool sal = ((uintptr_t)shared_up % 16) == 0 && ((uintptr_t)shared_down % 16) == 0 && ((uintptr_t)shared_z % 16) == 0;
+    const MoeShared sh{shared_up, shared_down, shared_z, shared_F, shared_packed, al && sal && E % per16 == 0 && ld_h % per16 == 0, sal && shared_F % per16 == 0};
     const int vu = al && E % per16 == 0 && ld_h % per16 == 0, vd = al && F % per16 == 0;
     if (dtype == XR_F32) {
-        k_moe_up<float><<<gu, 256, 0, stream>>>((float*)z, (const float*)h, (const float*)w_up, idx, E, F, ld_h, top, n, n_id, vu, gated, gate, param);
-        k_moe_down<float><<<gd, 256, 0, stream>>>(y, (const float*)z, (const float*)w_down, idx, wts, E, F, ld_y, top, n, n_id, accumulate, vd, y_side, g_side, (const float*)h, ld_h);
+        k_moe_up<float><<<gu, 256, 0, stream>>>((float*)z, (const float*)h, (const float*)w_up, idx, E, F, ld_h, top, n, n_id, vu, gated, gate, param, A, sh);
+        k_moe_down<float><<<gd, 256, 0, stream>>>(y, (const float*)z, (const float*)w_down, idx, wts, E, F, ld_y, top, n, n_id, accumulate, vd, y_side, g_side, (const float*)h, ld_h, sh);
     } else if (dtype == XR_BF16) {
-        k_moe_up<bf16_t><<<gu, 256, 0, stream>>>((bf16_t*)z, (const bf16_t*)h, (const bf16_t*)w_up, idx, E, F, ld_h, top, n, n_id, vu, gated, gate, param);
-        k_moe_down<bf16_t><<<gd, 256, 0, stream>>>(y, (const bf16_t*)z, (const bf16_t*)w_down, idx, wts, E, F, ld_y, top, n, n_id, accumulate, vd, y_side, g_side, (const bf16_t*)h, ld_h);
+        k_moe_up<bf16_t><<<gu, 256, 0, stream>>>((bf16_t*)z, (const bf16_t*)h, (const bf16_t*)w_up, idx, E, F, ld_h, top, n, n_id, vu, gated, gate, param, A, sh);
+        k_moe_down<bf16_t><<<gd, 256, 0, stream>>>(y, (const bf16_t*)z, (const bf16_t*)w_down, idx, wts, E, F, ld_y, top, n, n_id, accumulate, vd, y_side, g_side, (const bf16_t*)h, ld_h, sh);
     } else { xr_set_error("moe_experts: bad dtype %d", dtype); return XR_BAD_ARG; }
     XR_CHECK_LAUNCH("moe_experts");
     return XR_OK;

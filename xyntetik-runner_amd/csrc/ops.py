@@ -98,7 +98,7 @@ _PROTOS = {
     "xr_moe_route": [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p],
     "xr_moe_experts_grouped": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p, _i, _p],
     "xr_heads_gemm_bf16": [_p, _p, _p, _i, _i, _i, _i, _i, C.c_longlong, _i, C.c_longlong, _i, _p],
-    "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _i, _p],
+    "xr_moe_experts": [_p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _p, _i, _p, _p, _p, _i, _i, _p],
     "xr_delta_prepare": [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _p],
     "xr_linear_recurrence": [_p, _p, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p, _p, _i, _f, _f, _p],
     "xr_qkv_store": [_p, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p],
@@ -1324,11 +1324,12 @@ class Ops:
                                                    int(n_experts), 1.0 / top, _stream()))
         return idx, wts
 
+    SHARED_INLINE_ROWS = 2          # rows up to which a shared expert runs in the chosen experts' own launches
     GROUPED_EXPERTS_FROM = 32       # choices (rows x top) from which the experts' rows are sorted and run on the matrix cores
 
     def moe_experts(self, h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor,
                     out: Optional[torch.Tensor] = None, accumulate: bool = False, activation: str = "relu2", param: float = 0.0,
-                    beside=None, norm=None, identity: int = 0, post_alpha: Optional[float] = None):
+                    beside=None, norm=None, identity: int = 0, post_alpha: Optional[float] = None, shared=None):
         """``out[t] (+)= sum_j wts[t, j] * w_down[e] @ relu(w_up[e] @ h[t])^2`` with ``e = idx[t, j]``, as 32-bit
         rows; ``w_up [n, F, E]`` and ``w_down [n, E, F]`` in ``h``'s dtype.  ``activation`` "swiglu": gated experts,
         ``w_down[e] @ (silu(g) * u)`` with ``[g; u] = w_up[e] @ h[t]`` for ``w_up [n, 2F, E]`` (an expert's gate rows
@@ -1337,7 +1338,8 @@ class Ops:
         ``norm`` = (weight, eps, centred), the norm of the updated rows (an RMS norm, or with ``centred`` the layer norm with a
         32-bit weight): its result in ``h``'s dtype comes back instead of the rows.  With ``post_alpha`` the rows ``out``
         become ``norm(post_alpha * out + the sum)`` themselves (an RMS norm with a 32-bit weight).  ``identity``: choices
-        ``n .. n + identity - 1`` stand for experts whose output is ``h[t]`` itself.  A few choices stream the chosen
+        ``n .. n + identity - 1`` stand for experts whose output is ``h[t]`` itself.  ``shared`` = (up, down), for one or two
+        rows (``SHARED_INLINE_ROWS``): a shared expert ``down relu(up h)^2`` added to the sum in the same two launches.  A few choices stream the chosen
         experts' weights, a wave an output column; from ``GROUPED_EXPERTS_FROM`` choices on (bfloat16, widths
         that are multiples of 8) the rows are sorted by expert on the device, both products run on the matrix
         cores and a last kernel adds a token's experts up in the order of its choice (and writes the norm)."""
@@ -1347,6 +1349,8 @@ class Ops:
             raise KernelError(f"moe_experts: activation {activation!r} (known: {sorted(EXPERT_ACTIVATIONS)})")
         form, gate = EXPERT_ACTIVATIONS[activation]
         gated = form == 1
+        if shared is not None and (T > self.SHARED_INLINE_ROWS or T * idx.shape[1] >= self.GROUPED_EXPERTS_FROM):
+            raise KernelError(f"moe_experts: a shared expert runs beside the chosen ones for up to {self.SHARED_INLINE_ROWS} rows, not {T}")
         y_beside, g_beside = beside if beside is not None else (None, None)
         if beside is not None:
             self._dev(y_beside, g_beside)
@@ -1395,10 +1399,21 @@ class Ops:
                 return normed
             return self.post_norm(out, target, post_alpha, norm[0], norm[1], h.dtype) if post else self._then_norm(out, norm, h.dtype)
         target = torch.empty((T, E), dtype=torch.float32, device=h.device) if post else out
+        sh = (None, None, None, 0, 0)
+        if shared is not None:
+            packed = isinstance(shared[0], PackedWeight)
+            s_up, s_down = (w.data if isinstance(w, PackedWeight) else w for w in shared)
+            Fs = shared[0].shape[0]
+            self._dev(s_up, s_down)
+            if (tuple(shared[0].shape) != (Fs, E) or tuple(shared[1].shape) != (E, Fs) or s_up.dtype != h.dtype or s_down.dtype != h.dtype
+                    or packed != isinstance(shared[1], PackedWeight) or not s_up.is_contiguous() or not s_down.is_contiguous()):
+                raise KernelError("moe_experts: the shared expert's weights must be [F, E] and [E, F], both packed or neither")
+            s_z = torch.empty((T, Fs), dtype=h.dtype, device=h.device)
+            sh = (s_up.data_ptr(), s_down.data_ptr(), s_z.data_ptr(), Fs, 1 if packed else 0)
         self.lib.check(self.lib.xr_moe_experts(target.data_ptr(), z.data_ptr(), h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(),
                                                idx.data_ptr(), wts.data_ptr(), T, E, F, h.stride(0), target.stride(0), n, top,
                                                1 if accumulate else 0, dtype_code(h.dtype), form, gate, float(param),
-                                               _ptr(y_beside), _ptr(g_beside), int(identity), _stream()))
+                                               _ptr(y_beside), _ptr(g_beside), int(identity), *sh, _stream()))
         if post:
             return self.post_norm(out, target, post_alpha, norm[0], norm[1], h.dtype)
         return self._then_norm(out, norm, h.dtype)

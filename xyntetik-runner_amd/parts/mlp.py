@@ -257,6 +257,12 @@ class RoutedExperts(FeedForward):
         if self.shared is not None:
             self.shared.bind({name: tensors[name] for name in self.shared.param_specs()}, rt)
 
+    def _shared_inline(self, h) -> bool:
+        """Whether the shared expert runs in the chosen experts' launches (a row or two, relu squared, both matrices alike)."""
+        ops, sh = self.rt.ops, self.shared
+        return (isinstance(sh, DenseMLP) and sh.activation == "relu2" and h.shape[0] <= ops.SHARED_INLINE_ROWS
+                and h.shape[0] * self.top < ops.GROUPED_EXPERTS_FROM and type(sh.w_up) is type(sh.w_down))
+
     def _run(self, ctx, h, out=None, accumulate=False, norm=None, post_alpha=None):
         ops = self.rt.ops
         beside = None
@@ -267,11 +273,15 @@ class RoutedExperts(FeedForward):
         else:       # the shared expert's rows enter the sum of the chosen ones with the token's gate
             idx, wts, gate = ops.moe_route(h, self.router, self.correction, self.top, side_gate=True, **self.how)
             beside = (self.shared.forward_f32(ctx, h), gate)
+        shared = None
         if post_alpha is not None and self.shared is not None and beside is None:      # all of it before the norm
-            beside = (self.shared.forward_f32(ctx, h), None)
+            if self._shared_inline(h):
+                shared = (self.shared.w_up, self.shared.w_down)
+            else:
+                beside = (self.shared.forward_f32(ctx, h), None)
         out = ops.moe_experts(h, self.w_up, self.w_down, idx, wts, out=out, accumulate=accumulate, activation=self.activation,
-                              param=self.activation_param, beside=beside, norm=norm, identity=self.identity, post_alpha=post_alpha)
-        if self.shared is not None and beside is None:
+                              param=self.activation_param, beside=beside, norm=norm, identity=self.identity, post_alpha=post_alpha, shared=shared)
+        if self.shared is not None and beside is None and shared is None:
             self.shared.forward_add(ctx, h, out)
         return out
 
