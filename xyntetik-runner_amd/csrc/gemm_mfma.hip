@@ -206,7 +206,8 @@ __device__ inline void rope_store(const RopeFuse& rp, int tok, int nn, float val
 // wave's own LDS area, so that a lane then holds 4 consecutive columns of one row: a store
 // instruction writes whole 128-byte runs instead of 2 or 4 bytes a lane.  (Measured on a
 // 256x256 tile with bfloat16 output: 21 us of a tile's 137 us went to 128 two-byte stores a
-// lane and their addresses.)  mode: 0 store float, 1 add into float, 2 store bfloat16.
+// lane and their addresses.)  mode: 0 store float, 1 add into float, 2 store bfloat16;
+// 4 more: the square of what is positive.
 // A wave's LDS accesses are served in order, so it needs no barrier for an area of its own.
 constexpr int STAGE_FLOATS = 32 * (64 + 4);      // a wave's area: 32 rows of 64 columns, rows 16 bytes apart in the banks
 // What write_tiles will add to (mode 1), fetched ahead: a lane's 4 floats of each of its 4 NT rows.
@@ -244,10 +245,14 @@ __device__ inline void write_tiles(float* stage, const f32x16 (&t)[NT], void* ds
 #pragma unroll
     for (int it = 0; it < 32 / RPI; ++it) {
         const int row = it * RPI + lane / CPR, m = m_base + row;
-        const float4 x = *reinterpret_cast<const float4*>(stage + row * LD + ch * 4);
+        float4 x = *reinterpret_cast<const float4*>(stage + row * LD + ch * 4);
         if (m >= M || col >= col_end) continue;
         const uint32_t o = lane_off + (uint32_t)(it * RPI * ld);
-        if (mode == 2) {
+        if (mode & 4) {
+            x = make_float4(fmaxf(x.x, 0.f), fmaxf(x.y, 0.f), fmaxf(x.z, 0.f), fmaxf(x.w, 0.f));
+            x = make_float4(x.x * x.x, x.y * x.y, x.z * x.z, x.w * x.w);
+        }
+        if (mode & 2) {
             uint2 v;
             v.x = pack_bf16x2(x.x, x.y);
             v.y = pack_bf16x2(x.z, x.w);
@@ -255,7 +260,7 @@ __device__ inline void write_tiles(float* stage, const f32x16 (&t)[NT], void* ds
         } else {
             float4* q = reinterpret_cast<float4*>(dst32 + o);
             float4 y = x;
-            if (mode == 1) { const float4 o4 = old ? old[it] : *q; y.x += o4.x; y.y += o4.y; y.z += o4.z; y.w += o4.w; }
+            if (mode & 1) { const float4 o4 = old ? old[it] : *q; y.x += o4.x; y.y += o4.y; y.z += o4.z; y.w += o4.w; }
             *q = y;
         }
     }
@@ -890,32 +895,26 @@ __device__ __forceinline__ void gemm_tile(const GemmArgs& g, const int item, uin
                 const float b = g.bias && col < g.N ? g.bias[col] : 0.f;
 #pragma unroll
                 for (int e = 0; e < 16; ++e) t[n][e] = acc[i][j + n][e] + b;
-                if (g.epi == EPI_STORE && g.act == XR_POST_RELU2) {
-#pragma unroll
-                    for (int e = 0; e < 16; ++e) { const float v = fmaxf(t[n][e], 0.f); t[n][e] = v * v; }
-                }
             }
             if (rotate)
                 rope_tiles<NTP>(stage, t, g.rope, m0 + wm0 + i * 32, g.M, bx * BN + wn0 + j * 32, g.N, lane);
             else
-                write_tiles<NTP>(stage, t, g.out, g.ldo, g.epi == EPI_ACCUM ? 1 : (g.out_bf16 ? 2 : 0),
+                write_tiles<NTP>(stage, t, g.out, g.ldo, g.epi == EPI_ACCUM ? 1 : (g.out_bf16 ? 2 : 0) + (g.act == XR_POST_RELU2 && g.epi == EPI_STORE ? 4 : 0),
                                  m0 + wm0 + i * 32, g.M, bx * BN + wn0 + j * 32, g.N, lane, adding ? old[decltype(idx)::value & 1] : nullptr);
         });
         return;
     }
+    static_for<0, TM * TN>([&](auto idx) {      // (for the same reason)
+        constexpr int i = decltype(idx)::value / TN, j = decltype(idx)::value % TN;
+        const int n = bx * BN + wn0 + j * 32 + lr;
+        if (n >= g.N) return;
+        const float b = g.bias ? g.bias[n] : 0.f;
 #pragma unroll
-    for (int i = 0; i < TM; ++i)
-#pragma unroll
-        for (int j = 0; j < TN; ++j) {
-            int n = bx * BN + wn0 + j * 32 + lr;
-            if (n >= g.N) continue;
-            float b = g.bias ? g.bias[n] : 0.f;
-#pragma unroll
-            for (int e = 0; e < 16; ++e) {
-                int m = m0 + wm0 + i * 32 + (e / 4) * 8 + lg * 4 + (e % 4);
-                if (m < g.M) store_out(g, m, n, acc[i][j][e] + b);
-            }
+        for (int e = 0; e < 16; ++e) {
+            const int m = m0 + wm0 + i * 32 + (e / 4) * 8 + lg * 4 + (e % 4);
+            if (m < g.M) store_out(g, m, n, acc[i][j][e] + b);
         }
+    });
     }
 }
 
