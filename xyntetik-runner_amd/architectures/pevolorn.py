@@ -1,7 +1,7 @@
 """``Pevolorn``: a decoder whose residual stream is normed behind every sum, put together from parts.
 
-Every layer: ``x <- norm1(alpha x + mixer(x)); x <- norm2(alpha x + feed_forward(x))``, the feed-forward optional; the
-sublayers read x itself.  The norms are RMS norms whose weights are stored around zero.  Mixers by ``type``:
+Every layer: ``x <- norm1(alpha x + mixer(x)); x <- norm2(alpha x + feed_forward(x))``, the feed-forward optional; mixer and
+feed-forward take the stream as it is, with no norm in front.  Norm weights are stored around zero (RMS norms).  Mixers by ``type``:
 
 * "latent_attention": keys and values from one cached latent a token, with queries straight from the input, one rotated key
   part that the heads share (rotate-half layout) and a sigmoid gate a head; a layer with ``kv_from`` has no latent of its
